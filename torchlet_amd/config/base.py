@@ -114,6 +114,10 @@ class PairRotarySpec(PartSpec):
     dims: int = 0
     base: float = 10000.0
     factor: float = 1.0        # linear scaling: every frequency is divided by it
+    # ``yarn = (factor, original, fast, slow)``: frequencies are blended between themselves and themselves over ``factor``, pair by pair: pairs
+    # that turn more than ``fast`` times over ``original`` positions stay, pairs that turn less than ``slow`` times are divided, linearly in the
+    # pair's index between; cosines and sines are multiplied by ``0.1 ln(factor) + 1``
+    yarn: tuple | None = None
 
 
 @dataclass(frozen=True)
@@ -128,6 +132,7 @@ class HalfRotarySpec(PartSpec):
     # than ``original / high`` a frequency stays, longer than ``original / low`` it is divided by ``factor``, and between the two it is
     # ``(1 - s) f / factor + s f`` with ``s = (original / wavelength - low) / (high - low)``
     bands: tuple | None = None
+    yarn: tuple | None = None      # as in :class:`PairRotarySpec`
 
 
 @dataclass(frozen=True)
@@ -204,6 +209,13 @@ class CappedAttentionSpec(PartSpec):
     values_are_keys: bool = False
     qk_bias: bool = False
     o_bias: bool = False
+    # ``fixed_sink``: the softmax's denominator also holds ``exp`` of this fixed number, the same for all heads (0: one is added).
+    # ``value_norm``: every head's value is divided by its root mean square (``qk_norm_eps``, no weight) before it is cached.
+    # ``value_position``: an encoding over the first dimensions of a value: a cached value is turned by its own position, and a head's output
+    # (the sum over the values) at position ``i`` is turned back by ``i``.
+    fixed_sink: float | None = None
+    value_norm: bool = False
+    value_position: PartSpec | None = None
 
 
 @dataclass(frozen=True)
@@ -255,6 +267,33 @@ class SelectiveStateSpec(PartSpec):
     conv: int = 4
     norm_groups: int = 1
     norm_eps: float = 1e-6
+
+
+@dataclass(frozen=True)
+class WKVSpec(PartSpec):
+    """Time mixing with a matrix state whose decays depend on the token (RWKV): r, k, v, the gate and the decay each read a mix of the token's
+    input and the one's before it, ``h + (h' - h) * mu``; per head and key channel ``w = exp(-exp(w0 + W_w2 tanh(W_w1 mix)))``; per head ``o = (S +
+    diag(u) k v^T)^T r``, then ``S <- diag(w) S + k v^T``; each head's output is divided by its root mean square (``norm_eps``), multiplied by a
+    weight and by ``silu`` of the gate.  ``decay_rank``: the inner size of the decay's two matrices in the random-weights mode (a checkpoint's
+    tensors say their own)."""
+    kind: ClassVar[str] = "wkv"
+    hidden: int = 0
+    heads: int = 0
+    dim: int = 0
+    vdim: int = 0
+    decay_rank: int = 32
+    norm_eps: float = 1e-6
+
+
+@dataclass(frozen=True)
+class TokenSideSpec(PartSpec):
+    """A per-layer token input: with ``e`` the layer's slice (``dim`` numbers) of the token's row in a second table, ``y = proj(act(gate(x)) * e)``
+    enters the stream as ``x + y / sqrt(mean(y^2) + eps) * w``."""
+    kind: ClassVar[str] = "token_side"
+    hidden: int = 0
+    dim: int = 0
+    eps: float = 1e-6
+    activation: str = "gelu_tanh"
 
 
 @dataclass(frozen=True)
@@ -343,6 +382,15 @@ class SandwichBlockSpec(BlockSpec):
 
 
 @dataclass(frozen=True)
+class OutputNormBlockSpec(BlockSpec):
+    """One layer with norms on the sublayers' outputs only: ``x <- x + mixer_norm(mixer(x))``, then ``x <- x + ffn_norm(ffn(x))``; the sublayers
+    read ``x`` itself.  ``ffn`` (and then ``ffn_norm``) may be ``None``.  ``side``: a per-layer token input after them (``None``: none)."""
+    kind: ClassVar[str] = "output_norm_residual"
+    side: PartSpec | None = None
+    side_name: str = "side"
+
+
+@dataclass(frozen=True)
 class HyperBlockSpec(BlockSpec):
     """One layer over ``streams`` copies of the residual joined by hyper-connections.  Sublayer ``q`` (1: the mixer, 2: the
     feed-forward) has a read vector ``in [streams]``, a matrix ``mix [streams, streams]`` (indexed from, to) and a write vector
@@ -377,6 +425,13 @@ class HashedBigramSpec:
 
 
 @dataclass(frozen=True)
+class TokenSideTable:
+    """A second token table ``[vocab, layers * dim]`` under ``name``; layer ``i`` gets the columns ``[i * dim, (i + 1) * dim)``."""
+    name: str = "side.embed"
+    dim: int = 0
+
+
+@dataclass(frozen=True)
 class ModelSpec:
     """Everything needed to build a decoder: parts, their names, and the run order."""
     vocab_size: int
@@ -400,6 +455,7 @@ class ModelSpec:
     bigram: HashedBigramSpec | None = None   # a hashed bigram row added to every token's (scaled) embedding
     embed_norm: PartSpec | None = None       # a norm that the embedding's output passes before it becomes the stream
     embed_norm_name: str = "embed.norm"
+    token_side: TokenSideTable | None = None     # the table of the layers' per-layer token inputs
 
     def layer_name(self, i: int) -> str:
         return self.layers_format.format(i) if self.layers_format else f"{self.layers_prefix}.{i}"

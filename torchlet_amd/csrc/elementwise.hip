@@ -743,7 +743,7 @@ extern "C" int tl_bigram_embedding(const void* ids, const void* table, void* out
 // One block per output row, the row kept in shared memory between the passes:
 //   y = pending[row] (one tensor of the activation type, or `parts` float slabs added up);
 //   r = residual[row] (+ extra[row]) + y * (post ? rsqrt(mean(y^2) + post_eps) * post[i] : 1);   written back unless `rows` selects
-//   out = r * rsqrt(mean(r^2) + eps) * weight[i] * gain.
+//   out = r * rsqrt(mean(r^2) + eps) * weight[i] * gain, or, without a `weight`, r * gain (the sum itself, in the activation type).
 // `post` and `weight` are float vectors of post_n / weight_n numbers: `hidden` of them, or one for all coordinates.
 template <typename T>
 __global__ void sandwich_norm_kernel(float* __restrict__ residual, const void* __restrict__ pending, int parts, size_t part_stride,
@@ -781,8 +781,12 @@ __global__ void sandwich_norm_kernel(float* __restrict__ residual, const void* _
         sn_row[i] = r;
         ss = fmaf(r, r, ss);
     }
-    const float inv = rsqrtf(block_sum(ss, red) / (float)hidden + eps) * gain;
     T* dst = out + (size_t)orow * hidden;
+    if (!weight) {
+        for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = from_float<T>(sn_row[i] * gain);
+        return;
+    }
+    const float inv = rsqrtf(block_sum(ss, red) / (float)hidden + eps) * gain;
     for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = from_float<T>(sn_row[i] * inv * weight[weight_n == 1 ? 0 : i]);
 }
 
@@ -790,7 +794,7 @@ extern "C" int tl_sandwich_norm(void* residual, const void* pending, int parts, 
                                 const void* extra, const void* weight, int weight_n, float eps, float gain, void* out, const void* rows,
                                 int out_rows, int hidden, int act_dtype, hipStream_t stream) {
     TL_REQUIRE(parts >= 0 && parts <= 64 && out_rows >= 0 && hidden > 0 && hidden <= 12288, "sandwich_norm: bad sizes rows=%d hidden=%d parts=%d", out_rows, hidden, parts);
-    TL_REQUIRE(weight && (weight_n == 1 || weight_n == hidden) && (!post || post_n == 1 || post_n == hidden), "sandwich_norm: weights of one number or of %d", hidden);
+    TL_REQUIRE((!weight || weight_n == 1 || weight_n == hidden) && (!post || post_n == 1 || post_n == hidden), "sandwich_norm: weights of one number or of %d", hidden);
     if (out_rows == 0) return TL_OK;
     const size_t part_stride = (size_t)part_rows * hidden, smem = sizeof(float) * hidden;
     const int threads = hidden >= 2048 ? 512 : 256;
@@ -872,5 +876,145 @@ extern "C" int tl_embedding_norm(const void* ids, const void* table, int table_d
         embedding_norm_kernel<bf16_t><<<tokens, 256, smem, stream>>>((const int*)ids, (const bf16_t*)table, (float*)out, hidden, vocab, scale, (const float*)weight, eps);
     else TL_REQUIRE(false, "embedding_norm: unknown dtype %d", table_dtype);
     TL_CHECK_LAUNCH("embedding_norm");
+    return TL_OK;
+}
+
+// ------------------------------------------------------------------ the sum, and mixes of neighbouring tokens
+// x_t = residual[t] + y_t * (post ? rsqrt(mean(y_t^2) + post_eps) * post[i] : 1), y_t the pending output (the activation type, or `parts`
+// float slabs added up; null: x_t = residual[t]), written to `settled` (another place than the residual: a work-group also reads the row
+// before its own first one).  Then, with x' the token before's (of the request's slot, `tail`, for the first token that a request brings),
+//   mixes[s][t][i] = x_t[i] + (x'[i] - x_t[i]) * mu[s][i],   s < count.
+// A work-group takes `run` neighbouring tokens, row after row, and makes the row before the first of them a second time; a row's numbers
+// stay with the threads that made them, so the rows in shared memory need no barrier of their own.  All in float, one rounding of the mixes.
+__device__ __forceinline__ float4 load4(const float* p) { return *(const float4*)p; }
+__device__ __forceinline__ float4 load4(const bf16_t* p) {
+    const uint2 t = *(const uint2*)p;
+    return make_float4(__uint_as_float(t.x << 16), __uint_as_float(t.x & 0xffff0000u), __uint_as_float(t.y << 16), __uint_as_float(t.y & 0xffff0000u));
+}
+__device__ __forceinline__ void store4(float* p, float4 v) { *(float4*)p = v; }
+__device__ __forceinline__ void store4(bf16_t* p, float4 v) {
+    uint2 t;
+    t.x = (uint32_t)from_float<bf16_t>(v.x).bits | ((uint32_t)from_float<bf16_t>(v.y).bits << 16);
+    t.y = (uint32_t)from_float<bf16_t>(v.z).bits | ((uint32_t)from_float<bf16_t>(v.w).bits << 16);
+    *(uint2*)p = t;
+}
+// Up to four neighbouring numbers: all four at once where rows are multiples of four (VEC 4), one otherwise.
+template <int VEC, typename T> __device__ __forceinline__ void load_piece(const T* p, float (&v)[VEC]) {
+    if constexpr (VEC == 4) { const float4 f = load4(p); v[0] = f.x; v[1] = f.y; v[2] = f.z; v[3] = f.w; }
+    else v[0] = to_float(p[0]);
+}
+template <int VEC, typename T> __device__ __forceinline__ void store_piece(T* p, const float (&v)[VEC]) {
+    if constexpr (VEC == 4) store4(p, make_float4(v[0], v[1], v[2], v[3]));
+    else p[0] = from_float<T>(v[0]);
+}
+
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256)
+settle_shift_kernel(const float* __restrict__ residual, float* __restrict__ settled, const void* __restrict__ pending, int parts, size_t part_stride,
+                    const float* __restrict__ post, int post_n, float post_eps, const float* __restrict__ state, size_t slot_stride, size_t tail_off,
+                    const int* __restrict__ slots, const int* __restrict__ req_indptr, const int* __restrict__ token_req,
+                    const float* __restrict__ mu, T* __restrict__ mixes, int count, int tokens, int hidden, int run) {
+    extern __shared__ __attribute__((aligned(16))) float ss_rows[];       // two rows
+    __shared__ float red[16];
+    const int first = blockIdx.x * run, last = min(first + run, tokens) - 1;
+    const int step = blockDim.x * VEC;
+    // the settled row t into `buf` (each thread its own pieces)
+    auto settle = [&](int t, float* buf) {
+        const float* res = residual + (size_t)t * hidden;
+        float inv = 1.f;
+        if (pending) {
+            float ss = 0.f;
+            for (int i = threadIdx.x * VEC; i < hidden; i += step) {
+                float y[VEC];
+                if (parts == 0) load_piece<VEC>((const T*)pending + (size_t)t * hidden + i, y);
+                else {
+                    load_piece<VEC>((const float*)pending + (size_t)t * hidden + i, y);
+                    for (int p = 1; p < parts; ++p) {
+                        float z[VEC];
+                        load_piece<VEC>((const float*)pending + p * part_stride + (size_t)t * hidden + i, z);
+#pragma unroll
+                        for (int v = 0; v < VEC; ++v) y[v] += z[v];
+                    }
+                }
+#pragma unroll
+                for (int v = 0; v < VEC; ++v) ss = fmaf(y[v], y[v], ss);
+                store_piece<VEC>(buf + i, y);
+            }
+            if (post) inv = rsqrtf(block_sum(ss, red) / (float)hidden + post_eps);
+        }
+        for (int i = threadIdx.x * VEC; i < hidden; i += step) {
+            float r[VEC];
+            load_piece<VEC>(res + i, r);
+            if (pending) {
+                float y[VEC], w[VEC];
+                load_piece<VEC>(buf + i, y);
+                if (post) {
+                    if (post_n == 1) {
+#pragma unroll
+                        for (int v = 0; v < VEC; ++v) w[v] = post[0];
+                    } else load_piece<VEC>(post + i, w);
+                }
+#pragma unroll
+                for (int v = 0; v < VEC; ++v) r[v] += post ? y[v] * inv * w[v] : y[v];
+            }
+            store_piece<VEC>(buf + i, r);
+        }
+    };
+    float *cur = ss_rows, *before = ss_rows + hidden;
+    if (first > req_indptr[token_req[first]]) settle(first - 1, before);
+    for (int t = first; t <= last; ++t) {
+        const int req = token_req[t];
+        const float* tail = t == req_indptr[req] ? state + (size_t)slots[req] * slot_stride + tail_off : nullptr;
+        settle(t, cur);
+        for (int i = threadIdx.x * VEC; i < hidden; i += step) {
+            float x[VEC], b[VEC];
+            load_piece<VEC>(cur + i, x);
+            if (tail) {
+#pragma unroll
+                for (int v = 0; v < VEC; ++v) b[v] = tail[i + v];          // (a slot's tail may start anywhere)
+            } else load_piece<VEC>(before + i, b);
+            if (pending) store_piece<VEC>(settled + (size_t)t * hidden + i, x);
+            for (int s = 0; s < count; ++s) {
+                float m[VEC];
+                load_piece<VEC>(mu + (size_t)s * hidden + i, m);
+#pragma unroll
+                for (int v = 0; v < VEC; ++v) m[v] = fmaf(b[v] - x[v], m[v], x[v]);
+                store_piece<VEC>(mixes + ((size_t)s * tokens + t) * hidden + i, m);
+            }
+        }
+        float* other = cur; cur = before; before = other;
+    }
+}
+
+extern "C" int tl_settle_shift(const void* residual, void* settled, const void* pending, int parts, const void* post, int post_n, float post_eps,
+                               const void* state, long slot_stride, long tail_off, const void* slots, const void* req_indptr, const void* token_req,
+                               const void* mu, void* mixes, int count, int tokens, int hidden, int act_dtype, hipStream_t stream) {
+    TL_REQUIRE(parts >= 0 && parts <= 64 && tokens >= 0 && hidden > 0 && hidden <= 12288 && count > 0, "settle_shift: bad sizes tokens=%d hidden=%d", tokens, hidden);
+    TL_REQUIRE(!post || post_n == 1 || post_n == hidden, "settle_shift: a norm weight of one number or of %d", hidden);
+    TL_REQUIRE(!pending || settled != residual, "settle_shift: the sum goes to another place than the residual it is made from");
+    TL_REQUIRE(tail_off >= 0 && slot_stride >= tail_off + hidden, "settle_shift: the slots do not hold a row of %d numbers", hidden);
+    TL_REQUIRE(act_dtype == TL_DT_F32 || act_dtype == TL_DT_BF16, "settle_shift: unknown dtype %d", act_dtype);
+    if (tokens == 0) return TL_OK;
+    const int run = tokens >= 2048 ? 4 : (tokens >= 768 ? 2 : 1);
+    const size_t smem = sizeof(float) * 2 * hidden, part_stride = (size_t)tokens * hidden;
+    const bool vec = hidden % 4 == 0;
+    const int grid = (tokens + run - 1) / run;
+#define TL_SS(T, V)                                                                                                                              \
+    {                                                                                                                                            \
+        auto kernel = settle_shift_kernel<T, V>;                                                                                                 \
+        static bool raised = false;                                                                                                              \
+        if (smem > 48 * 1024 && !raised) {                                                                                                       \
+            hipError_t e = hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 96 * 1024 + 64);                 \
+            if (e != hipSuccess) { tl_set_error("settle_shift: cannot get %zu bytes of shared memory: %s", smem, hipGetErrorString(e)); return TL_ERR_HIP; } \
+            raised = true;                                                                                                                       \
+        }                                                                                                                                        \
+        kernel<<<grid, 256, smem, stream>>>((const float*)residual, (float*)settled, pending, parts, part_stride, (const float*)post, post_n, post_eps, \
+            (const float*)state, (size_t)slot_stride, (size_t)tail_off, (const int*)slots, (const int*)req_indptr, (const int*)token_req,        \
+            (const float*)mu, (T*)mixes, count, tokens, hidden, run);                                                                            \
+    }
+    if (act_dtype == TL_DT_F32) { if (vec) TL_SS(float, 4) else TL_SS(float, 1) }
+    else { if (vec) TL_SS(bf16_t, 4) else TL_SS(bf16_t, 1) }
+#undef TL_SS
+    TL_CHECK_LAUNCH("settle_shift");
     return TL_OK;
 }

@@ -372,3 +372,31 @@ extern "C" int tl_activation(void* x, long n, int act, int dtype, hipStream_t st
     TL_CHECK_LAUNCH("activation");
     return TL_OK;
 }
+
+// ------------------------------------------------------------------ a gate against a token's own row
+// out[t, n] = act(z[t, n]) * table[ids[t], n]: z float [tokens, dim] (a projection of the stream), `table` a slice of a token table (rows
+// table_ld numbers apart).
+template <typename T>
+__global__ void token_gate_kernel(const float* __restrict__ z, const int* __restrict__ ids, const T* __restrict__ table, int table_ld, int vocab,
+                                  T* __restrict__ out, int dim, int total, int act) {
+    const int i = blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= total) return;
+    const int t = i / dim, n = i % dim, id = ids[t];
+    if (id < 0 || id >= vocab) return;
+    out[i] = from_float<T>(activate(z[i], act) * to_float(table[(size_t)id * table_ld + n]));
+}
+
+extern "C" int tl_token_gate(const void* z, const void* ids, const void* table, int table_ld, int vocab, void* out, int tokens, int dim, int act,
+                             int dtype, hipStream_t stream) {
+    TL_REQUIRE(tokens >= 0 && dim > 0 && table_ld >= dim && vocab > 0 && (long)tokens * dim < (1L << 31), "token_gate: bad sizes");
+    TL_REQUIRE(known_activation(act) && !(act & ACT_PAIRS), "token_gate: unknown activation %d", act);
+    if (tokens == 0) return TL_OK;
+    const int total = tokens * dim, grid = (total + 255) / 256;
+    if (dtype == TL_DT_F32)
+        token_gate_kernel<float><<<grid, 256, 0, stream>>>((const float*)z, (const int*)ids, (const float*)table, table_ld, vocab, (float*)out, dim, total, act);
+    else if (dtype == TL_DT_BF16)
+        token_gate_kernel<bf16_t><<<grid, 256, 0, stream>>>((const float*)z, (const int*)ids, (const bf16_t*)table, table_ld, vocab, (bf16_t*)out, dim, total, act);
+    else TL_REQUIRE(false, "token_gate: unknown dtype %d", dtype);
+    TL_CHECK_LAUNCH("token_gate");
+    return TL_OK;
+}

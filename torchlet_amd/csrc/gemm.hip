@@ -466,6 +466,16 @@ extern "C" int tl_gemm_f32_variant(const void* x, const void* w, const void* bia
 typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
 typedef float f32x4_t __attribute__((ext_vector_type(4)));
 
+// Several products of equal shape in one launch (the mixes of a token and the one before it, each against its own matrix): product
+// blockIdx.z reads x and w and writes out these many elements further on.
+struct GroupStride {
+    long x, w, out;
+};
+struct Groups {
+    int count = 1;
+    GroupStride stride{0, 0, 0};
+};
+
 #define SK_KOFF(lg) (16 * (lg))     // a lane reads 32 contiguous bytes per step (other splits measured the same)
 #define SK_SECOND 8
 #define SK_LOAD(p) (*(const uint4*)(p))
@@ -579,7 +589,7 @@ __global__ __launch_bounds__(KS * 64) void gemm_skinny_kernel(const bf16_t* __re
                                                               const void* __restrict__ bias, int bias_f32,
                                                               TOut* __restrict__ out, int M, int N, int K, int ldx, int ldo,
                                                               int out_cols, int k_per_split, int rows_per_strip, int rows_per_group,
-                                                              RopeArgs ra, NormArgs na) {
+                                                              RopeArgs ra, NormArgs na, GroupStride gs) {
     static_assert(!NF || (XL && MT == 1), "the fused norm makes x in shared memory, for one row");
     static_assert(!SW || (R == 1 && KS % 2 == 0), "the fused gate deals a work-group's waves to a gate strip and its up strip");
     static_assert(!RP || (R <= 2 && MT == 1 && !SW), "the fused rotation is built for up to 16 rows of x");
@@ -587,6 +597,9 @@ __global__ __launch_bounds__(KS * 64) void gemm_skinny_kernel(const bf16_t* __re
     // [y * k_per_split, ...) of x and w and writes its own [M, ldo] slab of partial sums to out
     // (float, no bias); whoever reads them adds the slabs up.
     const int ldw = K;
+    x += blockIdx.z * gs.x;
+    w += blockIdx.z * gs.w;
+    out += blockIdx.z * gs.out;
     if (k_per_split > 0) {
         const int kb = blockIdx.y * k_per_split;
         x += kb;
@@ -942,10 +955,10 @@ static StripPlan plan_strips(int total, int most, int cap, bool even) {
 // rows_per_strip > 0: one strip of that many outputs per work-group, whatever else holds.
 template <int R, int MT, int KS, typename TOut, int SW, int D>
 static void launch_skinny_d(const void* x, const void* w, const void* bias, int bias_f32, void* out, int M, int N, int K,
-                            int ldx, int ldo, int out_cols, hipStream_t stream, int rows_per_strip = 0) {
+                            int ldx, int ldo, int out_cols, hipStream_t stream, int rows_per_strip = 0, Groups gr = Groups{}) {
     const int total = SW ? out_cols : N;
     const int rps = rows_per_strip > 0 ? rows_per_strip : 16 * R;
-    dim3 grid((total + rps - 1) / rps), block(KS * 64);
+    dim3 grid((total + rps - 1) / rps, 1, gr.count), block(KS * 64);
     const size_t red_bytes = (size_t)KS * R * MT * 1024;
     const size_t x_bytes = (size_t)M * (K + 8) * 2;
     // More than one row of x: two work-groups per compute unit copy x into shared memory once and walk
@@ -955,16 +968,16 @@ static void launch_skinny_d(const void* x, const void* w, const void* bias, int 
         auto kernel = gemm_skinny_kernel<R, MT, KS, TOut, SW, true, D>;
         static hipError_t allowed = allow_lds(kernel, 156 * 1024);
         if (allowed == hipSuccess) {
-            const int most = x_bytes <= SKINNY_XL_MAX_BYTES ? 2 * TL_COMPUTE_UNITS : TL_COMPUTE_UNITS;      // a larger x leaves room for one work-group only
-            StripPlan p = plan_strips(total, most, 16 * R, false);
+            const int most = (x_bytes <= SKINNY_XL_MAX_BYTES ? 2 * TL_COMPUTE_UNITS : TL_COMPUTE_UNITS) / gr.count;      // a larger x leaves room for one work-group only
+            StripPlan p = plan_strips(total, most > 0 ? most : 1, 16 * R, false);
             if (rows_per_strip > 0) p = StripPlan{(int)grid.x, rps, rps};
-            kernel<<<dim3(p.groups), block, red_bytes + x_bytes, stream>>>((const bf16_t*)x, (const bf16_t*)w, bias, bias_f32, (TOut*)out, M, N, K, ldx, ldo,
-                                                                           out_cols, 0, p.per_strip, p.per_group, RopeArgs{}, NormArgs{});
+            kernel<<<dim3(p.groups, 1, gr.count), block, red_bytes + x_bytes, stream>>>((const bf16_t*)x, (const bf16_t*)w, bias, bias_f32, (TOut*)out, M, N, K, ldx, ldo,
+                                                                           out_cols, 0, p.per_strip, p.per_group, RopeArgs{}, NormArgs{}, gr.stride);
             return;
         }
     }
     gemm_skinny_kernel<R, MT, KS, TOut, SW, false, D><<<grid, block, red_bytes, stream>>>((const bf16_t*)x, (const bf16_t*)w, bias, bias_f32, (TOut*)out, M, N, K, ldx, ldo,
-                                                                                          out_cols, 0, rps, 0, RopeArgs{}, NormArgs{});
+                                                                                          out_cols, 0, rps, 0, RopeArgs{}, NormArgs{}, gr.stride);
 }
 
 // A wave with many K steps ahead of it (a long K: the down projection) keeps as many in flight as
@@ -972,19 +985,19 @@ static void launch_skinny_d(const void* x, const void* w, const void* bias, int 
 // (measured at 3584 x 18944, one row: 33 -> 28 us with eight in flight; at 4608 x 3584: 11 -> 12.6 us).
 template <int R, int MT, int KS, typename TOut, int SW>
 static void launch_skinny_t(const void* x, const void* w, const void* bias, int bias_f32, void* out, int M, int N, int K,
-                            int ldx, int ldo, int out_cols, hipStream_t stream, int rows_per_strip = 0) {
+                            int ldx, int ldo, int out_cols, hipStream_t stream, int rows_per_strip = 0, Groups gr = Groups{}) {
     constexpr int deep = skinny_depth<R, MT, KS>();
     if (deep > 2 && K / 64 / KS >= 16)
-        launch_skinny_d<R, MT, KS, TOut, SW, deep>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, rows_per_strip);
+        launch_skinny_d<R, MT, KS, TOut, SW, deep>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, rows_per_strip, gr);
     else
-        launch_skinny_d<R, MT, KS, TOut, SW, 2>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, rows_per_strip);
+        launch_skinny_d<R, MT, KS, TOut, SW, 2>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, rows_per_strip, gr);
 }
 
 template <int R, int MT, int KS>
 static void launch_skinny(const void* x, const void* w, const void* bias, int bias_f32, void* out, int M, int N, int K,
-                          int ldx, int ldo, int out_f32, hipStream_t stream, int rows_per_strip = 0) {
-    if (out_f32) launch_skinny_t<R, MT, KS, float, false>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, 0, stream, rows_per_strip);
-    else launch_skinny_t<R, MT, KS, bf16_t, false>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, 0, stream, rows_per_strip);
+                          int ldx, int ldo, int out_f32, hipStream_t stream, int rows_per_strip = 0, Groups gr = Groups{}) {
+    if (out_f32) launch_skinny_t<R, MT, KS, float, false>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, 0, stream, rows_per_strip, gr);
+    else launch_skinny_t<R, MT, KS, bf16_t, false>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, 0, stream, rows_per_strip, gr);
 }
 
 // Rows a strip gets so that a matrix of N rows is dealt to the compute units in equal shares, one strip to
@@ -1004,26 +1017,26 @@ static int balanced_rows(int N, int* blocks) {
 
 template <int MT>
 static void pick_skinny(const void* x, const void* w, const void* bias, int bias_f32, void* out, int M, int N, int K,
-                        int ldx, int ldo, int out_f32, hipStream_t stream) {
+                        int ldx, int ldo, int out_f32, hipStream_t stream, Groups gr = Groups{}) {
     // Measured on MI355X at Qwen2.5-7B sizes (weights streamed from HBM, M = 8 and 64):
     // with up to 32 rows one strip of 16 weight rows per work-group is best throughout, with
     // 16 waves along K for wide matrices (gate_up, LM head: 4.7-5.0 TB/s) and 8 for narrow
     // ones (qkv, o, down); with 64 rows the x operand weighs more and several strips per wave
     // share each x load.
-    const int strips = (N + 15) / 16;
-    if (MT == 1) {
+    const int strips = (N + 15) / 16 * gr.count;
+    if (MT == 1 && gr.count == 1) {
         int blocks = 1;
         const int rows = balanced_rows(N, &blocks);
         if (rows > 0 && blocks == 1) return launch_skinny<1, 1, 8>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_f32, stream, rows);
         if (rows > 0) return launch_skinny<2, 1, 8>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_f32, stream, rows);
     }
     if (MT <= 2) {
-        if (strips >= 1024) launch_skinny<1, MT, 16>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_f32, stream);
-        else launch_skinny<1, MT, 8>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_f32, stream);
+        if (strips >= 1024) launch_skinny<1, MT, 16>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_f32, stream, 0, gr);
+        else launch_skinny<1, MT, 8>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_f32, stream, 0, gr);
     } else {
-        if (strips >= 2048) launch_skinny<4, MT, 4>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_f32, stream);
-        else if (strips >= 1024) launch_skinny<2, MT, 2>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_f32, stream);
-        else launch_skinny<1, MT, 8>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_f32, stream);
+        if (strips >= 2048) launch_skinny<4, MT, 4>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_f32, stream, 0, gr);
+        else if (strips >= 1024) launch_skinny<2, MT, 2>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_f32, stream, 0, gr);
+        else launch_skinny<1, MT, 8>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_f32, stream, 0, gr);
     }
 }
 
@@ -1263,7 +1276,7 @@ template <int BM, int BN, int WGM, int WGN, int STAGES, typename TOut, int SW = 
 __global__ __launch_bounds__(64 * WGM * WGN) void gemm_dl_tile_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
                                                                       const void* __restrict__ bias, int bias_f32,
                                                                       TOut* __restrict__ out, int M, int N, int K, int ldx, int ldo,
-                                                                      int out_cols, int k_per_split) {
+                                                                      int out_cols, int k_per_split, GroupStride gs) {
     static_assert(!SW || (BN / WGN) % 64 == 0, "the fused gate needs whole 64-row blocks per wave");
     static_assert(TK == 64 || TK == 32, "slabs of 64 or 32 columns");
     // A slab row holds PPR pieces of 16 bytes; one load instruction of a wave fills RPL rows.  With
@@ -1275,6 +1288,9 @@ __global__ __launch_bounds__(64 * WGM * WGN) void gemm_dl_tile_kernel(const bf16
     // Split K (k_per_split > 0, a multiple of 64): blockIdx.y owns the columns [y * k_per_split, ...) of
     // x and w and writes its own [M, ldo] slab of partial sums to out; whoever reads them adds the slabs up.
     const int ldw = K;
+    x += blockIdx.z * gs.x;
+    w += blockIdx.z * gs.w;
+    out += blockIdx.z * gs.out;
     if (k_per_split > 0) {
         const int kb = blockIdx.y * k_per_split;
         x += kb;
@@ -1589,13 +1605,13 @@ static double dl_estimate(DlTile t, long groups, int k, bool weights_only = fals
     return lag * (double)((groups + 2 * cus - 1) / (2 * cus)) * fmax(products / rate + DL_FIXED[t], groups > cus ? 2 * stream : stream);
 }
 
-static DlTile pick_dl_tile(int M, int N, int K, bool sw, double* estimate = nullptr, bool weights_only = false) {
+static DlTile pick_dl_tile(int M, int N, int K, bool sw, double* estimate = nullptr, bool weights_only = false, int products = 1) {
     DlTile best = DL_128x128;
     double best_t = 1e30;
     for (int t = 0; t < DL_TILES; ++t) {
         if (sw && (t == DL_64x64 || t == DL_256x192 || t == DL_64x320 || t == DL_256x160)) continue;      // a wave of the fused gate needs whole 64-row blocks of weights
         if (t == DL_256x320) continue;      // float slabs of partial sums only: a bfloat16 result tile of 160 KB does not fit its slab buffers
-        const long tiles = (long)((M + DL_BM[t] - 1) / DL_BM[t]) * ((N + DL_BN[t] - 1) / DL_BN[t]);
+        const long tiles = (long)((M + DL_BM[t] - 1) / DL_BM[t]) * ((N + DL_BN[t] - 1) / DL_BN[t]) * products;
         if (t == DL_128x128_S4 && (tiles > TL_COMPUTE_UNITS || M > 128)) continue;      // one round of work-groups, every weight drawn once
         // (the split planner's unsplit baseline is fitted without the 192-wide tiles: with them it kept 512 rows against the
         // 14B's query/key/value matrix whole, 74.8 us, where it used to split K, 53.9 us)
@@ -1638,7 +1654,7 @@ static DlSplit plan_dl_split(int M, int N, int K) {
 // parts > 1 (float results only): K is split into `parts` ranges of k_per columns and out holds that many [M, ldo] slabs.
 template <int BM, int BN, int WGM, int WGN, int STAGES, typename TOut, int SW, int TK = 64>
 static int launch_dl_tile_t(const void* x, const void* w, const void* bias, int bias_f32, void* out, int M, int N, int K,
-                            int ldx, int ldo, int out_cols, hipStream_t stream, int parts = 1, int k_per = 0) {
+                            int ldx, int ldo, int out_cols, hipStream_t stream, int parts = 1, int k_per = 0, Groups gr = Groups{}) {
     constexpr size_t lds = (size_t)STAGES * dl_slab_rows(BM, BN, WGM * WGN, TK) * TK * sizeof(bf16_t);
     // (a lane's offset from its tile's first row is kept in 32 bits)
     TL_REQUIRE((long)(BM > BN ? BM : BN) * (ldx > K ? ldx : K) * 2 < (1L << 31), "gemm_dl_tile: rows of %d elements are too long", ldx > K ? ldx : K);
@@ -1648,40 +1664,40 @@ static int launch_dl_tile_t(const void* x, const void* w, const void* bias, int 
         tl_set_error("gemm_dl_tile: cannot get %zu bytes of shared memory: %s", lds, hipGetErrorString(allowed));
         return TL_ERR_HIP;
     }
-    dim3 grid(((M + BM - 1) / BM) * ((N + BN - 1) / BN), parts), block(64 * WGM * WGN);
+    dim3 grid(((M + BM - 1) / BM) * ((N + BN - 1) / BN), parts, gr.count), block(64 * WGM * WGN);
     kernel<<<grid, block, lds, stream>>>((const bf16_t*)x, (const bf16_t*)w, bias, bias_f32, (TOut*)out, M, N, K, ldx, ldo, out_cols,
-                                         parts > 1 ? k_per : 0);
+                                         parts > 1 ? k_per : 0, gr.stride);
     return TL_OK;
 }
 
 template <typename TOut, int SW>
 static int launch_dl_tile(DlTile tile, const void* x, const void* w, const void* bias, int bias_f32, void* out, int M, int N, int K,
-                          int ldx, int ldo, int out_cols, hipStream_t stream, int parts = 1, int k_per = 0) {
+                          int ldx, int ldo, int out_cols, hipStream_t stream, int parts = 1, int k_per = 0, Groups gr = Groups{}) {
     switch (tile) {
     case DL_64x64:
-        if constexpr (!SW) return launch_dl_tile_t<64, 64, 2, 2, 4, TOut, false>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per);
+        if constexpr (!SW) return launch_dl_tile_t<64, 64, 2, 2, 4, TOut, false>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per, gr);
         else break;
-    case DL_64x256: return launch_dl_tile_t<64, 256, 1, 4, 3, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per);
-    case DL_128x128: return launch_dl_tile_t<128, 128, 2, 2, 2, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per);
-    case DL_128x128_S4: return launch_dl_tile_t<128, 128, 2, 2, 4, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per);
-    case DL_128x256: return launch_dl_tile_t<128, 256, 2, 4, 3, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per);
-    case DL_256x128: return launch_dl_tile_t<256, 128, 4, 2, 3, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per);
-    case DL_64x128: return launch_dl_tile_t<64, 128, 1, 2, 3, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per);
-    case DL_64x192: return launch_dl_tile_t<64, 192, 1, 3, 4, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per);
+    case DL_64x256: return launch_dl_tile_t<64, 256, 1, 4, 3, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per, gr);
+    case DL_128x128: return launch_dl_tile_t<128, 128, 2, 2, 2, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per, gr);
+    case DL_128x128_S4: return launch_dl_tile_t<128, 128, 2, 2, 4, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per, gr);
+    case DL_128x256: return launch_dl_tile_t<128, 256, 2, 4, 3, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per, gr);
+    case DL_256x128: return launch_dl_tile_t<256, 128, 4, 2, 3, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per, gr);
+    case DL_64x128: return launch_dl_tile_t<64, 128, 1, 2, 3, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per, gr);
+    case DL_64x192: return launch_dl_tile_t<64, 192, 1, 3, 4, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per, gr);
     case DL_64x320:
-        if constexpr (!SW) return launch_dl_tile_t<64, 320, 1, 5, 3, TOut, false>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per);
+        if constexpr (!SW) return launch_dl_tile_t<64, 320, 1, 5, 3, TOut, false>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per, gr);
         else break;
-    case DL_128x192: return launch_dl_tile_t<128, 192, 2, 3, 3, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per);
-    case DL_192x256: return launch_dl_tile_t<192, 256, 2, 4, 2, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per);
+    case DL_128x192: return launch_dl_tile_t<128, 192, 2, 3, 3, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per, gr);
+    case DL_192x256: return launch_dl_tile_t<192, 256, 2, 4, 2, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per, gr);
     case DL_256x192:
-        if constexpr (!SW) return launch_dl_tile_t<256, 192, 4, 2, 2, TOut, false>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per);
+        if constexpr (!SW) return launch_dl_tile_t<256, 192, 4, 2, 2, TOut, false>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per, gr);
         else break;
-    case DL_256x256: return launch_dl_tile_t<256, 256, 4, 2, 2, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per);
+    case DL_256x256: return launch_dl_tile_t<256, 256, 4, 2, 2, TOut, SW>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per, gr);
     case DL_256x160:
-        if constexpr (!SW) return launch_dl_tile_t<256, 160, 4, 1, 2, TOut, false>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per);
+        if constexpr (!SW) return launch_dl_tile_t<256, 160, 4, 1, 2, TOut, false>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per, gr);
         else break;
     case DL_256x320:
-        if constexpr (!SW && sizeof(TOut) == 4) return launch_dl_tile_t<256, 320, 4, 2, 2, float, false>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per);
+        if constexpr (!SW && sizeof(TOut) == 4) return launch_dl_tile_t<256, 320, 4, 2, 2, float, false>(x, w, bias, bias_f32, out, M, N, K, ldx, ldo, out_cols, stream, parts, k_per, gr);
         else break;
     default: break;
     }
@@ -1829,7 +1845,7 @@ static void launch_skinny_rope(const void* x, const void* w, const void* bias, i
     const size_t lds = (size_t)KS * R * 1024 + (XL ? (size_t)M * (K + 8) * 2 : 0);
     auto kernel = gemm_skinny_kernel<R, 1, KS, bf16_t, false, XL, 2, true>;
     if (XL) { static hipError_t allowed = allow_lds(kernel, 96 * 1024); (void)allowed; }
-    kernel<<<grid, block, lds, stream>>>((const bf16_t*)x, (const bf16_t*)w, bias, bias_f32, (bf16_t*)out, M, N, K, ldx, ldo, 0, 0, rps, 0, ra, NormArgs{});
+    kernel<<<grid, block, lds, stream>>>((const bf16_t*)x, (const bf16_t*)w, bias, bias_f32, (bf16_t*)out, M, N, K, ldx, ldo, 0, 0, rps, 0, ra, NormArgs{}, GroupStride{});
 }
 
 extern "C" int tl_gemm_partials_pay(int M, int N, int K);
@@ -1907,13 +1923,13 @@ extern "C" int tl_gemm_rope_normed(const void* residual, void* residual_out, con
     const size_t lds = (size_t)ks * blocks * 1024 + (size_t)(K + 8) * 2;
     if (rows > 0 && blocks == 2)
         gemm_skinny_kernel<2, 1, 8, bf16_t, false, true, 2, true, true><<<grid, dim3(8 * 64), lds, stream>>>(
-            nullptr, (const bf16_t*)w, bias, bias_f32, (bf16_t*)out, 1, N, K, K, ldo, 0, 0, rows, 0, ra, na);
+            nullptr, (const bf16_t*)w, bias, bias_f32, (bf16_t*)out, 1, N, K, K, ldo, 0, 0, rows, 0, ra, na, GroupStride{});
     else if (ks == 8)
         gemm_skinny_kernel<1, 1, 8, bf16_t, false, true, 2, true, true><<<grid, dim3(8 * 64), lds, stream>>>(
-            nullptr, (const bf16_t*)w, bias, bias_f32, (bf16_t*)out, 1, N, K, K, ldo, 0, 0, rows, 0, ra, na);
+            nullptr, (const bf16_t*)w, bias, bias_f32, (bf16_t*)out, 1, N, K, K, ldo, 0, 0, rows, 0, ra, na, GroupStride{});
     else
         gemm_skinny_kernel<1, 1, 16, bf16_t, false, true, 2, true, true><<<grid, dim3(16 * 64), lds, stream>>>(
-            nullptr, (const bf16_t*)w, bias, bias_f32, (bf16_t*)out, 1, N, K, K, ldo, 0, 0, 0, 0, ra, na);
+            nullptr, (const bf16_t*)w, bias, bias_f32, (bf16_t*)out, 1, N, K, K, ldo, 0, 0, 0, 0, ra, na, GroupStride{});
     TL_CHECK_LAUNCH("gemm_rope_normed");
     return TL_OK;
 }
@@ -1931,7 +1947,7 @@ extern "C" int tl_gemm_swiglu_normed(const void* residual, void* residual_out, c
     const StripPlan p = plan_strips(I, 2 * TL_COMPUTE_UNITS, 16, false);       // every work-group makes x once and walks its run of outputs
     const size_t lds = (size_t)16 * 1024 + (size_t)(K + 8) * 2;
     gemm_skinny_kernel<1, 1, 16, bf16_t, true, true, 2, false, true><<<dim3(p.groups), dim3(16 * 64), lds, stream>>>(
-        nullptr, (const bf16_t*)w, nullptr, 0, (bf16_t*)out, 1, N, K, K, I, I, 0, p.per_strip, p.per_group, RopeArgs{}, na);
+        nullptr, (const bf16_t*)w, nullptr, 0, (bf16_t*)out, 1, N, K, K, I, I, 0, p.per_strip, p.per_group, RopeArgs{}, na, GroupStride{});
     TL_CHECK_LAUNCH("gemm_swiglu_normed");
     return TL_OK;
 }
@@ -2049,7 +2065,7 @@ extern "C" int tl_gemm_partials(const void* x, const void* w, void* out, int M, 
         static hipError_t allowed = allow_lds(kernel, lds);
         TL_REQUIRE(allowed == hipSuccess, "gemm_partials: cannot get %zu bytes of shared memory", lds);
         dim3 grid(((M + 63) / 64) * ((N + 63) / 64), P), block(256);
-        kernel<<<grid, block, lds, stream>>>((const bf16_t*)x, (const bf16_t*)w, nullptr, 0, (float*)out, M, N, K, ldx, N, 0, k_per);
+        kernel<<<grid, block, lds, stream>>>((const bf16_t*)x, (const bf16_t*)w, nullptr, 0, (float*)out, M, N, K, ldx, N, 0, k_per, GroupStride{});
         TL_CHECK_LAUNCH("gemm_partials");
         return TL_OK;
     }
@@ -2057,15 +2073,49 @@ extern "C" int tl_gemm_partials(const void* x, const void* w, void* out, int M, 
     dim3 grid((N + 63) / 64, P), block(8 * 64);
     const size_t red_bytes = (size_t)8 * 4 * (M <= 16 ? 1 : (M <= 32 ? 2 : 4)) * 1024;
     if (M <= 16)
-        gemm_skinny_kernel<4, 1, 8, float, false, false, skinny_depth<4, 1, 8>()><<<grid, block, red_bytes, stream>>>((const bf16_t*)x, (const bf16_t*)w, nullptr, 0, (float*)out, M, N, K, ldx, N, 0, k_per, 0, 0, RopeArgs{}, NormArgs{});
+        gemm_skinny_kernel<4, 1, 8, float, false, false, skinny_depth<4, 1, 8>()><<<grid, block, red_bytes, stream>>>((const bf16_t*)x, (const bf16_t*)w, nullptr, 0, (float*)out, M, N, K, ldx, N, 0, k_per, 0, 0, RopeArgs{}, NormArgs{}, GroupStride{});
     else if (M <= 32)
-        gemm_skinny_kernel<4, 2, 8, float, false, false, skinny_depth<4, 2, 8>()><<<grid, block, red_bytes, stream>>>((const bf16_t*)x, (const bf16_t*)w, nullptr, 0, (float*)out, M, N, K, ldx, N, 0, k_per, 0, 0, RopeArgs{}, NormArgs{});
+        gemm_skinny_kernel<4, 2, 8, float, false, false, skinny_depth<4, 2, 8>()><<<grid, block, red_bytes, stream>>>((const bf16_t*)x, (const bf16_t*)w, nullptr, 0, (float*)out, M, N, K, ldx, N, 0, k_per, 0, 0, RopeArgs{}, NormArgs{}, GroupStride{});
     else {
         auto kernel = gemm_skinny_kernel<4, 4, 8, float, false, false, skinny_depth<4, 4, 8>()>;
         static hipError_t allowed = allow_lds(kernel, 128 * 1024);
         TL_REQUIRE(allowed == hipSuccess, "gemm_partials: cannot get %zu bytes of shared memory", red_bytes);
-        kernel<<<grid, block, red_bytes, stream>>>((const bf16_t*)x, (const bf16_t*)w, nullptr, 0, (float*)out, M, N, K, ldx, N, 0, k_per, 0, 0, RopeArgs{}, NormArgs{});
+        kernel<<<grid, block, red_bytes, stream>>>((const bf16_t*)x, (const bf16_t*)w, nullptr, 0, (float*)out, M, N, K, ldx, N, 0, k_per, 0, 0, RopeArgs{}, NormArgs{}, GroupStride{});
     }
     TL_CHECK_LAUNCH("gemm_partials");
+    return TL_OK;
+}
+
+// `groups` products of equal shape: out_g = x_g w_g^T with x_g = x + g * x_group (elements), w_g the g-th of the matrices [groups, N, K] and out_g =
+// out + g * out_group.  One launch where the few-rows kernel or the direct-load tiles take the shape (bfloat16), one per product otherwise.
+extern "C" int tl_gemm_groups(const void* x, long x_group, const void* w, void* out, long out_group, int groups, int M, int N, int K, int ldx, int ldo,
+                              int dtype, int out_f32, hipStream_t stream) {
+    TL_REQUIRE(groups > 0 && groups <= 64 && M >= 0 && N > 0 && K > 0 && ldx >= K && ldo >= N && x_group >= 0 && out_group >= 0, "gemm_groups: bad sizes groups=%d M=%d N=%d K=%d", groups, M, N, K);
+    if (M == 0) return TL_OK;
+    Groups gr;
+    gr.count = groups;
+    gr.stride = GroupStride{x_group, (long)N * K, out_group};
+    const bool aligned = K % 8 == 0 && ldx % 8 == 0 && x_group % 8 == 0 && out_group % 8 == 0 && ((uintptr_t)x % 16) == 0 && ((uintptr_t)w % 16) == 0;
+    if (dtype == TL_DT_BF16 && aligned && K % 64 == 0 && (M > 32 || (M > 8 && (long)N * groups >= 16384))) {
+        const DlTile tile = pick_dl_tile(M, N, K, false, nullptr, false, groups);
+        const int rc = out_f32 ? launch_dl_tile<float, false>(tile, x, w, nullptr, 0, out, M, N, K, ldx, ldo, 0, stream, 1, 0, gr)
+                               : launch_dl_tile<bf16_t, false>(tile, x, w, nullptr, 0, out, M, N, K, ldx, ldo, 0, stream, 1, 0, gr);
+        if (rc != TL_OK) return rc;
+        TL_CHECK_LAUNCH("gemm_groups");
+        return TL_OK;
+    }
+    if (dtype == TL_DT_BF16 && aligned && M <= 64) {
+        if (M <= 16) pick_skinny<1>(x, w, nullptr, 0, out, M, N, K, ldx, ldo, out_f32, stream, gr);
+        else if (M <= 32) pick_skinny<2>(x, w, nullptr, 0, out, M, N, K, ldx, ldo, out_f32, stream, gr);
+        else pick_skinny<4>(x, w, nullptr, 0, out, M, N, K, ldx, ldo, out_f32, stream, gr);
+        TL_CHECK_LAUNCH("gemm_groups");
+        return TL_OK;
+    }
+    const size_t esize = dtype == TL_DT_BF16 ? 2 : 4, osize = (dtype == TL_DT_BF16 && !out_f32) ? 2 : 4;
+    for (int g = 0; g < groups; ++g) {
+        const int rc = tl_gemm((const char*)x + esize * g * x_group, (const char*)w + esize * g * N * K, nullptr, 0, (char*)out + osize * g * out_group, M, N, K,
+                               ldx, ldo, dtype, out_f32, stream);
+        if (rc != TL_OK) return rc;
+    }
     return TL_OK;
 }

@@ -9,6 +9,7 @@
 // value for every block of `pool` positions that lies wholly before its window, blocks 0 .. (p - window + 1) / pool - 1; block b's key
 // and value are the means of the cached keys and values of the positions b * pool .. b * pool + pool - 1 and lie, as a token's would, in
 // row b of planes of their own with a block table of their own (pool_blocks_kernel makes them when a step brings a block's last token).
+// A third one: values that lie in the cache turned by their own positions; a head's output at position p is turned back by p.
 #include "common.h"
 
 // ------------------------------------------------------------------ cache write
@@ -63,6 +64,23 @@ struct LocalMask {
     }
 };
 
+// The turn of a head's output back from its position (freq == null: none): of the first `dims` columns the pair (2m, 2m + 1), or, `halves`,
+// (m, m + dims / 2), turns by -position * freq[m]; further columns pass.  Columns are taken in pairs, pair m at column_a(m) and column_b(m).
+struct OutputTurn {
+    const float* freq;       // [dims / 2]
+    int dims, halves;
+    __device__ __forceinline__ int column_a(int m) const { return (halves && m < dims / 2) ? m : 2 * m; }
+    __device__ __forceinline__ int column_b(int m) const { return (halves && m < dims / 2) ? m + dims / 2 : 2 * m + 1; }
+    __device__ __forceinline__ void turn(int m, int position, float& u, float& v) const {
+        if (m >= dims / 2) return;
+        float sn, c;
+        sincosf((float)position * freq[m], &sn, &c);
+        const float a = u, b = v;
+        u = __fmaf_rn(a, c, __fmul_rn(b, sn));
+        v = __fmaf_rn(b, c, -__fmul_rn(a, sn));
+    }
+};
+
 __device__ __forceinline__ float cap_score(float s, float cap) { return cap > 0.f ? cap * tanhf(s / cap) : s; }
 
 // ------------------------------------------------------------------ the general kernel
@@ -81,7 +99,7 @@ local_attention_kernel(const T* __restrict__ q, int q_ld, T* __restrict__ out, i
                        const T* __restrict__ v_plane, const int* __restrict__ block_table, int table_ld, const int* __restrict__ token_req,
                        const int* __restrict__ positions, int heads, int kv_heads, int dim, int vdim, int page_size, float scale, float cap,
                        LocalMask mask, float gain, const float* __restrict__ sink, const T* __restrict__ pk_plane, const T* __restrict__ pv_plane,
-                       const int* __restrict__ pool_table, int pool_table_ld, int pool) {
+                       const int* __restrict__ pool_table, int pool_table_ld, int pool, OutputTurn back) {
     __shared__ float sq[LA_MAX_DIM];
     __shared__ float sm[LA_WAVES], sl[LA_WAVES];
     __shared__ float sacc[LA_WAVES][LA_MAX_DIM];
@@ -154,10 +172,22 @@ local_attention_kernel(const T* __restrict__ q, int q_ld, T* __restrict__ out, i
         }
         if (sink) den += expf(sink[head] - top);
         const float norm = gain / den;
-        for (int col = lane; col < vdim; col += TL_WAVE) {
+        auto joined = [&](int col) {
             float o = 0.f;
             for (int w = 0; w < LA_WAVES; ++w) o = fmaf(sacc[w][col], f[w], o);
-            out[(size_t)t * out_ld + head * vdim + col] = from_float<T>(o * norm);
+            return o * norm;
+        };
+        T* orow = out + (size_t)t * out_ld + head * vdim;
+        if (back.freq) {
+            for (int m = lane; m < vdim / 2; m += TL_WAVE) {
+                const int ca = back.column_a(m), cb = back.column_b(m);
+                float u = joined(ca), v = joined(cb);
+                back.turn(m, p, u, v);
+                orow[ca] = from_float<T>(u);
+                orow[cb] = from_float<T>(v);
+            }
+        } else {
+            for (int col = lane; col < vdim; col += TL_WAVE) orow[col] = from_float<T>(joined(col));
         }
     }
 }
@@ -205,7 +235,8 @@ local_attention_mfma_kernel(const bf16_t* __restrict__ q, int q_ld, bf16_t* __re
                             const int* __restrict__ req_indptr, const int* __restrict__ ctx_lens, const int* __restrict__ tile_req,
                             const int* __restrict__ tile_tok0, int heads, int kv_heads, int page_size, float scale, float cap,
                             LocalMask mask, float gain, const float* __restrict__ sink, const bf16_t* __restrict__ pk_plane,
-                            const bf16_t* __restrict__ pv_plane, const int* __restrict__ pool_table, int pool_table_ld, int pool_table_width, int pool) {
+                            const bf16_t* __restrict__ pv_plane, const int* __restrict__ pool_table, int pool_table_ld, int pool_table_width, int pool,
+                            OutputTurn back) {
     constexpr int dim = DK * 32, vdim = DV * 16;
     extern __shared__ float la_smem[];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, li = lane & 15, kq = lane >> 4;
@@ -354,21 +385,44 @@ local_attention_mfma_kernel(const bf16_t* __restrict__ q, int q_ld, bf16_t* __re
     for (int j = 0; j < DV; ++j)
         *(float4*)(sm_o + ((size_t)wave * LAM_TOKENS + li) * vdim + 16 * j + 4 * kq) = make_float4(acc[j][0], acc[j][1], acc[j][2], acc[j][3]);
     __syncthreads();
-    for (int idx = threadIdx.x; idx < n_tile * vdim; idx += blockDim.x) {
-        const int tok = idx / vdim, col = idx % vdim;
+    const float sink2 = sink ? sink[head] * LA_LOG2E : -INFINITY;       // in units of log 2, like the maxima
+    // columns ca and cb of a token (cb < 0: ca alone)
+    auto joined = [&](int tok, int ca, int cb, float& u, float& v) {
         float top = sm_m[tok];
 #pragma unroll
         for (int w = 1; w < LAM_WAVES; ++w) top = fmaxf(top, sm_m[w * LAM_TOKENS + tok]);
-        const float sink2 = sink ? sink[head] * LA_LOG2E : -INFINITY;       // in units of log 2, like the maxima
         top = fmaxf(top, sink2);
-        float den = __builtin_amdgcn_exp2f(sink2 - top), o = 0.f;           // (0 without a sink)
+        float den = __builtin_amdgcn_exp2f(sink2 - top);                    // (0 without a sink)
+        u = v = 0.f;
 #pragma unroll
         for (int w = 0; w < LAM_WAVES; ++w) {
             const float f = __builtin_amdgcn_exp2f(sm_m[w * LAM_TOKENS + tok] - top);        // (0 for a wave that saw no key of this token)
             den = fmaf(sm_l[w * LAM_TOKENS + tok], f, den);
-            o = fmaf(sm_o[((size_t)w * LAM_TOKENS + tok) * vdim + col], f, o);
+            const float* o = sm_o + ((size_t)w * LAM_TOKENS + tok) * vdim;
+            u = fmaf(o[ca], f, u);
+            if (cb >= 0) v = fmaf(o[cb], f, v);
         }
-        out[(size_t)(first + tok0 + tok) * out_ld + head * vdim + col] = from_float<bf16_t>(o * (gain / den));
+        u *= gain / den;
+        v *= gain / den;
+    };
+    bf16_t* const orow0 = out + (size_t)(first + tok0) * out_ld + head * vdim;
+    if (back.freq) {
+        for (int idx = threadIdx.x; idx < n_tile * (vdim / 2); idx += blockDim.x) {
+            const int tok = idx / (vdim / 2), m = idx % (vdim / 2);
+            const int ca = back.column_a(m), cb = back.column_b(m);
+            float u, v;
+            joined(tok, ca, cb, u, v);
+            back.turn(m, p0 + tok, u, v);
+            orow0[(size_t)tok * out_ld + ca] = from_float<bf16_t>(u);
+            orow0[(size_t)tok * out_ld + cb] = from_float<bf16_t>(v);
+        }
+        return;
+    }
+    for (int idx = threadIdx.x; idx < n_tile * vdim; idx += blockDim.x) {
+        const int tok = idx / vdim, col = idx % vdim;
+        float u, v;
+        joined(tok, col, -1, u, v);
+        orow0[(size_t)tok * out_ld + col] = from_float<bf16_t>(u);
     }
 }
 
@@ -377,7 +431,7 @@ static void launch_local_mfma(const void* q, int q_ld, void* out, int out_ld, co
                               int table_ld, int table_width, const void* req_indptr, const void* ctx_lens, const void* tile_req,
                               const void* tile_tok0, int tiles, int heads, int kv_heads, int page_size, float scale, float cap, LocalMask mask,
                               float gain, const void* sink, const void* pk_plane, const void* pv_plane, const void* pool_table, int pool_table_ld,
-                              int pool_table_width, int pool, hipStream_t stream) {
+                              int pool_table_width, int pool, OutputTurn back, hipStream_t stream) {
     dim3 grid(tiles, heads), block(LAM_WAVES * TL_WAVE);
     const size_t smem = sizeof(float) * LAM_WAVES * LAM_TOKENS * (2 + DV * 16);
     auto kernel = local_attention_mfma_kernel<DK, DV>;
@@ -389,7 +443,7 @@ static void launch_local_mfma(const void* q, int q_ld, void* out, int out_ld, co
     kernel<<<grid, block, smem, stream>>>((const bf16_t*)q, q_ld, (bf16_t*)out, out_ld, (const bf16_t*)k_plane, (const bf16_t*)v_plane,
         (const int*)block_table, table_ld, table_width, (const int*)req_indptr, (const int*)ctx_lens, (const int*)tile_req, (const int*)tile_tok0,
         heads, kv_heads, page_size, scale, cap, mask, gain, (const float*)sink, (const bf16_t*)pk_plane, (const bf16_t*)pv_plane, (const int*)pool_table,
-        pool_table_ld, pool_table_width, pool);
+        pool_table_ld, pool_table_width, pool, back);
 }
 
 // Whether the matrix-core kernel is built for these sizes.
@@ -406,7 +460,8 @@ extern "C" int tl_local_attention_tiles(const void* q, int q_ld, void* out, int 
                                         const void* tile_req, const void* tile_tok0, int tiles, int heads, int kv_heads, int dim, int vdim,
                                         int page_size, float scale, float cap, int chunk, int window, float gain, const void* sink,
                                         const void* pk_plane, const void* pv_plane, const void* pool_table, int pool_table_ld, int pool_table_width,
-                                        int pool, int keep_first, hipStream_t stream) {
+                                        int pool, int keep_first, const void* turn_freq, int turn_dims, int turn_halves, hipStream_t stream) {
+    TL_REQUIRE(!turn_freq || (turn_dims > 0 && turn_dims % 2 == 0 && turn_dims <= vdim && vdim % 2 == 0), "local_attention_tiles: an output of %d columns turned over %d", vdim, turn_dims);
     TL_REQUIRE(keep_first >= 0 && (keep_first == 0 || (window > 0 && chunk == 0)), "local_attention_tiles: kept first tokens stand beside a window, without chunks");
     TL_REQUIRE(pool >= 0 && (pool == 0 || (window > 0 && pk_plane && pv_plane && pool_table && pool_table_ld >= pool_table_width && pool_table_width > 0)),
                "local_attention_tiles: pooled blocks need a window, their planes and their block table");
@@ -416,10 +471,11 @@ extern "C" int tl_local_attention_tiles(const void* q, int q_ld, void* out, int 
                "local_attention_tiles: rows too short or not aligned");
     if (tiles == 0) return TL_OK;
     const LocalMask mask{chunk, window, keep_first};
+    const OutputTurn back{(const float*)turn_freq, turn_dims, turn_halves};
 #define TL_LAM(DK, DV)                                                                                                                      \
     launch_local_mfma<DK, DV>(q, q_ld, out, out_ld, k_plane, v_plane, block_table, table_ld, table_width, req_indptr, ctx_lens, tile_req,  \
                               tile_tok0, tiles, heads, kv_heads, page_size, scale, cap, mask, gain, sink, pk_plane, pv_plane, pool_table,        \
-                              pool_table_ld, pool_table_width, pool, stream)
+                              pool_table_ld, pool_table_width, pool, back, stream)
 #define TL_LAM_V(DK)                                     \
     switch (vdim) {                                      \
         case 16: TL_LAM(DK, 1); break;                   \
@@ -448,7 +504,9 @@ extern "C" int tl_local_attention(const void* q, int q_ld, void* out, int out_ld
                                   const void* block_table, int table_ld, int table_width, const void* token_req, const void* positions,
                                   int tokens, int heads, int kv_heads, int dim, int vdim, int page_size, float scale, float cap, int chunk,
                                   int window, float gain, const void* sink, const void* pk_plane, const void* pv_plane, const void* pool_table,
-                                  int pool_table_ld, int pool, int keep_first, int dtype, hipStream_t stream) {
+                                  int pool_table_ld, int pool, int keep_first, const void* turn_freq, int turn_dims, int turn_halves, int dtype,
+                                  hipStream_t stream) {
+    TL_REQUIRE(!turn_freq || (turn_dims > 0 && turn_dims % 2 == 0 && turn_dims <= vdim && vdim % 2 == 0), "local_attention: an output of %d columns turned over %d", vdim, turn_dims);
     TL_REQUIRE(keep_first >= 0 && (keep_first == 0 || (window > 0 && chunk == 0)), "local_attention: kept first tokens stand beside a window, without chunks");
     TL_REQUIRE(pool >= 0 && (pool == 0 || (window > 0 && pk_plane && pv_plane && pool_table)), "local_attention: pooled blocks need a window, their planes and their block table");
     TL_REQUIRE(tokens >= 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && dim > 0 && vdim > 0 && page_size > 0, "local_attention: bad sizes");
@@ -457,15 +515,16 @@ extern "C" int tl_local_attention(const void* q, int q_ld, void* out, int out_ld
     TL_REQUIRE(heads <= 65535, "local_attention: too many heads");
     if (tokens == 0) return TL_OK;
     const LocalMask mask{chunk, window, keep_first};
+    const OutputTurn back{(const float*)turn_freq, turn_dims, turn_halves};
     dim3 grid(tokens, heads), block(LA_WAVES * TL_WAVE);
     if (dtype == TL_DT_F32)
         local_attention_kernel<float><<<grid, block, 0, stream>>>((const float*)q, q_ld, (float*)out, out_ld, (const float*)k_plane, (const float*)v_plane,
             (const int*)block_table, table_ld, (const int*)token_req, (const int*)positions, heads, kv_heads, dim, vdim, page_size, scale, cap, mask, gain,
-            (const float*)sink, (const float*)pk_plane, (const float*)pv_plane, (const int*)pool_table, pool_table_ld, pool);
+            (const float*)sink, (const float*)pk_plane, (const float*)pv_plane, (const int*)pool_table, pool_table_ld, pool, back);
     else if (dtype == TL_DT_BF16)
         local_attention_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)q, q_ld, (bf16_t*)out, out_ld, (const bf16_t*)k_plane, (const bf16_t*)v_plane,
             (const int*)block_table, table_ld, (const int*)token_req, (const int*)positions, heads, kv_heads, dim, vdim, page_size, scale, cap, mask, gain,
-            (const float*)sink, (const bf16_t*)pk_plane, (const bf16_t*)pv_plane, (const int*)pool_table, pool_table_ld, pool);
+            (const float*)sink, (const bf16_t*)pk_plane, (const bf16_t*)pv_plane, (const int*)pool_table, pool_table_ld, pool, back);
     else TL_REQUIRE(false, "local_attention: unknown dtype %d", dtype);
     TL_CHECK_LAUNCH("local_attention");
     return TL_OK;
@@ -542,25 +601,42 @@ extern "C" int tl_pool_blocks(const void* k_plane, const void* v_plane, int page
 //   rotation (inv_freq != null) of the first `dims` numbers by angle_i = float(position) * inv_freq[i]: pair (2i, 2i + 1), or, `halves`,
 //   pair (i, i + dims / 2); (u, v) <- (u cos - v sin, v cos + u sin).  What lies beyond `dims` is not turned.  One rounding at the end.
 // `raw_b` (optional, [T, raw_ld]): the heads_b heads as they come, before norm and rotation, are copied there (values that are the keys
-// as projected).
+// as projected).  `magnitude`: a factor on cosine and sine of these heads' rotation.
+// `values`: heads_c more heads of vdim numbers behind those (the values), with a norm without a weight (`unit`) and a rotation of their own.
+// `pages`: the heads_b and heads_c heads (keys and values) go to their pages instead of back to x, as kv_cache_write_kernel puts them there.
+struct ValueHeads {
+    int heads, vdim, unit;
+    const float* inv_freq;
+    int dims, halves;
+};
+template <typename T>
+struct PagesOf {
+    const int *token_req, *block_table;
+    int table_ld, table_width;
+    T *k_plane, *v_plane;            // null: x is written
+    int pages, page_size;
+};
 #define HNR_WAVES 4
 template <typename T>
 __global__ void __launch_bounds__(HNR_WAVES * TL_WAVE)
 head_norm_rotate_kernel(T* __restrict__ x, int ld, int tokens, int heads_a, int heads_b, int dim, const float* __restrict__ norm_a,
                         const float* __restrict__ norm_b, float eps, const int* __restrict__ positions, const float* __restrict__ inv_freq,
-                        int dims, int halves, T* __restrict__ raw_b, int raw_ld) {
+                        int dims, int halves, T* __restrict__ raw_b, int raw_ld, float magnitude, ValueHeads values, PagesOf<T> to) {
     __shared__ float sv[HNR_WAVES][LA_MAX_DIM];
     const int wave = threadIdx.x / TL_WAVE, lane = threadIdx.x % TL_WAVE;
-    const int heads = heads_a + heads_b;
+    const int heads_ab = heads_a + heads_b, heads = heads_ab + values.heads, keys_dim = dim;
     const long item = (long)blockIdx.x * HNR_WAVES + wave;
     const bool live = item < (long)tokens * heads;
     const int t = live ? (int)(item / heads) : 0, h = live ? (int)(item % heads) : 0;
-    T* row = x + (size_t)t * ld + (size_t)h * dim;
+    const bool is_value = h >= heads_ab;
+    T* row = x + (size_t)t * ld + (is_value ? (size_t)heads_ab * dim + (size_t)(h - heads_ab) * values.vdim : (size_t)h * dim);
     float* v = sv[wave];
-    const float* w = h < heads_a ? norm_a : norm_b;
+    const float* w = is_value ? nullptr : (h < heads_a ? norm_a : norm_b);
+    const bool normed = is_value ? values.unit != 0 : w != nullptr;
+    if (is_value) { dim = values.vdim; inv_freq = values.inv_freq; dims = values.dims; halves = values.halves; magnitude = 1.f; }
     float ss = 0.f;
     if (live) {
-        T* raw = (raw_b && h >= heads_a) ? raw_b + (size_t)t * raw_ld + (size_t)(h - heads_a) * dim : nullptr;
+        T* raw = (raw_b && h >= heads_a && !is_value) ? raw_b + (size_t)t * raw_ld + (size_t)(h - heads_a) * dim : nullptr;
         for (int d = lane; d < dim; d += TL_WAVE) {
             const T x0 = row[d];
             if (raw) raw[d] = x0;
@@ -569,9 +645,9 @@ head_norm_rotate_kernel(T* __restrict__ x, int ld, int tokens, int heads_a, int 
     }
     ss = wave_sum(ss);
     __syncthreads();
-    if (live && w) {
+    if (live && normed) {
         const float inv = 1.f / sqrtf(ss / (float)dim + eps);
-        for (int d = lane; d < dim; d += TL_WAVE) v[d] = v[d] * inv * w[d];
+        for (int d = lane; d < dim; d += TL_WAVE) v[d] = v[d] * inv * (w ? w[d] : 1.f);
     }
     __syncthreads();
     if (live && inv_freq) {
@@ -580,32 +656,59 @@ head_norm_rotate_kernel(T* __restrict__ x, int ld, int tokens, int heads_a, int 
             const int ia = halves ? i : 2 * i, ib = halves ? i + dims / 2 : 2 * i + 1;
             float sn, c;
             sincosf(pos * inv_freq[i], &sn, &c);
+            sn *= magnitude;
+            c *= magnitude;
             const float a = v[ia], b = v[ib];
             v[ia] = __fmaf_rn(a, c, -__fmul_rn(b, sn));
             v[ib] = __fmaf_rn(b, c, __fmul_rn(a, sn));
         }
     }
     __syncthreads();
-    if (live)
+    if (!live) return;
+    if (!to.k_plane || h < heads_a) {
         for (int d = lane; d < dim; d += TL_WAVE) row[d] = from_float<T>(v[d]);
+        return;
+    }
+    const int p = positions[t], block = p / to.page_size;
+    if (p < 0 || block >= to.table_width) return;
+    const int page = to.block_table[(size_t)to.token_req[t] * to.table_ld + block];
+    if (page <= 0 || page >= to.pages) return;          // page 0, the sentinel of rows that belong to no request, is never written
+    const int at = p % to.page_size;
+    if (is_value) {
+        T* dst = to.v_plane + ((size_t)page * values.heads + h - heads_ab) * dim * to.page_size + at;
+        for (int d = lane; d < dim; d += TL_WAVE) dst[(size_t)d * to.page_size] = from_float<T>(v[d]);
+    } else {
+        T* dst = to.k_plane + (((size_t)page * heads_b + h - heads_a) * to.page_size + at) * keys_dim;
+        for (int d = lane; d < dim; d += TL_WAVE) dst[d] = from_float<T>(v[d]);
+    }
 }
 
 extern "C" int tl_head_norm_rotate(void* x, int ld, int tokens, int heads_a, int heads_b, int dim, const void* norm_a, const void* norm_b, float eps,
-                                   const void* positions, const void* inv_freq, int dims, int halves, void* raw_b, int raw_ld, int dtype, hipStream_t stream) {
+                                   const void* positions, const void* inv_freq, int dims, int halves, void* raw_b, int raw_ld, float magnitude,
+                                   int heads_c, int vdim, int unit_c, const void* inv_freq_c, int dims_c, int halves_c, const void* token_req,
+                                   const void* block_table, int table_ld, int table_width, void* k_plane, void* v_plane, int pages, int page_size,
+                                   int dtype, hipStream_t stream) {
+    TL_REQUIRE(heads_c >= 0 && (heads_c == 0 || (vdim > 0 && vdim <= LA_MAX_DIM && ld >= (heads_a + heads_b) * dim + heads_c * vdim)), "head_norm_rotate: bad sizes of the values");
+    TL_REQUIRE(heads_c == 0 || !inv_freq_c || (positions && dims_c > 0 && dims_c % 2 == 0 && dims_c <= vdim), "head_norm_rotate: a rotation over %d of %d numbers of a value", dims_c, vdim);
+    TL_REQUIRE(!k_plane || (v_plane && heads_c == heads_b && heads_c > 0 && positions && token_req && block_table && table_width > 0 && table_ld >= table_width && pages > 0 && page_size > 0),
+               "head_norm_rotate: keys and values for the pages need as many heads of each, positions, planes and a block table");
     TL_REQUIRE(!raw_b || raw_ld >= heads_b * dim, "head_norm_rotate: the rows of the copy are too short");
     TL_REQUIRE(tokens >= 0 && heads_a >= 0 && heads_b >= 0 && heads_a + heads_b > 0 && dim > 0 && dim <= LA_MAX_DIM && ld >= (heads_a + heads_b) * dim,
                "head_norm_rotate: bad sizes");
     TL_REQUIRE(!inv_freq || (positions && dims > 0 && dims % 2 == 0 && dims <= dim), "head_norm_rotate: a rotation over %d of %d numbers", dims, dim);
     TL_REQUIRE((norm_a == nullptr) == (norm_b == nullptr) || heads_a == 0 || heads_b == 0, "head_norm_rotate: a norm for both kinds of heads or for neither");
     if (tokens == 0) return TL_OK;
-    const long items = (long)tokens * (heads_a + heads_b);
+    const long items = (long)tokens * (heads_a + heads_b + heads_c);
+    const ValueHeads values{heads_c, vdim, unit_c, (const float*)inv_freq_c, dims_c, halves_c};
     const int grid = (int)((items + HNR_WAVES - 1) / HNR_WAVES);
     if (dtype == TL_DT_F32)
         head_norm_rotate_kernel<float><<<grid, HNR_WAVES * TL_WAVE, 0, stream>>>((float*)x, ld, tokens, heads_a, heads_b, dim, (const float*)norm_a,
-            (const float*)norm_b, eps, (const int*)positions, (const float*)inv_freq, dims, halves, (float*)raw_b, raw_ld);
+            (const float*)norm_b, eps, (const int*)positions, (const float*)inv_freq, dims, halves, (float*)raw_b, raw_ld, magnitude, values,
+            PagesOf<float>{(const int*)token_req, (const int*)block_table, table_ld, table_width, (float*)k_plane, (float*)v_plane, pages, page_size});
     else if (dtype == TL_DT_BF16)
         head_norm_rotate_kernel<bf16_t><<<grid, HNR_WAVES * TL_WAVE, 0, stream>>>((bf16_t*)x, ld, tokens, heads_a, heads_b, dim, (const float*)norm_a,
-            (const float*)norm_b, eps, (const int*)positions, (const float*)inv_freq, dims, halves, (bf16_t*)raw_b, raw_ld);
+            (const float*)norm_b, eps, (const int*)positions, (const float*)inv_freq, dims, halves, (bf16_t*)raw_b, raw_ld, magnitude, values,
+            PagesOf<bf16_t>{(const int*)token_req, (const int*)block_table, table_ld, table_width, (bf16_t*)k_plane, (bf16_t*)v_plane, pages, page_size});
     else TL_REQUIRE(false, "head_norm_rotate: unknown dtype %d", dtype);
     TL_CHECK_LAUNCH("head_norm_rotate");
     return TL_OK;

@@ -1,5 +1,5 @@
 // Recurrent mixers with a fixed-size state per request: the matrix-memory recurrence (mLSTM), the gated delta rule behind its
-// short convolutions, and the gated per-head norm of their outputs.  State, gates, decays and the output's quotient are float whatever the
+// short convolutions, a recurrence whose decays are each key channel's and each token's own (the time mixing of RWKV), and the gated per-head norm of their outputs.  State, gates, decays and the output's quotient are float whatever the
 // activation type; queries, keys and values come in the activation type as the projection left them.
 #include "common.h"
 
@@ -829,5 +829,249 @@ extern "C" int tl_silu_float(const void* x, int ld, void* out, int rows, int col
     else if (dtype == TL_DT_BF16) silu_float_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)x, ld, (float*)out, cols, total);
     else TL_REQUIRE(false, "silu_float: unknown dtype %d", dtype);
     TL_CHECK_LAUNCH("silu_float");
+    return TL_OK;
+}
+
+// ------------------------------------------------------------------ decays per key channel
+// decay[t, n] = exp(-exp(w0[n] + sum_j w2t[j][n] * tanh(z[t, j]))): z float [tokens, rank], w2t float [rank][channels].  A work-group of 256
+// threads takes 256 channels of TT tokens, a thread a channel; the order of a sum does not depend on TT.
+template <int TT>
+__global__ void __launch_bounds__(256)
+channel_decay_kernel(const float* __restrict__ z, const float* __restrict__ w2t, const float* __restrict__ w0, float* __restrict__ decay,
+                     int tokens, int rank, int channels) {
+    extern __shared__ __attribute__((aligned(16))) float cd_tanh[];          // [rank][TT]
+    const int t0 = blockIdx.y * TT, n = blockIdx.x * 256 + threadIdx.x;
+    for (int i = threadIdx.x; i < rank * TT; i += 256) {
+        const int tt = i / rank, j = i % rank;
+        cd_tanh[j * TT + tt] = t0 + tt < tokens ? tanhf(z[(size_t)(t0 + tt) * rank + j]) : 0.f;
+    }
+    __syncthreads();
+    if (n >= channels) return;
+    float acc[TT];
+    const float start = w0[n];
+#pragma unroll
+    for (int tt = 0; tt < TT; ++tt) acc[tt] = start;
+#pragma unroll 8
+    for (int j = 0; j < rank; ++j) {
+        const float w = w2t[(size_t)j * channels + n];
+#pragma unroll
+        for (int tt = 0; tt < TT; ++tt) acc[tt] = fmaf(w, cd_tanh[j * TT + tt], acc[tt]);
+    }
+#pragma unroll
+    for (int tt = 0; tt < TT; ++tt)
+        if (t0 + tt < tokens) decay[(size_t)(t0 + tt) * channels + n] = expf(-expf(acc[tt]));
+}
+
+extern "C" int tl_channel_decay(const void* z, const void* w2t, const void* w0, void* decay, int tokens, int rank, int channels, hipStream_t stream) {
+    TL_REQUIRE(tokens >= 0 && rank > 0 && channels > 0, "channel_decay: bad sizes");
+    TL_REQUIRE(rank <= 1024, "channel_decay: built for ranks up to 1024, got %d", rank);
+    if (tokens == 0) return TL_OK;
+    const int blocks = (channels + 255) / 256;
+    if ((long)blocks * tokens <= 1024)
+        channel_decay_kernel<1><<<dim3(blocks, tokens), 256, sizeof(float) * rank, stream>>>((const float*)z, (const float*)w2t, (const float*)w0, (float*)decay, tokens, rank, channels);
+    else
+        channel_decay_kernel<8><<<dim3(blocks, (tokens + 7) / 8), 256, sizeof(float) * 8 * rank, stream>>>((const float*)z, (const float*)w2t, (const float*)w0, (float*)decay, tokens, rank, channels);
+    TL_CHECK_LAUNCH("channel_decay");
+    return TL_OK;
+}
+
+// ------------------------------------------------------------------ the recurrence with decays per key channel and a bonus
+// Per request and head a state S of dim x vdim numbers; per token, with r, k (dim), v (vdim), the decays w (dim) and the head's bonus u (dim):
+//   o = (S + diag(u) k v^T)^T r,   then   S <- diag(w) S + k v^T.
+// Column j of S needs only its own sum_i r[i] S[i][j] and the number sum_i r[i] u[i] k[i], which all columns of the head share and which is
+// made once per token.  The 16 lanes of a row of the wave share a column: lane i owns the rows 64 q + 4 i .. + 3 (q < RPL / 4) of it in
+// registers for all tokens of the step, so the lanes' pieces of r, k and w lie side by side in shared memory and those of the state side by
+// side in memory ([vdim][dim] per head).  Nothing but S itself passes from token to token: the sums over the lanes leave the chain.  A wave
+// has 4 columns, a work-group of four waves 16.  The order of every sum is fixed by dim, so a token's result depends neither on how its
+// request was cut into steps nor on what else the step holds.  Tokens are taken TB at a time (1, 4 or 16, by the longest portion of the
+// step), fetched into registers one batch ahead; a request's last batch is filled up with tokens that change nothing (k = 0, w = 1).
+// `last_rows` (optional, float [tokens, row_width]): the row of the request's last token goes to its slot from tail_off on (what the next
+// portion's first token finds of the token before it).
+template <typename T> __device__ __forceinline__ float4 wkv_load4(const T* p);
+template <> __device__ __forceinline__ float4 wkv_load4<float>(const float* p) { return *(const float4*)p; }
+template <> __device__ __forceinline__ float4 wkv_load4<bf16_t>(const bf16_t* p) {
+    const uint2 t = *(const uint2*)p;
+    return make_float4(__uint_as_float(t.x << 16), __uint_as_float(t.x & 0xffff0000u), __uint_as_float(t.y << 16), __uint_as_float(t.y & 0xffff0000u));
+}
+
+template <typename T, int RPL, int TB>
+__global__ void __launch_bounds__(256)
+wkv_scan_kernel(const T* __restrict__ rkv, int ld, int k_off, int v_off, const float* __restrict__ decay, const float* __restrict__ bonus,
+                float* __restrict__ state, size_t slot_stride, const int* __restrict__ slots, const int* __restrict__ req_indptr,
+                float* __restrict__ out, int heads, int dim, int vdim, int vec, const float* __restrict__ last_rows, int row_width, size_t tail_off) {
+    constexpr int ROWS = DELTA_L * RPL, Q = RPL / 4;            // ROWS >= dim
+    constexpr int PPT = ROWS / 4, PIECES = TB * PPT, NP = (PIECES + 255) / 256;      // pieces of four numbers: per token, per batch, per thread
+    __shared__ __attribute__((aligned(16))) float sr[TB * ROWS], sk[TB * ROWS], sw[TB * ROWS];
+    __shared__ float sv[TB * DELTA_COLS], sb[TB];
+    const int req = blockIdx.z, head = blockIdx.y, col0 = blockIdx.x * DELTA_COLS;
+    const int tok0 = req_indptr[req], tok1 = req_indptr[req + 1];
+    if (tok0 >= tok1) return;
+    const int tid = threadIdx.x, wave = tid / TL_WAVE, lane = tid % TL_WAVE;
+    const int rg = lane & 15, cw = wave * 4 + (lane >> 4);       // the lane's place in its column, and the column within the work-group
+    const int col = col0 + cw;
+    const bool col_ok = col < vdim;
+    float* slot = state + (size_t)slots[req] * slot_stride;
+    float* st = slot + ((size_t)head * vdim + col) * dim;
+
+    float S[RPL], ub[RPL];
+    const bool vec_state = vec && ((uintptr_t)state & 15) == 0 && (slot_stride & 3) == 0;
+#pragma unroll
+    for (int q = 0; q < Q; ++q) {
+        const int row = 64 * q + 4 * rg;
+        if (vec_state && col_ok && row + 4 <= dim) {
+            const float4 x = *(const float4*)(st + row);
+            S[4 * q] = x.x; S[4 * q + 1] = x.y; S[4 * q + 2] = x.z; S[4 * q + 3] = x.w;
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) S[4 * q + e] = (col_ok && row + e < dim) ? st[row + e] : 0.f;
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ub[4 * q + e] = row + e < dim ? bonus[head * dim + row + e] : 0.f;
+    }
+
+    float4 pr[NP], pk[NP], pw[NP];
+    float pv = 0.f;
+    auto fetch = [&](int base) {
+        const int nb = min(TB, tok1 - base);
+#pragma unroll
+        for (int j = 0; j < NP; ++j) {
+            const int idx = tid + j * 256, t = idx / PPT, e = (idx % PPT) * 4;
+            pr[j] = pk[j] = make_float4(0.f, 0.f, 0.f, 0.f);
+            pw[j] = make_float4(1.f, 1.f, 1.f, 1.f);
+            if (idx < PIECES && t < nb && e < dim) {
+                const T* row = rkv + (size_t)(base + t) * ld + head * dim + e;
+                const float* wrow = decay + ((size_t)(base + t) * heads + head) * dim + e;
+                if (vec) {
+                    pr[j] = wkv_load4<T>(row);
+                    pk[j] = wkv_load4<T>(row + k_off);
+                    pw[j] = *(const float4*)wrow;
+                } else {
+                    float a[4], b[4], c[4];
+#pragma unroll
+                    for (int u = 0; u < 4; ++u) {
+                        const bool ok = e + u < dim;
+                        a[u] = ok ? to_float(row[u]) : 0.f;
+                        b[u] = ok ? to_float(row[k_off + u]) : 0.f;
+                        c[u] = ok ? wrow[u] : 1.f;
+                    }
+                    pr[j] = make_float4(a[0], a[1], a[2], a[3]);
+                    pk[j] = make_float4(b[0], b[1], b[2], b[3]);
+                    pw[j] = make_float4(c[0], c[1], c[2], c[3]);
+                }
+            }
+        }
+        if (tid < TB * DELTA_COLS) {
+            const int t = tid / DELTA_COLS, c = tid % DELTA_COLS;
+            pv = (t < nb && col0 + c < vdim) ? to_float(rkv[(size_t)(base + t) * ld + v_off + head * vdim + col0 + c]) : 0.f;
+        }
+    };
+    fetch(tok0);
+    for (int base = tok0; base < tok1; base += TB) {
+        const int nb = min(TB, tok1 - base);
+        shared_barrier();                              // the batch before has been worked on
+#pragma unroll
+        for (int j = 0; j < NP; ++j) {
+            const int idx = tid + j * 256;
+            if (idx < PIECES) {
+                *(float4*)(sr + idx * 4) = pr[j];
+                *(float4*)(sk + idx * 4) = pk[j];
+                *(float4*)(sw + idx * 4) = pw[j];
+            }
+        }
+        if (tid < TB * DELTA_COLS) sv[tid] = pv;
+        if (base + TB < tok1) fetch(base + TB);
+        shared_barrier();
+        // the bonus sums: the 16 lanes of column cw make token cw's
+        if (cw < TB) {
+            float b4[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int q = 0; q < Q; ++q) {
+                const float4 k4 = *(const float4*)(sk + cw * ROWS + 64 * q + 4 * rg), r4 = *(const float4*)(sr + cw * ROWS + 64 * q + 4 * rg);
+                b4[0] = fmaf(k4.x * ub[4 * q], r4.x, b4[0]);
+                b4[1] = fmaf(k4.y * ub[4 * q + 1], r4.y, b4[1]);
+                b4[2] = fmaf(k4.z * ub[4 * q + 2], r4.z, b4[2]);
+                b4[3] = fmaf(k4.w * ub[4 * q + 3], r4.w, b4[3]);
+            }
+            const float b = row16_sum((b4[0] + b4[1]) + (b4[2] + b4[3]));
+            if (rg == 0) sb[cw] = b;
+        }
+        shared_barrier();
+        float mine = 0.f;                              // the output of token rg of the batch
+#pragma unroll 4
+        for (int t = 0; t < TB; ++t) {
+            const float vt = sv[t * DELTA_COLS + cw];
+            float o4[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int q = 0; q < Q; ++q) {
+                const int at = t * ROWS + 64 * q + 4 * rg;
+                const float4 r4 = *(const float4*)(sr + at), k4 = *(const float4*)(sk + at), w4 = *(const float4*)(sw + at);
+                o4[0] = fmaf(r4.x, S[4 * q], o4[0]);
+                o4[1] = fmaf(r4.y, S[4 * q + 1], o4[1]);
+                o4[2] = fmaf(r4.z, S[4 * q + 2], o4[2]);
+                o4[3] = fmaf(r4.w, S[4 * q + 3], o4[3]);
+                S[4 * q] = fmaf(w4.x, S[4 * q], k4.x * vt);
+                S[4 * q + 1] = fmaf(w4.y, S[4 * q + 1], k4.y * vt);
+                S[4 * q + 2] = fmaf(w4.z, S[4 * q + 2], k4.z * vt);
+                S[4 * q + 3] = fmaf(w4.w, S[4 * q + 3], k4.w * vt);
+            }
+            const float o = fmaf(sb[t], vt, row16_sum((o4[0] + o4[1]) + (o4[2] + o4[3])));
+            if (rg == t) mine = o;
+        }
+        if (rg < nb && col_ok) out[((size_t)(base + rg) * heads + head) * vdim + col] = mine;
+    }
+#pragma unroll
+    for (int q = 0; q < Q; ++q) {
+        const int row = 64 * q + 4 * rg;
+        if (vec_state && col_ok && row + 4 <= dim) *(float4*)(st + row) = make_float4(S[4 * q], S[4 * q + 1], S[4 * q + 2], S[4 * q + 3]);
+        else if (col_ok) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                if (row + e < dim) st[row + e] = S[4 * q + e];
+        }
+    }
+    if (last_rows && blockIdx.x == 0) {                // the heads' first work-groups share the row
+        for (int i = head * 256 + tid; i < row_width; i += heads * 256) slot[tail_off + i] = last_rows[(size_t)(tok1 - 1) * row_width + i];
+    }
+}
+
+template <typename T>
+static void launch_wkv_scan(const void* rkv, int ld, int k_off, int v_off, const void* decay, const void* bonus, void* state, long slot_stride,
+                            const void* slots, const void* req_indptr, void* out, int requests, int heads, int dim, int vdim, int longest,
+                            const void* last_rows, int row_width, long tail_off, hipStream_t stream) {
+    const int rpl = dim <= 64 ? 4 : dim <= 128 ? 8 : dim <= 192 ? 12 : 16;
+    const int tb = longest <= 1 ? 1 : (longest <= 4 ? 4 : DELTA_TB);
+    const int vec = dim % 4 == 0 && ld % 4 == 0 && k_off % 4 == 0 && ((uintptr_t)rkv % (4 * sizeof(T))) == 0 && ((uintptr_t)decay & 15) == 0;
+    dim3 grid((vdim + DELTA_COLS - 1) / DELTA_COLS, heads, requests), block(256);
+#define TL_WKV_B(R, B)                                                                                                                       \
+    wkv_scan_kernel<T, R, B><<<grid, block, 0, stream>>>((const T*)rkv, ld, k_off, v_off, (const float*)decay, (const float*)bonus, (float*)state, \
+        (size_t)slot_stride, (const int*)slots, (const int*)req_indptr, (float*)out, heads, dim, vdim, vec, (const float*)last_rows, row_width, (size_t)tail_off)
+#define TL_WKV(R)                        \
+    if (tb == 1) TL_WKV_B(R, 1);         \
+    else if (tb == 4) TL_WKV_B(R, 4);    \
+    else TL_WKV_B(R, DELTA_TB)
+    if (rpl == 4) { TL_WKV(4); }
+    else if (rpl == 8) { TL_WKV(8); }
+    else if (rpl == 12) { TL_WKV(12); }
+    else { TL_WKV(16); }
+#undef TL_WKV
+#undef TL_WKV_B
+}
+
+// rkv [tokens, ld]: r of all heads at column 0 (heads * dim), k at k_off, v at v_off (heads * vdim); decay float [tokens, heads * dim]; bonus
+// float [heads * dim]; the state of a head column by column ([vdim][dim]) from head * dim * vdim on in its slot; out float [tokens, heads * vdim].
+extern "C" int tl_wkv_scan(const void* rkv, int ld, int k_off, int v_off, const void* decay, const void* bonus, void* state, long slot_stride,
+                           const void* slots, const void* req_indptr, void* out, int requests, int heads, int dim, int vdim, int longest,
+                           const void* last_rows, int row_width, long tail_off, int dtype, hipStream_t stream) {
+    TL_REQUIRE(requests >= 0 && heads > 0 && dim > 0 && vdim > 0 && ld > 0 && k_off >= 0 && v_off >= 0, "wkv_scan: bad sizes");
+    TL_REQUIRE(dim <= DELTA_L * 16, "wkv_scan: built for up to %d key dimensions per head, got %d", DELTA_L * 16, dim);
+    TL_REQUIRE(slot_stride >= (long)heads * dim * vdim, "wkv_scan: the state rows are too short");
+    TL_REQUIRE(!last_rows || (row_width > 0 && tail_off >= (long)heads * dim * vdim && slot_stride >= tail_off + row_width),
+               "wkv_scan: the slots do not hold a row of %d numbers behind the states", row_width);
+    TL_REQUIRE(requests <= 65535 && heads <= 65535, "wkv_scan: too many requests or heads for one launch");
+    if (requests == 0) return TL_OK;
+    if (dtype == TL_DT_F32) launch_wkv_scan<float>(rkv, ld, k_off, v_off, decay, bonus, state, slot_stride, slots, req_indptr, out, requests, heads, dim, vdim, longest, last_rows, row_width, tail_off, stream);
+    else if (dtype == TL_DT_BF16) launch_wkv_scan<bf16_t>(rkv, ld, k_off, v_off, decay, bonus, state, slot_stride, slots, req_indptr, out, requests, heads, dim, vdim, longest, last_rows, row_width, tail_off, stream);
+    else TL_REQUIRE(false, "wkv_scan: unknown dtype %d", dtype);
+    TL_CHECK_LAUNCH("wkv_scan");
     return TL_OK;
 }

@@ -188,10 +188,11 @@ def bigram_embedding(token_ids: torch.Tensor, table: torch.Tensor, out: torch.Te
 
 
 def sandwich_norm(residual: torch.Tensor, pending: torch.Tensor | None, post_weight: torch.Tensor | None, post_eps: float,
-                  extra: torch.Tensor | None, weight: torch.Tensor, eps: float, out: torch.Tensor, rows: torch.Tensor | None = None,
+                  extra: torch.Tensor | None, weight: torch.Tensor | None, eps: float, out: torch.Tensor, rows: torch.Tensor | None = None,
                   gain: float = 1.0) -> None:
     """``r = residual (+ extra) + (pending / sqrt(mean(pending^2) + post_eps) * post_weight, or pending as it is without a post_weight)``, written
-    back to the float32 residual ``[T, H]`` unless ``rows`` selects rows; ``out = r / sqrt(mean(r^2) + eps) * weight * gain`` in its own dtype.
+    back to the float32 residual ``[T, H]`` unless ``rows`` selects rows; ``out = r / sqrt(mean(r^2) + eps) * weight * gain`` in its own dtype, or
+    (``weight=None``) ``r * gain``, the sum without a norm of its own.
     ``pending``: ``[T, H]`` of ``out``'s dtype or float32 slabs ``[P, T, H]`` that are added up; ``extra``: float32 ``[T, H]``; ``weight`` and
     ``post_weight``: float32, one number or ``H`` of them."""
     T, H = residual.shape
@@ -217,8 +218,46 @@ def sandwich_norm(residual: torch.Tensor, pending: torch.Tensor | None, post_wei
     lib = _lib("elementwise")
     _check(lib, lib.tl_sandwich_norm(_ptr(residual), _ptr(pending), c_int(parts), c_int(T), _ptr(post_weight if pending is not None else None),
                                      c_int(post_weight.numel() if post_weight is not None else 0), c_float(post_eps), _ptr(extra), _ptr(weight),
-                                     c_int(weight.numel()), c_float(eps), c_float(gain), _ptr(out), _ptr(rows), c_int(n), c_int(H),
+                                     c_int(weight.numel() if weight is not None else 0), c_float(eps), c_float(gain), _ptr(out), _ptr(rows), c_int(n), c_int(H),
                                      c_int(_dt(out, "sandwich_norm")), _stream()))
+
+
+def settle_shift(residual: torch.Tensor, pending: torch.Tensor | None, post_weight: torch.Tensor | None, post_eps: float, state: torch.Tensor,
+                 tail_off: int, slots: torch.Tensor, req_indptr: torch.Tensor, token_req: torch.Tensor, mu: torch.Tensor, mixes: torch.Tensor) -> torch.Tensor:
+    """``x = residual + (pending / sqrt(mean(pending^2) + post_eps) * post_weight, or pending as it is without a post_weight)`` row by row,
+    and mixes of neighbouring tokens of a request: ``mixes[s][t] = x[t] + (x[t - 1] - x[t]) * mu[s]``, where the row before the first token that
+    a request brings is ``state[slot, tail_off : tail_off + H]`` (float32).  ``residual`` float32 ``[T, H]``, ``pending`` ``[T, H]`` of the mixes'
+    dtype or float32 slabs ``[P, T, H]``, ``mu`` float32 ``[S, H]``, ``mixes [S, T, H]``.  Returns ``x``: a new float32 tensor, or ``residual`` itself
+    when nothing is pending.  The slots are left as they are."""
+    T, H = residual.shape
+    R = req_indptr.numel() - 1
+    if residual.dtype != torch.float32 or not residual.is_contiguous():
+        raise KernelError("settle_shift: the residual must be contiguous float32")
+    S = mu.shape[0]
+    if mu.dtype != torch.float32 or mu.shape != (S, H) or not mu.is_contiguous() or mixes.shape != (S, T, H) or not mixes.is_contiguous():
+        raise KernelError(f"settle_shift: mu must be float32 [S, {H}] and mixes [S, {T}, {H}], both contiguous")
+    parts = 0
+    if pending is not None:
+        if pending.dim() == 3:
+            parts = pending.shape[0]
+            if pending.dtype != torch.float32 or pending.shape[1:] != residual.shape or not pending.is_contiguous():
+                raise KernelError(f"settle_shift: partial sums {pending.dtype} {tuple(pending.shape)} are not float32 [P, {T}, {H}]")
+        elif pending.shape != residual.shape or pending.dtype != mixes.dtype or not pending.is_contiguous():
+            raise KernelError(f"settle_shift: pending {pending.dtype} {tuple(pending.shape)} does not match the residual and the mixes' dtype")
+    if post_weight is not None and (post_weight.dtype != torch.float32 or not post_weight.is_contiguous() or post_weight.numel() not in (1, H)):
+        raise KernelError(f"settle_shift: post_weight must be float32, one number or {H}")
+    if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 or state.shape[1] < tail_off + H:
+        raise KernelError(f"settle_shift: state {tuple(state.shape)} does not hold the last tokens' rows")
+    _i32(slots, "slots", R)
+    _i32(req_indptr, "req_indptr", R + 1)
+    _i32(token_req, "token_req", T)
+    settled = torch.empty_like(residual) if pending is not None else residual
+    lib = _lib("elementwise")
+    _check(lib, lib.tl_settle_shift(_ptr(residual), _ptr(settled), _ptr(pending), c_int(parts), _ptr(post_weight if pending is not None else None),
+                                    c_int(post_weight.numel() if post_weight is not None else 0), c_float(post_eps), _ptr(state),
+                                    ctypes.c_long(state.stride(0)), ctypes.c_long(tail_off), _ptr(slots), _ptr(req_indptr), _ptr(token_req), _ptr(mu),
+                                    _ptr(mixes), c_int(S), c_int(T), c_int(H), c_int(_dt(mixes, "settle_shift")), _stream()))
+    return settled
 
 
 def normed_sum(x: torch.Tensor, weights: torch.Tensor, eps: float, out: torch.Tensor) -> None:
@@ -351,6 +390,19 @@ def linear(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | None, out
     _check(lib, entry(_ptr(x), _ptr(weight), _ptr(bias), c_int(bf), _ptr(out), c_int(M), c_int(N), c_int(K),
                                     c_int(x.stride(0)), c_int(out.stride(0)), c_int(_dt(x, "linear")),
                                     c_int(1 if out.dtype == torch.float32 else 0), _stream()))
+
+
+def linear_groups(x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor) -> None:
+    """``out[:, g * N : (g + 1) * N] = x[g] @ weight[g].T`` for every group ``g``: ``x [G, T, K]`` and ``weight [G, N, K]`` contiguous and of one dtype,
+    ``out [T, G * N]`` (rows may be strided) of that dtype or float32; one launch where the library has the shape."""
+    G, T, K = x.shape
+    N = weight.shape[1]
+    if weight.shape != (G, N, K) or out.shape != (T, G * N) or x.dtype != weight.dtype or not x.is_contiguous() or not weight.is_contiguous() \
+            or out.stride(1) != 1 or out.dtype not in (x.dtype, torch.float32):
+        raise KernelError(f"linear_groups: x{tuple(x.shape)} weight{tuple(weight.shape)} out{tuple(out.shape)} do not fit")
+    lib = _lib("gemm")
+    _check(lib, lib.tl_gemm_groups(_ptr(x), ctypes.c_long(T * K), _ptr(weight), _ptr(out), ctypes.c_long(N), c_int(G), c_int(T), c_int(N), c_int(K),
+                                   c_int(K), c_int(out.stride(0)), c_int(_dt(x, "linear_groups")), c_int(1 if out.dtype == torch.float32 else 0), _stream()))
 
 
 def linear_f32_variant(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | None, out: torch.Tensor, matrix_cores) -> None:
@@ -1112,6 +1164,55 @@ def silu_float(x: torch.Tensor, out: torch.Tensor) -> None:
     _check(lib, lib.tl_silu_float(_ptr(x), c_int(x.stride(0)), _ptr(out), c_int(x.shape[0]), c_int(x.shape[1]), c_int(_dt(x, "silu_float")), _stream()))
 
 
+# ------------------------------------------------------------- time mixing with decays per key channel
+
+CHANNEL_DECAY_MAX_RANK = 1024
+
+
+def channel_decay(z: torch.Tensor, w2t: torch.Tensor, w0: torch.Tensor, decay: torch.Tensor) -> None:
+    """``decay = exp(-exp(w0 + tanh(z) @ w2t))``: ``z`` float32 ``[T, rank]``, ``w2t`` float32 ``[rank, channels]``, ``w0`` float32 ``[channels]``,
+    ``decay`` float32 ``[T, channels]``."""
+    T, rank = z.shape
+    C = w0.numel()
+    for t, shape, what in ((z, (T, rank), "z"), (w2t, (rank, C), "w2t"), (w0, (C,), "w0"), (decay, (T, C), "decay")):
+        if t.dtype != torch.float32 or t.shape != shape or not t.is_contiguous():
+            raise KernelError(f"channel_decay: {what} must be contiguous float32 {list(shape)}")
+    lib = _lib("recurrent")
+    _check(lib, lib.tl_channel_decay(_ptr(z), _ptr(w2t), _ptr(w0), _ptr(decay), c_int(T), c_int(rank), c_int(C), _stream()))
+
+
+def wkv_scan(rkv: torch.Tensor, k_off: int, v_off: int, decay: torch.Tensor, bonus: torch.Tensor, state: torch.Tensor, slots: torch.Tensor,
+             req_indptr: torch.Tensor, out: torch.Tensor, heads: int, dim: int, vdim: int, max_new_tokens: int | None = None,
+             last_rows: torch.Tensor | None = None, tail_off: int = 0) -> None:
+    """A recurrence with decays per token and key channel and a bonus for the current token, over the step's tokens, request by request from
+    the state its slot holds: ``rkv [T, >=]`` holds per token r at column 0 (``heads * dim``), k at ``k_off`` and v at ``v_off`` (``heads * vdim``);
+    ``decay`` float32 ``[T, heads * dim]``; ``bonus`` float32 ``[heads * dim]``; head ``h`` of ``state[slot]`` (float32, ``dim x vdim`` numbers from ``h *
+    dim * vdim`` on, column by column: ``[vdim][dim]``) gives ``o = (S + diag(bonus) k v^T)^T r`` (to ``out`` float32 ``[T, heads * vdim]``) and moves
+    by ``S <- diag(decay) S + k v^T``.  ``last_rows`` float32 ``[T, H]``: every request's last row goes to ``state[slot, tail_off : tail_off + H]``."""
+    T = rkv.shape[0]
+    R = req_indptr.numel() - 1
+    if rkv.dim() != 2 or rkv.stride(1) != 1 or rkv.shape[1] < max(heads * dim, k_off + heads * dim, v_off + heads * vdim):
+        raise KernelError("wkv_scan: the rows of rkv do not hold r, k and v at the given columns")
+    for t, shape, what in ((decay, (T, heads * dim), "decay"), (bonus, (heads * dim,), "bonus"), (out, (T, heads * vdim), "out")):
+        if t.dtype != torch.float32 or t.shape != shape or not t.is_contiguous():
+            raise KernelError(f"wkv_scan: {what} must be contiguous float32 {list(shape)}")
+    if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 or state.shape[1] < heads * dim * vdim or dim > DELTA_MAX_DIM:
+        raise KernelError(f"wkv_scan: state {tuple(state.shape)} does not hold {heads} states of {dim} x {vdim} (up to {DELTA_MAX_DIM} rows)")
+    width = 0
+    if last_rows is not None:
+        width = last_rows.shape[1]
+        if last_rows.dtype != torch.float32 or last_rows.shape[0] != T or not last_rows.is_contiguous() or tail_off < heads * dim * vdim \
+                or state.shape[1] < tail_off + width:
+            raise KernelError("wkv_scan: the last rows must be contiguous float32 [T, H] with room for one behind the states of a slot")
+    _i32(slots, "slots", R)
+    _i32(req_indptr, "req_indptr", R + 1)
+    lib = _lib("recurrent")
+    _check(lib, lib.tl_wkv_scan(_ptr(rkv), c_int(rkv.stride(0)), c_int(k_off), c_int(v_off), _ptr(decay), _ptr(bonus), _ptr(state),
+                                ctypes.c_long(state.stride(0)), _ptr(slots), _ptr(req_indptr), _ptr(out), c_int(R), c_int(heads), c_int(dim),
+                                c_int(vdim), c_int(max(1, T - R + 1) if max_new_tokens is None else max_new_tokens), _ptr(last_rows), c_int(width),
+                                ctypes.c_long(tail_off), c_int(_dt(rkv, "wkv_scan")), _stream()))
+
+
 # ------------------------------------------------------------- attention with two head sizes, a cap and a local mask
 
 LOCAL_ATTENTION_MAX_DIM = 256
@@ -1157,7 +1258,7 @@ def local_attention_mfma_fits(dtype: torch.dtype, dim: int, vdim: int, page_size
 def local_attention(q: torch.Tensor, out: torch.Tensor, k_plane: torch.Tensor, v_plane: torch.Tensor, block_table: torch.Tensor,
                     token_req: torch.Tensor, positions: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int, page_size: int,
                     scale: float, softcap: float = 0.0, chunk: int = 0, window: int = 0, gain: float = 1.0, tiles=None,
-                    sink: torch.Tensor | None = None, pooled=None, keep_first: int = 0) -> None:
+                    sink: torch.Tensor | None = None, pooled=None, keep_first: int = 0, turn_back=None) -> None:
     """Attention of the step's queries ``q [T, heads * dim]`` over their requests' cached keys and values (which hold the step's own tokens
     already): query head ``i`` reads key/value head ``i // (heads / kv_heads)``; ``score = q . k * scale``, then (``softcap > 0``) ``softcap *
     tanh(score / softcap)``; a query at position ``p`` reads the keys ``j <= p`` with ``j // chunk == p // chunk`` (``chunk > 0``) and ``j > p -
@@ -1167,7 +1268,9 @@ def local_attention(q: torch.Tensor, out: torch.Tensor, k_plane: torch.Tensor, v
     context makes them) runs the matrix-core kernel, where :func:`local_attention_mfma_fits` says it is built.  ``sink`` (float32 ``[heads]``):
     ``exp(sink[head])`` joins the softmax's denominator.  ``pooled = (pk_plane, pv_plane, pool_table, pool)`` (with a window): a query at
     ``p`` also reads the rows ``0 .. (p - window + 1) // pool - 1`` of these planes (laid out like the tokens', with a block table of their own).
-    ``keep_first`` (with a window, without chunks): a query also reads the keys at the positions ``0 .. keep_first - 1``, wherever it stands."""
+    ``keep_first`` (with a window, without chunks): a query also reads the keys at the positions ``0 .. keep_first - 1``, wherever it stands.
+    ``turn_back = (inv_freq, dims, halves)``: the first ``dims`` columns of a head's output at position ``p`` turn by ``-float32(p) * inv_freq[m]``
+    (float32 ``[dims / 2]``), pair ``m`` being ``2m`` and ``2m + 1`` or, ``halves``, ``m`` and ``m + dims / 2``."""
     T = q.shape[0]
     if keep_first < 0 or (keep_first and (window <= 0 or chunk)):
         raise KernelError("local_attention: kept first tokens stand beside a window, without chunks")
@@ -1182,6 +1285,12 @@ def local_attention(q: torch.Tensor, out: torch.Tensor, k_plane: torch.Tensor, v
         if pool <= 0 or window <= 0 or pool_table.dtype != torch.int32 or pool_table.dim() != 2 or pool_table.stride(1) != 1 \
                 or pool_table.shape[0] != block_table.shape[0]:
             raise KernelError("local_attention: pooled blocks need a window, a block size and an int32 block table [requests, blocks]")
+    turn_args = (c_void_p(0), c_int(0), c_int(0))
+    if turn_back is not None:
+        freq, turn_dims, turn_halves = turn_back
+        if turn_dims <= 0 or turn_dims % 2 or turn_dims > vdim or vdim % 2 or freq.dtype != torch.float32 or freq.shape != (turn_dims // 2,) or not freq.is_contiguous():
+            raise KernelError(f"local_attention: an output of {vdim} columns turned over {turn_dims} needs float32 frequencies [{turn_dims // 2}]")
+        turn_args = (_ptr(freq), c_int(turn_dims), c_int(1 if turn_halves else 0))
     pool_args = (_ptr(sink), _ptr(pk_plane), _ptr(pv_plane), _ptr(pool_table), c_int(pool_table.stride(0) if pool else 0))
     if q.shape != (T, heads * dim) or out.shape != (T, heads * vdim) or q.stride(1) != 1 or out.stride(1) != 1 or out.dtype != q.dtype \
             or heads % kv_heads or max(dim, vdim) > LOCAL_ATTENTION_MAX_DIM:
@@ -1205,14 +1314,14 @@ def local_attention(q: torch.Tensor, out: torch.Tensor, k_plane: torch.Tensor, v
                                                  _ptr(req_indptr), _ptr(ctx_lens), _ptr(tile_req), _ptr(tile_tok0), c_int(n_tiles), c_int(heads),
                                                  c_int(kv_heads), c_int(dim), c_int(vdim), c_int(page_size), c_float(scale), c_float(softcap),
                                                  c_int(chunk), c_int(window), c_float(gain), *pool_args, c_int(pool_table.shape[1] if pool else 0),
-                                                 c_int(pool), c_int(keep_first), _stream()))
+                                                 c_int(pool), c_int(keep_first), *turn_args, _stream()))
         return
     _i32(token_req, "token_req", T)
     _i32(positions, "positions", T)
     _check(lib, lib.tl_local_attention(_ptr(q), c_int(q.stride(0)), _ptr(out), c_int(out.stride(0)), _ptr(k_plane), _ptr(v_plane), c_int(k_plane.shape[0]),
                                        _ptr(block_table), c_int(block_table.stride(0)), c_int(block_table.shape[1]), _ptr(token_req), _ptr(positions),
                                        c_int(T), c_int(heads), c_int(kv_heads), c_int(dim), c_int(vdim), c_int(page_size), c_float(scale),
-                                       c_float(softcap), c_int(chunk), c_int(window), c_float(gain), *pool_args, c_int(pool), c_int(keep_first),
+                                       c_float(softcap), c_int(chunk), c_int(window), c_float(gain), *pool_args, c_int(pool), c_int(keep_first), *turn_args,
                                        c_int(_dt(q, "local_attention")), _stream()))
 
 
@@ -1243,17 +1352,22 @@ def pool_blocks(k_plane: torch.Tensor, v_plane: torch.Tensor, block_table: torch
 
 def head_norm_rotate(x: torch.Tensor, heads_a: int, heads_b: int, dim: int, norm_a: torch.Tensor | None, norm_b: torch.Tensor | None, eps: float,
                      positions: torch.Tensor | None, inv_freq: torch.Tensor | None, dims: int, halves: bool,
-                     raw_b: torch.Tensor | None = None) -> None:
+                     raw_b: torch.Tensor | None = None, magnitude: float = 1.0, values=None, pages=None) -> None:
     """In place on ``x [T, (heads_a + heads_b) * dim]`` (a row-strided view: queries, then keys), per token and head, in 32-bit with one rounding:
     a root-mean-square norm over the head's ``dim`` numbers with the weight ``norm_a`` (the first ``heads_a`` heads) or ``norm_b`` (float32
     ``[dim]``; ``None``: no norm), then the rotation of the first ``dims`` numbers by ``float32(position) * inv_freq[i]`` (float32 ``[dims / 2]``;
     ``None``: no rotation), pairing ``2i`` with ``2i + 1`` or, ``halves``, ``i`` with ``i + dims / 2``.  ``raw_b [T, heads_b * dim]`` (of ``x``'s
-    dtype, rows may be strided) receives the last ``heads_b`` heads as they come, before norm and rotation."""
+    dtype, rows may be strided) receives the last ``heads_b`` heads as they come, before norm and rotation.  ``magnitude``: a factor on the cosines
+    and sines of these heads.  ``values = (heads_c, vdim, unit, inv_freq, dims, halves)``: behind those heads ``x`` holds ``heads_c`` of ``vdim`` numbers
+    that are divided by their root mean square (``unit``; the same ``eps``) and turned likewise (``inv_freq=None``: not).  ``pages = (token_req, block_table,
+    k_plane, v_plane, page_size)``: the second heads and the values go to their places in the pages, as :func:`kv_cache_write` puts keys and
+    values there, instead of back to ``x``."""
     T = x.shape[0]
     heads = heads_a + heads_b
+    heads_c, vdim, unit, c_freq, c_dims, c_halves = values if values is not None else (0, 0, False, None, 0, False)
     if raw_b is not None and (raw_b.dtype != x.dtype or raw_b.shape != (T, heads_b * dim) or raw_b.stride(1) != 1):
         raise KernelError(f"head_norm_rotate: the copy of the second heads must be [T, {heads_b * dim}] of {x.dtype}")
-    if x.dim() != 2 or x.stride(1) != 1 or x.shape[1] != heads * dim or dim > LOCAL_ATTENTION_MAX_DIM:
+    if x.dim() != 2 or x.stride(1) != 1 or x.shape[1] != heads * dim + heads_c * vdim or max(dim, vdim) > LOCAL_ATTENTION_MAX_DIM:
         raise KernelError(f"head_norm_rotate: x {tuple(x.shape)} is not [T, {heads} heads of {dim}] (up to {LOCAL_ATTENTION_MAX_DIM} numbers a head)")
     for w in (norm_a, norm_b):
         if w is not None and (w.dtype != torch.float32 or w.shape != (dim,) or not w.is_contiguous()):
@@ -1266,10 +1380,30 @@ def head_norm_rotate(x: torch.Tensor, heads_a: int, heads_b: int, dim: int, norm
         _i32(positions, "positions", T)
         if positions is None:
             raise KernelError("head_norm_rotate: a rotation needs the tokens' positions")
+    if c_freq is not None and (c_dims <= 0 or c_dims % 2 or c_dims > vdim or c_freq.dtype != torch.float32 or c_freq.shape != (c_dims // 2,) or not c_freq.is_contiguous()):
+        raise KernelError(f"head_norm_rotate: a rotation over {c_dims} of {vdim} numbers of a value needs float32 frequencies [{c_dims // 2}]")
+    if c_freq is not None or pages is not None:
+        _i32(positions, "positions", T)
+        if positions is None:
+            raise KernelError("head_norm_rotate: a rotation and the pages need the tokens' positions")
+    page_args = (c_void_p(0), c_void_p(0), c_int(0), c_int(0), c_void_p(0), c_void_p(0), c_int(0), c_int(0))
+    if pages is not None:
+        token_req, block_table, k_plane, v_plane, page_size = pages
+        if heads_c != heads_b or heads_b == 0:
+            raise KernelError("head_norm_rotate: keys and values for the pages come in equal numbers of heads")
+        _check_local_planes("head_norm_rotate", k_plane, v_plane, x.dtype, heads_b, dim, vdim, page_size)
+        _i32(token_req, "token_req", T)
+        if block_table.dtype != torch.int32 or block_table.dim() != 2 or block_table.stride(1) != 1:
+            raise KernelError("head_norm_rotate: the block table must be int32 [requests, blocks]")
+        page_args = (_ptr(token_req), _ptr(block_table), c_int(block_table.stride(0)), c_int(block_table.shape[1]), _ptr(k_plane), _ptr(v_plane),
+                     c_int(k_plane.shape[0]), c_int(page_size))
+    used = positions if inv_freq is not None or c_freq is not None or pages is not None else None
     lib = _lib("local_attention")
     _check(lib, lib.tl_head_norm_rotate(_ptr(x), c_int(x.stride(0)), c_int(T), c_int(heads_a), c_int(heads_b), c_int(dim), _ptr(norm_a), _ptr(norm_b),
-                                        c_float(eps), _ptr(positions if inv_freq is not None else None), _ptr(inv_freq), c_int(dims if inv_freq is not None else 0),
-                                        c_int(1 if halves else 0), _ptr(raw_b), c_int(raw_b.stride(0) if raw_b is not None else 0),
+                                        c_float(eps), _ptr(used), _ptr(inv_freq), c_int(dims if inv_freq is not None else 0),
+                                        c_int(1 if halves else 0), _ptr(raw_b), c_int(raw_b.stride(0) if raw_b is not None else 0), c_float(magnitude),
+                                        c_int(heads_c), c_int(vdim), c_int(1 if unit else 0), _ptr(c_freq), c_int(c_dims if c_freq is not None else 0),
+                                        c_int(1 if c_halves else 0), *page_args,
                                         c_int(_dt(x, "head_norm_rotate")), _stream()))
 
 
@@ -1484,6 +1618,19 @@ def combine(y: torch.Tensor, pair_slot: torch.Tensor, weights: torch.Tensor, out
     lib = _lib("experts")
     _check(lib, lib.tl_combine(_ptr(y), _ptr(pair_slot), _ptr(weights), _ptr(out), _ptr(x), _ptr(offsets), c_int(experts), c_int(T), c_int(top),
                                c_int(W), _ptr(addend), c_int(_dt(out, "combine")), _stream()))
+
+
+def token_gate(z: torch.Tensor, token_ids: torch.Tensor, table: torch.Tensor, out: torch.Tensor, activation: str = "gelu_tanh") -> None:
+    """``out[t] = act(z[t]) * table[token_ids[t]]``: ``z`` float32 ``[T, n]``, ``table [vocab, n]`` a row-strided view (a slice of a token table) and
+    ``out [T, n]`` of one dtype; the product in 32-bit, rounded once."""
+    T, n = z.shape
+    if z.dtype != torch.float32 or not z.is_contiguous() or out.shape != (T, n) or not out.is_contiguous() or table.dim() != 2 or table.shape[1] != n \
+            or table.stride(1) != 1 or table.dtype != out.dtype or ACTIVATIONS[activation] >= 16:
+        raise KernelError("token_gate: shapes or dtypes do not fit")
+    _i32(token_ids, "token_ids", T)
+    lib = _lib("experts")
+    _check(lib, lib.tl_token_gate(_ptr(z), _ptr(token_ids), _ptr(table), c_int(table.stride(0)), c_int(table.shape[0]), _ptr(out), c_int(T), c_int(n),
+                                  c_int(ACTIVATIONS[activation]), c_int(_dt(out, "token_gate")), _stream()))
 
 
 def activation(x: torch.Tensor, kind: str) -> None:

@@ -1,7 +1,7 @@
 """A decoder built from a :class:`~torchlet_amd.config.base.ModelSpec`.
 
 embedding (times ``embed_scale``, plus the position's row of a learned table if the specification names one, plus a hashed bigram row if
-it names one) -> the runs of the layer order (before a run that says so the embedding's output enters the stream again) -> final norm on the wanted rows
+it names one) -> the runs of the layer order (a layer may read its own slice of the tokens' rows in a second table; before a run that says so the embedding's output enters the stream again) -> final norm on the wanted rows
 (times ``logit_scale``) -> LM head (plus its bias, if the specification says it has one)
 (/root/reference/src/torchlet/v10_triton_paged_gqa/model/qwen2_5.py:55-87, where the factors are 1 and
 there is no bias).  The class
@@ -32,6 +32,7 @@ class DecoderModel:
         self.head_bias: torch.Tensor | None = None
         self.position_table: torch.Tensor | None = None
         self.bigram_table: torch.Tensor | None = None
+        self.side_table: torch.Tensor | None = None
         self.keeps_embedding = any(e.add_embedding for e in spec.order)
         self.embed_norm = NORMS.build(spec.embed_norm, dtype, self.device) if spec.embed_norm is not None else None
         if self.embed_norm is not None and (not hasattr(self.embed_norm, "embed") or spec.bigram is not None or spec.position_table_name
@@ -41,6 +42,8 @@ class DecoderModel:
             raise ValueError("a bigram embedding or an embedding that enters the stream again runs over one plain residual")
         if spec.bigram is not None and spec.position_table_name:
             raise ValueError("a bigram embedding beside a learned position table is not built")
+        if (spec.token_side is not None) != any(getattr(b, "side", None) is not None for b in self.blocks):
+            raise ValueError("a model's table of token inputs goes with blocks that read it")
 
     # ------------------------------------------------------------------ weights
     def weight_specs(self) -> dict[str, WeightSpec]:
@@ -50,6 +53,8 @@ class DecoderModel:
             specs[join_name(s.position_table_name, s.weight_suffix)] = WeightSpec((s.max_positions, s.hidden), keep=KEEP_STORED)
         if s.bigram is not None:
             specs[join_name(s.bigram.name, s.weight_suffix)] = WeightSpec((s.bigram.buckets + 1, s.hidden))
+        if s.token_side is not None:
+            specs[join_name(s.token_side.name, s.weight_suffix)] = WeightSpec((s.vocab_size, len(s.layers) * s.token_side.dim))
         for i, block in enumerate(self.blocks):
             for k, v in block.weight_specs().items():
                 specs[join_name(s.layer_name(i), k)] = v
@@ -71,6 +76,12 @@ class DecoderModel:
             self.position_table = place(tensors[join_name(s.position_table_name, s.weight_suffix)], KEEP_STORED, self.dtype, self.device)
         if s.bigram is not None:
             self.bigram_table = place(tensors[join_name(s.bigram.name, s.weight_suffix)], KEEP_COMPUTE, self.dtype, self.device)
+        if s.token_side is not None:
+            n = s.token_side.dim
+            self.side_table = place(tensors[join_name(s.token_side.name, s.weight_suffix)], KEEP_COMPUTE, self.dtype, self.device)
+            for i, block in enumerate(self.blocks):
+                if block.side is not None:
+                    block.side.attach(self.side_table[:, i * n: (i + 1) * n])
         for i, block in enumerate(self.blocks):      # (`tensors` may read from disk on access: each name is touched once)
             block.load_weights(under(tensors, s.layer_name(i)))
         self.final_norm.load_weights(under(tensors, s.final_norm_name))

@@ -80,11 +80,13 @@ class WeightSpec:
     ``init``: the name of a law in :data:`INIT_LAWS` for the random-weights mode (``normal`` =
     N(0, std), ``one_plus_normal`` = 1 + N(0, std), ``random_table`` = integers).
     ``optional``: the checkpoint may leave it out (a tied head).
+    ``free_axes``: axes whose size the checkpoint's tensor decides; ``shape`` holds the random-weights mode's size there.
     """
     shape: tuple[int, ...]
     keep: str = KEEP_COMPUTE
     init: str = "normal"
     optional: bool = False
+    free_axes: tuple[int, ...] = ()
 
     def __post_init__(self):
         if self.keep not in DTYPE_POLICIES:
@@ -95,6 +97,10 @@ class WeightSpec:
     @property
     def integer(self) -> bool:
         return self.keep == KEEP_INT32
+
+    def fits(self, shape: tuple[int, ...]) -> bool:
+        """Whether a stored tensor of this shape is one the part takes."""
+        return len(shape) == len(self.shape) and all(g == w or (i in self.free_axes and g > 0) for i, (g, w) in enumerate(zip(shape, self.shape)))
 
 
 def join_name(prefix: str, name: str) -> str:
@@ -220,7 +226,8 @@ class Stream:
     Blocks that norm a branch's output before it is added leave that norm on the stream as well: ``post = (weight, eps)`` means that
     ``pending`` enters as ``pending / sqrt(mean(pending^2) + eps) * weight`` (32-bit; ``weight`` one number or ``hidden`` of them).
     ``extra``: a 32-bit ``[T, hidden]`` tensor that the next norm adds to the residual too (an embedding that enters the stream again).
-    Only norms that say ``folds_post_norm`` know the two."""
+    Only norms that say ``folds_post_norm`` know the two.  A mixer that says ``reads_stream`` may be handed the stream itself: it reads the
+    32-bit residual with what is pending on it and leaves the stream settled (nothing pending)."""
 
     __slots__ = ("residual", "pending", "normed", "fold", "post", "extra")
 
@@ -287,6 +294,11 @@ class Norm(Part):
     def renorm(self, stream: Stream, alpha: float = 1.0) -> torch.Tensor:
         """The norm after the sum: ``stream.residual <- norm(alpha * residual + pending)`` in 32-bit (the pending branch is
         used up), returned in the activation dtype as well, for the next sublayer to read."""
+        raise NotImplementedError
+
+    def settle(self, stream: Stream) -> torch.Tensor:
+        """Add what is pending (``pending`` with its ``post`` norm, ``extra``) into ``stream.residual`` and return the sum itself, without a norm, in
+        the activation dtype.  Offered by norms that say ``folds_post_norm``."""
         raise NotImplementedError
 
     def lazy(self, stream: Stream) -> "LazyNorm | None":

@@ -13,11 +13,15 @@ A third one keeps several copies of the residual, joined by hyper-connections (:
 
 A fourth one norms a sublayer's output as well as its input (:class:`SandwichBlock`): ``x <- x + post1(mixer(norm1(x)))``, then ``x <- x +
 post2(ffn(norm2(x)))``; the output is left pending with its norm's weight, and the next norm's kernel norms it, adds it and norms the sum.
+
+A fifth one norms the sublayers' outputs only (:class:`OutputNormBlock`): ``x <- x + norm1(mixer(x))``, then ``x <- x + norm2(ffn(x))``, and may add a
+per-layer token input after them.
 """
 from __future__ import annotations
 
 from ..config.base import ConfigError
 from .base import BLOCKS, FEED_FORWARDS, KEEP_FLOAT32, MIXERS, NORMS, Block, Stream, WeightSpec, join_name, under
+from .token_side import TokenSide
 
 
 @BLOCKS.register("prenorm_residual")
@@ -174,4 +178,43 @@ class SandwichBlock(Block):
         if self.ffn is not None:
             h = self.ffn_norm.forward(stream)
             stream.pending, stream.post = self.ffn.forward(h, ctx), (self.ffn_post.weight, self.ffn_post.eps)
+        return stream
+
+
+@BLOCKS.register("output_norm_residual")
+class OutputNormBlock(Block):
+    """Norms on the sublayers' outputs only.  As in :class:`SandwichBlock` a norm is left on the stream beside the pending output; what reads the
+    stream next (the second sublayer, the token input, the next block's mixer, the model's final norm) settles it: one kernel norms the output,
+    adds it in 32-bit and leaves the sum in the activation dtype.  A mixer that says ``reads_stream`` is handed the stream and does this itself."""
+    graph_safe = True
+
+    def __init__(self, spec, dtype, device):
+        super().__init__(spec, dtype, device)
+        self.mixer = MIXERS.build(spec.mixer, dtype, device)
+        self.mixer_norm = NORMS.build(spec.mixer_norm, dtype, device)
+        self.ffn = FEED_FORWARDS.build(spec.ffn, dtype, device) if spec.ffn is not None else None
+        self.ffn_norm = NORMS.build(spec.ffn_norm, dtype, device) if spec.ffn is not None else None
+        self.side = TokenSide(spec.side, dtype, device) if spec.side is not None else None
+        self._children = {spec.mixer_name: self.mixer, spec.mixer_norm_name: self.mixer_norm}
+        if self.ffn is not None:
+            self._children.update({spec.ffn_name: self.ffn, spec.ffn_norm_name: self.ffn_norm})
+        if self.side is not None:
+            self._children[spec.side_name] = self.side
+        for norm in (self.mixer_norm, self.ffn_norm):
+            if norm is not None and not getattr(norm, "folds_post_norm", False):
+                raise ConfigError(f"a block with norms on its sublayers' outputs needs norms that fold a normed branch output; {type(norm).__name__} does not")
+
+    parts = PreNormBlock.parts
+    weight_specs = PreNormBlock.weight_specs
+    load_weights = PreNormBlock.load_weights
+
+    def forward(self, stream: Stream, ctx, cache) -> Stream:
+        h = stream if getattr(self.mixer, "reads_stream", False) else self.mixer_norm.settle(stream)
+        stream.pending, stream.post = self.mixer.forward(h, ctx, cache), (self.mixer_norm.weight, self.mixer_norm.eps)
+        if self.ffn is not None:
+            h = self.mixer_norm.settle(stream)
+            stream.pending, stream.post = self.ffn.forward(h, ctx), (self.ffn_norm.weight, self.ffn_norm.eps)
+        if self.side is not None:
+            h = self.mixer_norm.settle(stream)
+            stream.pending, stream.post = self.side.forward(h, ctx), (self.side.norm, self.side.eps)
         return stream

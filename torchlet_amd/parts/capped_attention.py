@@ -21,6 +21,11 @@ Three more.  Kept first tokens: beside a window a query also reads the first ``k
 positions; the pages that hold them are not given back with the window's.  Values that are the keys: no value projection; the values are
 the keys as projected (bias added) before norm and rotation, copied by the kernel that turns the keys.  Biases on the query and key
 projections and on the output projection.
+
+Three more.  A sink that is no parameter: a fixed number for all heads.  Normed values: divided by their root mean square per head before
+they are cached.  Turned values: a value is cached turned by its own position, and a head's output is turned back by the query's, so that what
+a value contributes depends on how far it lies from the query; the turn back is the last thing the attention kernels do before they store.
+With either of the last two one kernel norms and turns queries, keys and values and puts keys and values into their pages.
 """
 from __future__ import annotations
 
@@ -67,12 +72,26 @@ class CappedAttention(StagedMixer):
         if self.position is not None and (not hasattr(self.position, "halves") or self.position.dims > spec.dim):
             raise ConfigError(f"attention: the encoding {spec.position.kind!r} is not one over the first dimensions of a head of {spec.dim}")
         self.qk_norm = bool(spec.qk_norm)
+        self.value_norm = bool(spec.value_norm)
+        self.value_position = POSITION_ENCODINGS.build(spec.value_position, dtype, device) if spec.value_position is not None else None
+        if self.value_position is not None and (not hasattr(self.value_position, "halves") or self.value_position.dims > spec.vdim or spec.vdim % 2
+                                                or self.value_position.magnitude != 1.0):
+            raise ConfigError(f"attention: the encoding {spec.value_position.kind!r} is not a plain one over the first dimensions of a value of {spec.vdim}")
+        self.own_values = self.value_norm or self.value_position is not None       # values that are not cached as projected
+        if self.own_values and (self.shared_kv or self.pool):
+            raise ConfigError("attention: normed or turned values beside values that are the keys, or beside pooled blocks, are not built")
+        if spec.sink and spec.fixed_sink is not None:
+            raise ConfigError("attention: a sink is either learned or fixed")
         self.q_norm = self.k_norm = self.sink = None
+        if spec.fixed_sink is not None:
+            self.sink = torch.full((spec.heads,), float(spec.fixed_sink), dtype=torch.float32, device=device)
 
     def parts(self):
         yield self
         if self.position is not None:
             yield from self.position.parts()
+        if self.value_position is not None:
+            yield from self.value_position.parts()
 
     def paged_need(self):
         planes = ((self.kv_heads, self.dim), (self.kv_heads, self.vdim))
@@ -127,29 +146,39 @@ class CappedAttention(StagedMixer):
             values = torch.empty((proj.shape[0], self.k_width), dtype=self.dtype, device=proj.device)
         else:
             values = proj[:, self.q_width + self.k_width:]
-        if self.qk_norm or self.position is not None or self.shared_kv:
+        turn = self.position
+        rotation = (turn.inv_freq, turn.dims, bool(turn.halves)) if turn is not None else (None, 0, False)
+        magnitude = turn.magnitude if turn is not None else 1.0
+        turned = self.value_position
+        turn_values = (turned.inv_freq, turned.dims, bool(turned.halves)) if turned is not None else None
+        if self.own_values:
+            # queries, keys and values normed and turned by one kernel, which puts keys and values into their pages as well
+            width = self.q_width + (self.k_width + self.v_width if cache.writable else 0)
+            kv = self.kv_heads if cache.writable else 0
+            ops.head_norm_rotate(proj[:, : width], self.heads, kv, self.dim, self.q_norm, self.k_norm, float(self.spec.qk_norm_eps), ctx.positions,
+                                 *rotation, magnitude=magnitude,
+                                 values=(kv, self.vdim, self.value_norm, *(turn_values or (None, 0, False))) if kv else None,
+                                 pages=(ctx.token_req, table, k_plane, v_plane, cache.page_size) if kv else None)
+        elif self.qk_norm or self.position is not None or self.shared_kv:
             # queries and keys lie side by side in the projection's rows: normed per head and turned in place, in 32-bit, with one rounding
             ops.head_norm_rotate(proj[:, : self.q_width + self.k_width], self.heads, self.kv_heads, self.dim, self.q_norm, self.k_norm,
-                                 float(self.spec.qk_norm_eps), ctx.positions,
-                                 self.position.inv_freq if self.position is not None else None,
-                                 self.position.dims if self.position is not None else 0,
-                                 bool(self.position.halves) if self.position is not None else False,
+                                 float(self.spec.qk_norm_eps), ctx.positions, *rotation, magnitude=magnitude,
                                  raw_b=values if self.shared_kv else None)
         pooled = None
         if self.pool:
             pool_group, (pk_plane, pv_plane) = cache.more[0]
             pv_plane = pv_plane.view(pv_plane.shape[0], self.kv_heads, self.vdim, cache.page_size)
             pooled = (pk_plane, pv_plane, ctx.block_tables[pool_group], self.pool)
-        if cache.writable:
+        if cache.writable and not self.own_values:
             ops.kv_cache_write(proj[:, self.q_width: self.q_width + self.k_width], values,
                                ctx.token_req, ctx.positions, table, k_plane, v_plane, cache.page_size)
-            if pooled is not None:      # the blocks whose last token this step brings
-                ops.pool_blocks(k_plane, v_plane, table, pk_plane, pv_plane, pooled[2], ctx.req_indptr, ctx.ctx_lens,
-                                ctx.max_new_tokens // self.pool + 1, cache.page_size, self.pool)
+        if cache.writable and pooled is not None:      # the blocks whose last token this step brings
+            ops.pool_blocks(k_plane, v_plane, table, pk_plane, pv_plane, pooled[2], ctx.req_indptr, ctx.ctx_lens,
+                            ctx.max_new_tokens // self.pool + 1, cache.page_size, self.pool)
         tiles = None
         if h.is_cuda and ops.local_attention_mfma_fits(self.dtype, self.dim, self.vdim, cache.page_size) \
                 and proj.stride(0) % 8 == 0 and proj.data_ptr() % 16 == 0:
             tiles = (ctx.req_indptr, ctx.ctx_lens, *ctx.tiles(ops.LOCAL_ATTENTION_TILE_TOKENS))
         ops.local_attention(q, out, k_plane, v_plane, table, ctx.token_req, ctx.positions, self.heads, self.kv_heads, self.dim, self.vdim,
                             cache.page_size, self.scale, self.softcap, self.chunk, self.window, gain, tiles=tiles, sink=self.sink, pooled=pooled,
-                            keep_first=self.keep_first)
+                            keep_first=self.keep_first, turn_back=turn_values)

@@ -48,6 +48,8 @@ class LatentAttention(Mixer):
         self.position = POSITION_ENCODINGS.build(spec.position, dtype, device) if spec.position is not None else None
         if self.position is not None and not hasattr(self.position, "inv_freq"):
             raise ConfigError("latent attention folds a rotation in pairs into its kernels; its position encoding must offer inv_freq")
+        if self.position is not None and getattr(self.position, "magnitude", 1.0) != 1.0:
+            raise ConfigError("latent attention folds a plain rotation into its kernels; a magnitude on cosine and sine is not built there")
         # tiles of 64 rows where the matrix-core kernel is built for these sizes, of 16 for the general kernel
         on_matrix_cores = torch.device(device).type == "cuda" and ops.latent_attention_mfma_fits(dtype, self.heads, self.rank, self.rot)
         self.tile_tokens = ops.latent_tile_tokens(self.heads, ops.LATENT_MFMA_ROWS if on_matrix_cores else ops.LATENT_ATTENTION_ROWS)

@@ -31,6 +31,20 @@ def _no_post_norm(stream: Stream, kind: str) -> None:
         raise ValueError(f"a {kind} does not fold a normed branch output or a second addend into the stream; a norm that says folds_post_norm does")
 
 
+def _settle(stream: Stream, dtype: torch.dtype) -> torch.Tensor:
+    """What is pending enters the residual; the sum itself in the activation dtype (a 32-bit engine's residual is that already)."""
+    if stream.residual.dim() != 2 or stream.fold is not None:
+        raise ValueError("a stream is settled over one plain residual")
+    nothing = stream.pending is None and stream.extra is None
+    if nothing and dtype == stream.residual.dtype:
+        return stream.residual
+    out = torch.empty(stream.residual.shape, dtype=dtype, device=stream.residual.device)
+    post_w, post_eps = stream.post if stream.post is not None else (None, 0.0)
+    ops.sandwich_norm(stream.residual, stream.pending, post_w, post_eps, stream.extra, None, 0.0, out)
+    stream.pending = stream.post = stream.extra = None
+    return out
+
+
 @NORMS.register("rmsnorm")
 class RMSNorm(Norm):
     graph_safe = True
@@ -133,6 +147,9 @@ class ScalarRMSNorm(Norm):
             stream.pending = stream.post = stream.extra = None
         return out
 
+    def settle(self, stream: Stream) -> torch.Tensor:
+        return _settle(stream, self.dtype)
+
 
 @NORMS.register("offset_rmsnorm")
 class OffsetRMSNorm(Norm):
@@ -165,6 +182,9 @@ class OffsetRMSNorm(Norm):
         if rows is None:
             stream.pending = stream.post = stream.extra = None
         return out
+
+    def settle(self, stream: Stream) -> torch.Tensor:
+        return _settle(stream, self.dtype)
 
     def embed(self, token_ids: torch.Tensor, table: torch.Tensor, out: torch.Tensor, scale: float = 1.0) -> None:
         """``out[t] = norm(table[token_ids[t]] * scale)``: the embedding's rows normed on their way into the 32-bit stream, one kernel."""

@@ -8,6 +8,8 @@ inside the kernel, so no table of ``max_positions`` rows is kept.
 """
 from __future__ import annotations
 
+import math
+
 import torch
 
 from ..config.base import ConfigError
@@ -46,7 +48,8 @@ class PairRotaryEncoding(PositionEncoding):
     """The interleaved layout: of the first ``dims`` entries of a vector, entry ``2i`` is paired with ``2i + 1`` and the pair
     ``(u, v)`` at position ``p`` becomes ``(u cos a - v sin a, v cos a + u sin a)`` with ``a = float32(p) * f_i``,
     ``f_i = base**(-2i / dims)`` (taken in 64-bit on the host, then rounded once to 32-bit); entries beyond ``dims`` pass
-    unchanged.  Mixers fold the rotation into their own kernels through :attr:`inv_freq`; :meth:`apply` turns whole heads."""
+    unchanged.  Mixers fold the rotation into their own kernels through :attr:`inv_freq` and :attr:`magnitude` (a factor on cosine and sine);
+    :meth:`apply` turns whole heads."""
     graph_safe = True
 
     def __init__(self, spec, dtype, device):
@@ -56,7 +59,11 @@ class PairRotaryEncoding(PositionEncoding):
         self.dims = spec.dims
         self.halves = False
         i = torch.arange(spec.dims // 2, dtype=torch.float64)
-        self.inv_freq = (float(spec.base) ** (-2.0 * i / spec.dims) / float(getattr(spec, "factor", 1.0))).to(torch.float32).to(device)
+        freq = float(spec.base) ** (-2.0 * i / spec.dims) / float(getattr(spec, "factor", 1.0))
+        self.magnitude = 1.0
+        if getattr(spec, "yarn", None) is not None:
+            freq, self.magnitude = stretch_by_turns(freq, spec.dims, float(spec.base), *(float(y) for y in spec.yarn))
+        self.inv_freq = freq.to(torch.float32).to(device)
 
     def apply(self, q, k, positions):
         for x in (q, k):
@@ -64,6 +71,9 @@ class PairRotaryEncoding(PositionEncoding):
                 continue
             T, heads, hd = x.shape
             flat = x.as_strided((T, heads * hd), (x.stride(0), 1))
+            if self.magnitude != 1.0:
+                ops.head_norm_rotate(flat, heads, 0, hd, None, None, 0.0, positions, self.inv_freq, self.dims, False, magnitude=self.magnitude)
+                continue
             ops.rotate_pairs(flat, hd, 0, flat, hd, 0, positions, self.inv_freq, heads, hd)
 
 
@@ -77,6 +87,18 @@ def scale_by_wavelength(freq: torch.Tensor, factor: float, low: float, high: flo
     s = (original / wavelength - low) / (high - low)
     blended = (1.0 - s) * freq / factor + s * freq
     return torch.where(wavelength < original / high, freq, torch.where(wavelength > original / low, freq / factor, blended))
+
+
+def stretch_by_turns(freq: torch.Tensor, dims: int, base: float, factor: float, original: float, fast: float, slow: float) -> tuple[torch.Tensor, float]:
+    """YaRN: frequencies (64-bit, pair ``i`` of ``dims / 2``) blended between themselves and themselves over ``factor``, ``f (1 - r_i) + f / factor r_i``,
+    and the magnitude ``0.1 ln(factor) + 1`` of cosine and sine.  ``r_i`` rises linearly from 0 at the pair that turns ``fast`` times over
+    ``original`` positions (rounded down) to 1 at the pair that turns ``slow`` times (rounded up)."""
+    if not (factor > 0 and original > 0 and fast > 0 and slow > 0 and base > 1):
+        raise ConfigError(f"rotary encoding: YaRN wants base > 1 and positive factor, original, fast and slow, got {(base, factor, original, fast, slow)}")
+    pair_of = lambda turns: dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+    lo, hi = max(math.floor(pair_of(fast)), 0), min(math.ceil(pair_of(slow)), dims - 1)
+    ramp = ((torch.arange(dims // 2, dtype=torch.float64) - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    return freq / factor * ramp + freq * (1.0 - ramp), 0.1 * math.log(factor) + 1.0
 
 
 @POSITION_ENCODINGS.register("rope_halves")
@@ -99,6 +121,9 @@ class HalfRotaryEncoding(PositionEncoding):
         freq = float(spec.base) ** (-2.0 * i / spec.dims) / float(spec.factor)
         if spec.bands is not None:
             freq = scale_by_wavelength(freq, *(float(b) for b in spec.bands))
+        self.magnitude = 1.0
+        if spec.yarn is not None:
+            freq, self.magnitude = stretch_by_turns(freq, spec.dims, float(spec.base), *(float(y) for y in spec.yarn))
         self.inv_freq = freq.to(torch.float32).to(device)
 
     def apply(self, q, k, positions):
@@ -107,4 +132,4 @@ class HalfRotaryEncoding(PositionEncoding):
                 continue
             T, heads, hd = x.shape
             flat = x.as_strided((T, heads * hd), (x.stride(0), 1))
-            ops.head_norm_rotate(flat, heads, 0, hd, None, None, 0.0, positions, self.inv_freq, self.dims, True)
+            ops.head_norm_rotate(flat, heads, 0, hd, None, None, 0.0, positions, self.inv_freq, self.dims, True, magnitude=self.magnitude)

@@ -103,8 +103,8 @@ def check_against(specs: dict[str, WeightSpec], source) -> None:
     for n, s in specs.items():
         if n in source:
             got = shape_of(n)
-            if got != tuple(s.shape):
-                wrong.append(f"{n}: stored {list(got)}, model wants {list(s.shape)}")
+            if not s.fits(got):
+                wrong.append(f"{n}: stored {list(got)}, model wants {['any' if i in s.free_axes else d for i, d in enumerate(s.shape)]}")
             elif not kind_ok(n, s):
                 wrong.append(f"{n}: stored element type does not fit {'an integer table' if s.integer else 'a floating-point tensor'}")
     if missing or unexpected or wrong:

@@ -49,6 +49,6 @@ def cpu_ops(monkeypatch):
                  "latent_attention", "heads_linear", "experts_linear", "route", "combine", "activation", "compute_units",
                  "streams_norm", "delta_prepare", "delta_scan", "kv_cache_write", "local_attention", "local_attention_mfma_fits",
                  "pool_blocks", "head_norm_rotate", "decay_scan", "silu_float", "bigram_embedding", "sandwich_norm", "normed_sum",
-                 "selective_prepare", "selective_scan", "embedding_norm"):
+                 "selective_prepare", "selective_scan", "embedding_norm", "settle_shift", "linear_groups", "channel_decay", "wkv_scan", "token_gate"):
         monkeypatch.setattr(ops, name, getattr(emulated_ops, name))
     return ops

@@ -373,7 +373,7 @@ def local_attention_mfma_fits(dtype, dim, vdim, page_size):
 
 
 def local_attention(q, out, k_plane, v_plane, block_table, token_req, positions, heads, kv_heads, dim, vdim, page_size, scale,
-                    softcap=0.0, chunk=0, window=0, gain=1.0, tiles=None, sink=None, pooled=None, keep_first=0):
+                    softcap=0.0, chunk=0, window=0, gain=1.0, tiles=None, sink=None, pooled=None, keep_first=0, turn_back=None):
     group = heads // kv_heads
     for t in range(q.shape[0]):
         p, r = int(positions[t]), int(token_req[t])
@@ -399,7 +399,10 @@ def local_attention(q, out, k_plane, v_plane, block_table, token_req, positions,
             w = torch.softmax(torch.cat((s, sink.float()[:, None]), -1), -1)[:, :-1]
         else:
             w = torch.softmax(s, -1)
-        out[t] = (torch.einsum("hn,nhd->hd", w, v).reshape(-1) * gain).to(out.dtype)
+        o = torch.einsum("hn,nhd->hd", w, v)[None]
+        if turn_back is not None:
+            _turn_heads(o, positions[t: t + 1], *turn_back, sign=-1.0)
+        out[t] = (o.reshape(-1) * gain).to(out.dtype)
 
 
 def pool_blocks(k_plane, v_plane, block_table, pk_plane, pv_plane, pool_table, req_indptr, ctx_lens, most_blocks, page_size, pool):
@@ -416,25 +419,43 @@ def pool_blocks(k_plane, v_plane, block_table, pk_plane, pv_plane, pool_table, r
             pv_plane[ppage, :, :, b % page_size] = v_plane[pages, :, :, keys % page_size].float().mean(0).to(pv_plane.dtype)
 
 
-def head_norm_rotate(x, heads_a, heads_b, dim, norm_a, norm_b, eps, positions, inv_freq, dims, halves, raw_b=None):
+def _turn_heads(v, positions, inv_freq, dims, halves, magnitude=1.0, sign=1.0):
+    """v [T, heads, n] float, in place: the first ``dims`` numbers of every head turned by ``sign * position * inv_freq``."""
+    ang = sign * positions.float()[:, None, None] * inv_freq.float()[None, None, :]
+    c, sn = ang.cos() * magnitude, ang.sin() * magnitude
+    if halves:
+        a, b = v[..., : dims // 2].clone(), v[..., dims // 2: dims].clone()
+        v[..., : dims // 2], v[..., dims // 2: dims] = a * c - b * sn, b * c + a * sn
+    else:
+        a, b = v[..., 0:dims:2].clone(), v[..., 1:dims:2].clone()
+        v[..., 0:dims:2], v[..., 1:dims:2] = a * c - b * sn, b * c + a * sn
+
+
+def head_norm_rotate(x, heads_a, heads_b, dim, norm_a, norm_b, eps, positions, inv_freq, dims, halves, raw_b=None, magnitude=1.0, values=None, pages=None):
     T = x.shape[0]
+    width = (heads_a + heads_b) * dim
     if raw_b is not None:
-        raw_b.copy_(x[:, heads_a * dim:])
-    v = x.float().reshape(T, heads_a + heads_b, dim).clone()
+        raw_b.copy_(x[:, heads_a * dim: width])
+    v = x[:, :width].float().reshape(T, heads_a + heads_b, dim).clone()
     if norm_a is not None or norm_b is not None:
         w = torch.cat([(norm_a if norm_a is not None else torch.ones(dim)).float().expand(heads_a, dim),
                        (norm_b if norm_b is not None else torch.ones(dim)).float().expand(heads_b, dim)])
         v = v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps) * w
     if inv_freq is not None:
-        ang = positions.float()[:, None, None] * inv_freq.float()[None, None, :]
-        c, sn = ang.cos(), ang.sin()
-        if halves:
-            a, b = v[..., : dims // 2].clone(), v[..., dims // 2: dims].clone()
-            v[..., : dims // 2], v[..., dims // 2: dims] = a * c - b * sn, b * c + a * sn
-        else:
-            a, b = v[..., 0:dims:2].clone(), v[..., 1:dims:2].clone()
-            v[..., 0:dims:2], v[..., 1:dims:2] = a * c - b * sn, b * c + a * sn
-    x.copy_(v.reshape(T, -1).to(x.dtype))
+        _turn_heads(v, positions, inv_freq, dims, halves, magnitude)
+    x[:, :width] = v.reshape(T, -1).to(x.dtype)
+    if values is None:
+        return
+    heads_c, vdim, unit, c_freq, c_dims, c_halves = values
+    c = x[:, width:].float().reshape(T, heads_c, vdim).clone()
+    if unit:
+        c = c / torch.sqrt(c.pow(2).mean(-1, keepdim=True) + eps)
+    if c_freq is not None:
+        _turn_heads(c, positions, c_freq, c_dims, c_halves)
+    x[:, width:] = c.reshape(T, -1).to(x.dtype)
+    if pages is not None:
+        token_req, block_table, k_plane, v_plane, page_size = pages
+        kv_cache_write(x[:, heads_a * dim: width], x[:, width:], token_req, positions, block_table, k_plane, v_plane, page_size)
 
 
 def decay_scan(qkv, decay, state, slots, req_indptr, out, heads, dim, vdim, max_new_tokens=None):
@@ -490,7 +511,60 @@ def sandwich_norm(residual, pending, post_weight, post_eps, extra, weight, eps, 
             r = residual
         else:
             r = r + add
-    out.copy_((r / torch.sqrt(r.pow(2).mean(-1, keepdim=True) + eps) * gain * weight.float()).to(out.dtype))
+    if weight is None:
+        out.copy_((r * gain).to(out.dtype))
+    else:
+        out.copy_((r / torch.sqrt(r.pow(2).mean(-1, keepdim=True) + eps) * gain * weight.float()).to(out.dtype))
+
+
+def settle_shift(residual, pending, post_weight, post_eps, state, tail_off, slots, req_indptr, token_req, mu, mixes):
+    x = residual
+    H = residual.shape[1]
+    if pending is not None:
+        y = pending.sum(0) if pending.dim() == 3 else pending.float()
+        if post_weight is not None:
+            y = y / torch.sqrt(y.pow(2).mean(-1, keepdim=True) + post_eps) * post_weight.float()
+        x = residual + y
+    before = torch.empty_like(x)
+    for t in range(x.shape[0]):
+        r = int(token_req[t])
+        before[t] = x[t - 1] if t > int(req_indptr[r]) else state[int(slots[r]), tail_off: tail_off + H]
+    mixes.copy_((x[None] + (before - x)[None] * mu[:, None, :]).to(mixes.dtype))
+    return x
+
+
+def linear_groups(x, weight, out):
+    N = weight.shape[1]
+    for g in range(weight.shape[0]):
+        out[:, g * N: (g + 1) * N] = (x[g].float() @ weight[g].float().T).to(out.dtype)
+
+
+def channel_decay(z, w2t, w0, decay):
+    decay.copy_(torch.exp(-torch.exp(w0 + torch.tanh(z) @ w2t)))
+
+
+def wkv_scan(rkv, k_off, v_off, decay, bonus, state, slots, req_indptr, out, heads, dim, vdim, max_new_tokens=None, last_rows=None, tail_off=0):
+    u = bonus.view(heads, dim)
+    for r in range(req_indptr.numel() - 1):
+        first, last = int(req_indptr[r]), int(req_indptr[r + 1])
+        if last <= first:
+            continue
+        st = state[int(slots[r])]
+        S = st[: heads * dim * vdim].view(heads, vdim, dim).transpose(1, 2).clone()
+        for t in range(first, last):
+            q = rkv[t, : heads * dim].float().view(heads, dim)
+            k = rkv[t, k_off: k_off + heads * dim].float().view(heads, dim)
+            v = rkv[t, v_off: v_off + heads * vdim].float().view(heads, vdim)
+            kv = k[:, :, None] * v[:, None, :]
+            out[t] = torch.einsum("hde,hd->he", S + u[:, :, None] * kv, q).reshape(-1)
+            S = decay[t].view(heads, dim)[:, :, None] * S + kv
+        st[: heads * dim * vdim] = S.transpose(1, 2).reshape(-1)
+        if last_rows is not None:
+            st[tail_off: tail_off + last_rows.shape[1]] = last_rows[last - 1]
+
+
+def token_gate(z, token_ids, table, out, activation="gelu_tanh"):
+    out.copy_((_act(z, activation) * table[token_ids.long()].float()).to(out.dtype))
 
 
 def normed_sum(x, weights, eps, out):

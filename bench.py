@@ -3,7 +3,7 @@
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch B] [--layers L] [--dtype bfloat16]
                     [--shape 7b|14b|32b] [--context N] [--new-tokens G] [--prefill-tokens T]
-                    [--workload decode|serve|migurax|nebutar|fotovik|bafulorn] [--only decode|step|prefill] [--all]
+                    [--workload decode|serve|migurax|nebutar|fotovik|bafulorn|vabelorn] [--only decode|step|prefill] [--all]
 
 The default run has the layer sizes of Qwen2.5-7B (28 layers, hidden 3584, 28 heads, 4 KV heads, head
 size 128, intermediate 18944, vocabulary 152064) with random weights and goes through the whole engine
@@ -55,6 +55,12 @@ attention over a cached latent in a window with a gate; grouped-query attention 
 first tokens; a selective state-space recurrence; gated dense feed-forwards and experts routed by sigmoid scores with a shared expert),
 beside the Migurax model of the same width and layer count (the closest one the framework has: latent attention, a recurrent state per
 request, routed experts), and the kernels it added or changed beside their like.
+
+``--workload vabelorn [--size s|m]`` does the same for the Vabelorn design (norms on the sublayers' outputs only; time mixing with a matrix
+state and decays per token and key channel; grouped-query attention with normed queries and keys, values cached turned by their position,
+one added to the softmax's denominator; gated dense feed-forwards; a per-layer token input), beside the Fotovik model of the same width and
+layer count (the closest one the framework has: the same attention kernels, recurrences with a matrix state, normed sublayer outputs, dense
+feed-forwards), and the kernels it added or changed beside their like.
 """
 from __future__ import annotations
 
@@ -97,8 +103,8 @@ def parse_args(argv=None):
     p.add_argument("--context", type=int, default=CONTEXT, help="prompt tokens of each request in the decode runs")
     p.add_argument("--new-tokens", type=int, default=None, help="tokens each request may generate (decode: 256, serve: 128)")
     p.add_argument("--prefill-tokens", type=int, default=2048)
-    p.add_argument("--workload", choices=["decode", "serve", "migurax", "nebutar", "fotovik", "bafulorn"], default="decode")
-    p.add_argument("--size", choices=["s", "m"], default="s", help="migurax, nebutar, fotovik, bafulorn: layer sizes (s: width 2048, m: width 4096)")
+    p.add_argument("--workload", choices=["decode", "serve", "migurax", "nebutar", "fotovik", "bafulorn", "vabelorn"], default="decode")
+    p.add_argument("--size", choices=["s", "m"], default="s", help="migurax, nebutar, fotovik, bafulorn, vabelorn: layer sizes (s: width 2048, m: width 4096)")
     p.add_argument("--requests", type=int, default=32)
     p.add_argument("--prompt-min", type=int, default=128)
     p.add_argument("--prompt-max", type=int, default=4096)
@@ -1308,6 +1314,151 @@ def bafulorn(args) -> dict:
     return out
 
 
+# ---------------------------------------------------------------------------------------------- the Vabelorn design
+
+def vabelorn_sizes(size: str) -> dict:
+    """A Vabelorn configuration of four layers at the width of the other designs' sizes: time mixing with heads of 64 x 64 over the width and
+    decays through 64 numbers; causal attention with heads of 128 + 128 in groups of four, half a head rotated with stretched frequencies; both
+    twice, each with a gated dense feed-forward; token inputs of 256 numbers a layer."""
+    width, heads, ff = dict(s=(2048, 16, 5632), m=(4096, 32, 11264))[size]
+    wkv = dict(heads=width // 64, dim=64, decay_rank=64)
+    attention = dict(heads=heads, kv_heads=heads // 4, dim=128, vdim=128, scale=128 ** -0.5,
+                     rot=dict(dims=64, base=500000.0, scaling=dict(factor=8.0, original=4096, fast=32.0, slow=1.0)))
+    dense = dict(kind="dense", ff=ff)
+    return dict(architecture="Vabelorn", vocab=32000, width=width, max_positions=8192, norm=dict(eps=1e-6), logit_scale=0.5, token_side=dict(dim=256),
+                layers=[dict(type=t, mixer=m, mlp=dense) for t, m in (("wkv", wkv), ("attention", attention)) * 2])
+
+
+def vabelorn_kernels(ours: dict, like: dict, batch: int, context: int, tokens: int) -> list[dict]:
+    """Each kernel that the design added or changed, alone, at the sizes of ``ours``, in a decode step of ``batch`` requests on ``context`` cached
+    tokens and in a prompt of ``tokens`` tokens, beside the like kernel of the closest path the framework had.  ``frac``: bytes that must
+    move / time against 8 TB/s, or operations / time against the matrix cores' bfloat16 rate (against the 32-bit rate for the recurrences)."""
+    import torch
+    from torchlet_amd.kernels import ops
+    dev, bf = "cuda", torch.bfloat16
+    rows = []
+
+    def add(name, kind, launch, nbytes=0.0, flops=0.0, peak=MFMA_PEAK_TFLOPS["bfloat16"]):
+        ms = _best_ms(launch, rounds=3, calls=5)
+        row = {"kernel": name, "like": kind, "ms": round(ms, 4)}
+        if nbytes:
+            row.update(bytes=int(nbytes), frac=round(nbytes / (ms * 1e-3) / 1e9 / HBM_PEAK_GBS, 4), bound="hbm")
+        else:
+            row.update(flops=flops, frac=round(flops / (ms * 1e-3) / (peak * 1e12), 4), bound="flops")
+        rows.append(row)
+        say(f"  {name}: {ms:.4f} ms, {row['frac']} of its bound")
+
+    def tables(n_req, total):
+        blocks = -(-total // PAGE)
+        table = (torch.arange(n_req * blocks, dtype=torch.int32, device=dev) + 1).view(n_req, blocks)
+        return table, n_req * blocks + 1
+
+    def one_request(T, reqs):
+        return (torch.arange(reqs, dtype=torch.int32, device=dev), torch.arange(reqs + 1, dtype=torch.int32, device=dev) * (T // reqs),
+                torch.arange(T, dtype=torch.int32, device=dev) // (T // reqs))
+
+    width = ours["width"]
+    wkv, att = ours["layers"][0]["mixer"], ours["layers"][1]["mixer"]
+    h, d, rank, side = wkv["heads"], wkv["dim"], wkv["decay_rank"], ours["token_side"]["dim"]
+    K = h * d
+    # ---- the recurrence beside the linear attention with fixed decays, states of the same size: a decode step reads and writes every state
+    #      once; a prompt does 4 operations per state element and token either way (the decay, the update, one sum over the rows)
+    for kind, T, reqs in (("decode", batch, batch), (f"prompt {tokens}", tokens, 1)):
+        slots, indptr, token_req = one_request(T, reqs)
+        rkv = (torch.randn(T, 4 * K, device=dev) * 0.3).to(bf)
+        decay, bonus = torch.rand(T, K, device=dev) * 0.5 + 0.5, torch.randn(K, device=dev)
+        state = torch.zeros(reqs + 1, K * d + width, device=dev)
+        out, x = torch.empty(T, K, device=dev), torch.randn(T, width, device=dev)
+        launch = lambda: ops.wkv_scan(rkv, K, 2 * K, decay, bonus, state, slots, indptr, out, h, d, d, max_new_tokens=T // reqs, last_rows=x, tail_off=K * d)
+        qkv, fixed = torch.randn(T, 3 * K, device=dev) * 0.1, torch.rand(h, device=dev)
+        launch2 = lambda: ops.decay_scan(qkv, fixed, state, slots, indptr, out, h, d, d, max_new_tokens=T // reqs)
+        how = dict(nbytes=2.0 * reqs * K * d * 4) if reqs > 1 else dict(flops=4.0 * T * K * d, peak=MFMA_PEAK_TFLOPS["float32"])
+        add(f"wkv_scan {kind}", f"decay_scan {kind}", launch, **how)
+        add(f"decay_scan {kind} (states of the same size)", "", launch2, **how)
+        # ---- the sum and the five mixes (residual read and written, output read, mixes written) beside the norm that adds and norms
+        res, pen, wv = torch.randn(T, width, device=dev), torch.randn(T, width, device=dev).to(bf), torch.ones(width, device=dev)
+        mu, mixes, act = torch.rand(5, width, device=dev), torch.empty(5, T, width, dtype=bf, device=dev), torch.empty(T, width, dtype=bf, device=dev)
+        add(f"settle_shift {kind}", f"sandwich_norm {kind}", lambda: ops.settle_shift(res, pen, wv, 1e-6, state, K * d, slots, indptr, token_req, mu, mixes),
+            nbytes=float(T) * width * (4 + 4 + 2 + 10))
+        add(f"sandwich_norm {kind}, without a norm of the sum", f"sandwich_norm {kind}", lambda: ops.sandwich_norm(res, pen, wv, 1e-6, None, None, 0.0, act), nbytes=float(T) * width * 12)
+        add(f"sandwich_norm {kind} (Fotovik path)", "", lambda: ops.sandwich_norm(res, pen, wv, 1e-6, None, wv, 1e-6, act), nbytes=float(T) * width * 12)
+        # ---- the four products of four mixes beside one product as large
+        w4 = (torch.randn(4, K, width, device=dev) * 0.02).to(bf)
+        how = dict(nbytes=4.0 * K * width * 2) if reqs > 1 else dict(flops=8.0 * T * K * width)
+        add(f"linear_groups {kind}, four of {K} x {width}", f"linear {kind}", lambda: ops.linear_groups(mixes[:4], w4, rkv), **how)
+        add(f"linear {kind}, {4 * K} x {width}", "", lambda: ops.linear(act, w4.view(4 * K, width), None, rkv), **how)
+        # ---- the decays: their inner products read, the decays written in 32-bit (a decode step reads the matrix), beside the delta rule's
+        #      preparation, which writes as many 32-bit channels; the gated norm per head is the delta rule's
+        z, w2t, w0 = torch.randn(T, rank, device=dev), torch.randn(rank, K, device=dev), torch.zeros(K, device=dev)
+        add(f"channel_decay {kind}", f"delta_prepare {kind}", lambda: ops.channel_decay(z, w2t, w0, decay), nbytes=float(T) * (K + rank) * 4 + rank * K * 4)
+        dh = h // 2                                         # a delta rule with as many channels: queries, keys and values of h / 2 heads and h / 4 key heads
+        gates, conv_w, a_log = torch.randn(T, 2 * dh, device=dev), torch.randn(K, 4, device=dev) * 0.3, torch.zeros(dh, device=dev)
+        prep, dstate = torch.empty(T, K, device=dev), torch.zeros(reqs + 1, 3 * K, device=dev)
+        add(f"delta_prepare {kind} (as many channels)", "", lambda: ops.delta_prepare(rkv, conv_w, gates, a_log, a_log, dstate, 0, slots, indptr, token_req, prep, dh, dh // 2, d, d, 4,
+                                                                                      1.0, 1e-6), nbytes=float(T) * K * 6)
+        # ---- the token input's gate
+        zg, ids, table, gg = torch.randn(T, side, device=dev), torch.randint(0, ours["vocab"], (T,), dtype=torch.int32, device=dev), torch.randn(ours["vocab"], 4 * side, device=dev).to(bf), torch.empty(T, side, dtype=bf, device=dev)
+        add(f"token_gate {kind}", f"silu_float {kind}", lambda: ops.token_gate(zg, ids, table[:, side: 2 * side], gg), nbytes=float(T) * side * 8)
+        sf = torch.empty(T, side, device=dev)
+        add(f"silu_float {kind} (as many numbers)", "", lambda: ops.silu_float(gg, sf), nbytes=float(T) * side * 6)
+        # ---- norm and rotation of queries, keys and values straight into the pages, beside the rotation and the cache write of the Fotovik path
+        H, G, dk = att["heads"], att["kv_heads"], att["dim"]
+        ctx = context - 1 if reqs > 1 else 0
+        total = ctx + T // reqs
+        tab, pages = tables(reqs, total)
+        k_plane, v_plane = (torch.randn(pages, G, PAGE, dk, device=dev) * 0.3).to(bf), (torch.randn(pages, G, dk, PAGE, device=dev) * 0.3).to(bf)
+        qkvp = torch.randn(T, (H + 2 * G) * dk, device=dev).to(bf)
+        wq, inv, inv_v = torch.ones(dk, device=dev), torch.rand(32, device=dev), torch.rand(dk // 2, device=dev)
+        positions = (torch.arange(T, dtype=torch.int32, device=dev) % (T // reqs)) + ctx
+        add(f"head_norm_rotate {kind}, values too, into the pages", f"head_norm_rotate + kv_cache_write {kind}",
+            lambda: ops.head_norm_rotate(qkvp, H, G, dk, wq, wq, 1e-6, positions, inv, 64, False, magnitude=1.2, values=(G, dk, True, inv_v, dk, False),
+                                         pages=(token_req, tab, k_plane, v_plane, PAGE)), nbytes=float(T) * (H + 2 * G) * dk * 4)
+
+        def two_kernels():
+            ops.head_norm_rotate(qkvp[:, : (H + G) * dk], H, G, dk, wq, wq, 1e-6, positions, inv, 64, False)
+            ops.kv_cache_write(qkvp[:, H * dk: (H + G) * dk], qkvp[:, (H + G) * dk:], token_req, positions, tab, k_plane, v_plane, PAGE)
+        add(f"head_norm_rotate + kv_cache_write {kind} (Fotovik path)", "", two_kernels, nbytes=float(T) * ((H + G) * dk * 4 + 2 * G * dk * 4))
+        # ---- the attention with its output turned back, beside the plain causal one
+        q, o = (torch.randn(T, H * dk, device=dev) * 0.3).to(bf), torch.empty(T, H * dk, dtype=bf, device=dev)
+        if reqs == 1:
+            n_tiles = -(-T // ops.LOCAL_ATTENTION_TILE_TOKENS)
+            tiles = (indptr, torch.zeros(1, dtype=torch.int32, device=dev), torch.zeros(n_tiles, dtype=torch.int32, device=dev),
+                     torch.arange(n_tiles, dtype=torch.int32, device=dev) * ops.LOCAL_ATTENTION_TILE_TOKENS, n_tiles)
+        else:
+            tiles = (indptr, torch.full((reqs,), ctx, dtype=torch.int32, device=dev), None, None, reqs)
+        sink = torch.zeros(H, device=dev)
+        how = dict(nbytes=float(reqs) * (ctx + 1) * G * 2 * dk * 2) if reqs > 1 else dict(flops=4.0 * H * dk * T * (T + 1) / 2)
+        add(f"local_attention {kind}, one added, output turned back", f"local_attention {kind}", lambda: ops.local_attention(
+            q, o, k_plane, v_plane, tab, token_req, positions, H, G, dk, dk, PAGE, att["scale"], tiles=tiles, sink=sink, turn_back=(inv_v, dk, False)), **how)
+        add(f"local_attention {kind} (causal, Fotovik path)", "", lambda: ops.local_attention(
+            q, o, k_plane, v_plane, tab, token_req, positions, H, G, dk, dk, PAGE, att["scale"], tiles=tiles), **how)
+    return rows
+
+
+def vabelorn(args) -> dict:
+    import torch
+    ours, like = vabelorn_sizes(args.size), fotovik_sizes(args.size)
+    out = {"metric": f"Vabelorn design, size {args.size} (width {ours['width']}, 4 layers), prefill of {args.prefill_tokens} tokens and decode at batch "
+                     f"{args.batch} on {args.context}-token caches, beside the Fotovik design at equal width and layer count, one MI355X",
+           "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
+           "data": "synthetic: seeded random weights, token ids and cache contents", "config": {"vabelorn": ours, "fotovik": like}}
+    for key, d in (("vabelorn", ours), ("fotovik", like)):
+        say(f"building the {key} model")
+        cfg, model = _build_from(d, args.dtype)
+        pms, pbest = time_prefill(model, args.prefill_tokens)
+        dms = _decode_ms(model, args.batch, min(args.steps, 64), args.warmup, args.context)
+        out[key] = {"weight_bytes": _weight_bytes(model),
+                    "prefill": {"tokens": args.prefill_tokens, "ms": round(pms, 3), "ms_best": round(pbest, 3), "tokens_per_s": round(args.prefill_tokens * 1e3 / pms, 1)},
+                    "decode": {"batch": args.batch, "context": args.context, "ms_per_step": round(dms, 4), "tokens_per_s": round(args.batch * 1e3 / dms, 1)}}
+        say(f"{key}: {out[key]}")
+        del model
+        torch.cuda.empty_cache()
+    out["value"] = out["vabelorn"]["decode"]["tokens_per_s"]
+    if args.dtype == "bfloat16" and not args.no_points:
+        out["kernels"] = vabelorn_kernels(ours, like, args.batch, args.context, args.prefill_tokens)
+    return out
+
+
 def main(argv=None) -> int:
     args = parse_args(argv)
     args.serve_new_tokens = args.new_tokens or 128
@@ -1330,6 +1481,9 @@ def main(argv=None) -> int:
         return 0
     if args.workload == "bafulorn":
         print(json.dumps(bafulorn(args)))
+        return 0
+    if args.workload == "vabelorn":
+        print(json.dumps(vabelorn(args)))
         return 0
     name, sizes = SHAPES[args.shape]
     full_layers = sizes["num_hidden_layers"]

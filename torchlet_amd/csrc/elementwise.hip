@@ -739,6 +739,102 @@ extern "C" int tl_bigram_embedding(const void* ids, const void* table, void* out
     return TL_OK;
 }
 
+// ------------------------------------------------------------------ rows in pieces of four numbers
+__device__ __forceinline__ float4 load4(const float* p) { return *(const float4*)p; }
+__device__ __forceinline__ float4 load4(const bf16_t* p) {
+    const uint2 t = *(const uint2*)p;
+    return make_float4(__uint_as_float(t.x << 16), __uint_as_float(t.x & 0xffff0000u), __uint_as_float(t.y << 16), __uint_as_float(t.y & 0xffff0000u));
+}
+__device__ __forceinline__ void store4(float* p, float4 v) { *(float4*)p = v; }
+__device__ __forceinline__ void store4(bf16_t* p, float4 v) {
+    uint2 t;
+    t.x = (uint32_t)from_float<bf16_t>(v.x).bits | ((uint32_t)from_float<bf16_t>(v.y).bits << 16);
+    t.y = (uint32_t)from_float<bf16_t>(v.z).bits | ((uint32_t)from_float<bf16_t>(v.w).bits << 16);
+    *(uint2*)p = t;
+}
+// Up to four neighbouring numbers: all four at once where rows are multiples of four (VEC 4), one otherwise.
+template <int VEC, typename T> __device__ __forceinline__ void load_piece(const T* p, float (&v)[VEC]) {
+    if constexpr (VEC == 4) { const float4 f = load4(p); v[0] = f.x; v[1] = f.y; v[2] = f.z; v[3] = f.w; }
+    else v[0] = to_float(p[0]);
+}
+template <int VEC, typename T> __device__ __forceinline__ void store_piece(T* p, const float (&v)[VEC]) {
+    if constexpr (VEC == 4) store4(p, make_float4(v[0], v[1], v[2], v[3]));
+    else p[0] = from_float<T>(v[0]);
+}
+
+// A row of `hidden` numbers (a multiple of four) held by a work-group in registers: piece n of a thread is the four numbers from
+// 4 (thread + n * threads) on.  All fetches of a row are requested before the first is used.
+template <int NP> struct RowPieces {
+    float v[NP][4];
+};
+template <int NP, typename T>
+__device__ __forceinline__ void load_row(const T* p, int hidden, RowPieces<NP>& r) {
+#pragma unroll
+    for (int n = 0; n < NP; ++n) {
+        const int i = 4 * (threadIdx.x + n * blockDim.x);
+        if (i < hidden) load_piece<4>(p + i, r.v[n]);
+        else { r.v[n][0] = r.v[n][1] = r.v[n][2] = r.v[n][3] = 0.f; }
+    }
+}
+template <int NP, typename T>
+__device__ __forceinline__ void store_row(T* p, int hidden, const RowPieces<NP>& r) {
+#pragma unroll
+    for (int n = 0; n < NP; ++n) {
+        const int i = 4 * (threadIdx.x + n * blockDim.x);
+        if (i < hidden) store_piece<4>(p + i, r.v[n]);
+    }
+}
+// A branch's output: one row of the activation type, or the sum of `parts` float slabs (four requested at a time, added in their order).
+template <int NP, typename T>
+__device__ __forceinline__ void load_branch(const void* pending, int parts, size_t part_stride, size_t row_off, int hidden, RowPieces<NP>& y) {
+    if (parts == 0) { load_row<NP>((const T*)pending + row_off, hidden, y); return; }
+    const float* slab = (const float*)pending + row_off;
+#pragma unroll
+    for (int n = 0; n < NP; ++n) {
+        const int i = 4 * (threadIdx.x + n * blockDim.x);
+#pragma unroll
+        for (int v = 0; v < 4; ++v) y.v[n][v] = 0.f;
+        if (i >= hidden) continue;
+        for (int p = 0; p < parts; p += 4) {
+            float z[4][4];
+#pragma unroll
+            for (int u = 0; u < 4; ++u) load_piece<4>(slab + (size_t)min(p + u, parts - 1) * part_stride + i, z[u]);
+#pragma unroll
+            for (int u = 0; u < 4; ++u)
+                if (p + u < parts) {
+#pragma unroll
+                    for (int v = 0; v < 4; ++v) y.v[n][v] += z[u][v];
+                }
+        }
+    }
+}
+template <int NP>
+__device__ __forceinline__ float row_squares(const RowPieces<NP>& r) {
+    float ss = 0.f;
+#pragma unroll
+    for (int n = 0; n < NP; ++n)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) ss = fmaf(r.v[n][v], r.v[n][v], ss);
+    return ss;
+}
+// The weights of a norm: a vector, or one number for all coordinates.
+template <int NP>
+__device__ __forceinline__ void load_weights(const float* w, int count, int hidden, RowPieces<NP>& r) {
+    if (count != 1) { load_row<NP>(w, hidden, r); return; }
+    const float one = w[0];
+#pragma unroll
+    for (int n = 0; n < NP; ++n)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) r.v[n][v] = one;
+}
+// Threads and pieces per thread for a row: up to 1024 threads, then up to three pieces each (12288 numbers).
+struct RowPlan { int threads, pieces; };
+static RowPlan plan_row(int hidden) {
+    const int n = hidden / 4;
+    const int threads = n <= 64 ? 64 : n <= 128 ? 128 : n <= 256 ? 256 : n <= 512 ? 512 : 1024;
+    return RowPlan{threads, (n + threads - 1) / threads};
+}
+
 // ------------------------------------------------------------------ norm of the branch output, addition, norm of the sum
 // One block per output row, the row kept in shared memory between the passes:
 //   y = pending[row] (one tensor of the activation type, or `parts` float slabs added up);
@@ -790,6 +886,40 @@ __global__ void sandwich_norm_kernel(float* __restrict__ residual, const void* _
     for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = from_float<T>(sn_row[i] * inv * weight[weight_n == 1 ? 0 : i]);
 }
 
+// The same with the row in registers (hidden a multiple of four, aligned rows): what the residual, the weights and the branch's slabs hold is
+// requested at once, so a decode step's few rows pay one trip to memory.
+template <typename T, int NP>
+__global__ void __launch_bounds__(1024)
+sandwich_norm_rows_kernel(float* __restrict__ residual, const void* __restrict__ pending, int parts, size_t part_stride,
+                          const float* __restrict__ post, int post_n, float post_eps, const float* __restrict__ extra,
+                          const float* __restrict__ weight, int weight_n, float eps, float gain, T* __restrict__ out,
+                          const int* __restrict__ rows, int hidden) {
+    __shared__ float red[16];
+    const int srow = rows ? rows[blockIdx.x] : blockIdx.x;
+    const size_t at = (size_t)srow * hidden;
+    RowPieces<NP> r, y, pw, w, ex;
+    load_row<NP>(residual + at, hidden, r);
+    if (pending) load_branch<NP, T>(pending, parts, part_stride, at, hidden, y);
+    if (pending && post) load_weights<NP>(post, post_n, hidden, pw);
+    if (extra) load_row<NP>(extra + at, hidden, ex);
+    if (weight) load_weights<NP>(weight, weight_n, hidden, w);
+    const float inv_y = pending && post ? rsqrtf(block_sum(row_squares(y), red) / (float)hidden + post_eps) : 1.f;
+#pragma unroll
+    for (int n = 0; n < NP; ++n)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            if (extra) r.v[n][v] += ex.v[n][v];
+            if (pending) r.v[n][v] += post ? y.v[n][v] * inv_y * pw.v[n][v] : y.v[n][v];
+        }
+    if ((pending || extra) && !rows) store_row<NP>(residual + at, hidden, r);
+    const float inv = weight ? rsqrtf(block_sum(row_squares(r), red) / (float)hidden + eps) * gain : gain;
+#pragma unroll
+    for (int n = 0; n < NP; ++n)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) r.v[n][v] = weight ? r.v[n][v] * inv * w.v[n][v] : r.v[n][v] * inv;
+    store_row<NP>(out + (size_t)blockIdx.x * hidden, hidden, r);
+}
+
 extern "C" int tl_sandwich_norm(void* residual, const void* pending, int parts, int part_rows, const void* post, int post_n, float post_eps,
                                 const void* extra, const void* weight, int weight_n, float eps, float gain, void* out, const void* rows,
                                 int out_rows, int hidden, int act_dtype, hipStream_t stream) {
@@ -797,6 +927,20 @@ extern "C" int tl_sandwich_norm(void* residual, const void* pending, int parts, 
     TL_REQUIRE((!weight || weight_n == 1 || weight_n == hidden) && (!post || post_n == 1 || post_n == hidden), "sandwich_norm: weights of one number or of %d", hidden);
     if (out_rows == 0) return TL_OK;
     const size_t part_stride = (size_t)part_rows * hidden, smem = sizeof(float) * hidden;
+    TL_REQUIRE(act_dtype == TL_DT_F32 || act_dtype == TL_DT_BF16, "sandwich_norm: unknown dtype %d", act_dtype);
+    const uintptr_t bits = (uintptr_t)residual | (uintptr_t)pending | (uintptr_t)post | (uintptr_t)extra | (uintptr_t)weight | (uintptr_t)out;
+    if (hidden % 4 == 0 && bits % 16 == 0) {
+        const RowPlan plan = plan_row(hidden);
+#define TL_SN(T, N)                                                                                                                               \
+    sandwich_norm_rows_kernel<T, N><<<out_rows, plan.threads, 0, stream>>>((float*)residual, pending, parts, part_stride, (const float*)post, post_n, post_eps, \
+        (const float*)extra, (const float*)weight, weight_n, eps, gain, (T*)out, (const int*)rows, hidden)
+#define TL_SN_T(T) if (plan.pieces == 1) TL_SN(T, 1); else if (plan.pieces == 2) TL_SN(T, 2); else TL_SN(T, 3)
+        if (act_dtype == TL_DT_F32) { TL_SN_T(float); } else { TL_SN_T(bf16_t); }
+#undef TL_SN_T
+#undef TL_SN
+        TL_CHECK_LAUNCH("sandwich_norm");
+        return TL_OK;
+    }
     const int threads = hidden >= 2048 ? 512 : 256;
     if (act_dtype == TL_DT_F32)
         sandwich_norm_kernel<float><<<out_rows, threads, smem, stream>>>((float*)residual, pending, parts, part_stride, (const float*)post, post_n, post_eps,
@@ -884,105 +1028,115 @@ extern "C" int tl_embedding_norm(const void* ids, const void* table, int table_d
 // float slabs added up; null: x_t = residual[t]), written to `settled` (another place than the residual: a work-group also reads the row
 // before its own first one).  Then, with x' the token before's (of the request's slot, `tail`, for the first token that a request brings),
 //   mixes[s][t][i] = x_t[i] + (x'[i] - x_t[i]) * mu[s][i],   s < count.
-// A work-group takes `run` neighbouring tokens, row after row, and makes the row before the first of them a second time; a row's numbers
-// stay with the threads that made them, so the rows in shared memory need no barrier of their own.  All in float, one rounding of the mixes.
-__device__ __forceinline__ float4 load4(const float* p) { return *(const float4*)p; }
-__device__ __forceinline__ float4 load4(const bf16_t* p) {
-    const uint2 t = *(const uint2*)p;
-    return make_float4(__uint_as_float(t.x << 16), __uint_as_float(t.x & 0xffff0000u), __uint_as_float(t.y << 16), __uint_as_float(t.y & 0xffff0000u));
-}
-__device__ __forceinline__ void store4(float* p, float4 v) { *(float4*)p = v; }
-__device__ __forceinline__ void store4(bf16_t* p, float4 v) {
-    uint2 t;
-    t.x = (uint32_t)from_float<bf16_t>(v.x).bits | ((uint32_t)from_float<bf16_t>(v.y).bits << 16);
-    t.y = (uint32_t)from_float<bf16_t>(v.z).bits | ((uint32_t)from_float<bf16_t>(v.w).bits << 16);
-    *(uint2*)p = t;
-}
-// Up to four neighbouring numbers: all four at once where rows are multiples of four (VEC 4), one otherwise.
-template <int VEC, typename T> __device__ __forceinline__ void load_piece(const T* p, float (&v)[VEC]) {
-    if constexpr (VEC == 4) { const float4 f = load4(p); v[0] = f.x; v[1] = f.y; v[2] = f.z; v[3] = f.w; }
-    else v[0] = to_float(p[0]);
-}
-template <int VEC, typename T> __device__ __forceinline__ void store_piece(T* p, const float (&v)[VEC]) {
-    if constexpr (VEC == 4) store4(p, make_float4(v[0], v[1], v[2], v[3]));
-    else p[0] = from_float<T>(v[0]);
+// A work-group takes `run` neighbouring tokens, row after row, and makes the row before the first of them a second time.  All in float, one
+// rounding of the mixes.  Rows of a multiple of four numbers are held in registers; others in shared memory, where a row's numbers stay with
+// the threads that made them, so that they need no barrier of their own.
+struct ShiftArgs {
+    const float* residual;
+    float* settled;
+    const void* pending;
+    int parts;
+    size_t part_stride;
+    const float* post;
+    int post_n;
+    float post_eps;
+    const float* state;            // the slots: the row of the token before at slot * slot_stride + tail_off
+    size_t slot_stride, tail_off;
+    const int *slots, *req_indptr, *token_req;
+    const float* mu;
+    int count, tokens, hidden, run;
+};
+
+template <typename T, int NP>
+__global__ void __launch_bounds__(1024)
+settle_shift_rows_kernel(ShiftArgs a, T* __restrict__ mixes) {
+    __shared__ float red[16];
+    const int first = blockIdx.x * a.run, last = min(first + a.run, a.tokens) - 1, hidden = a.hidden;
+    RowPieces<NP> pw;
+    if (a.pending && a.post) load_weights<NP>(a.post, a.post_n, hidden, pw);
+    auto settle = [&](int t, RowPieces<NP>& r) {
+        const size_t at = (size_t)t * hidden;
+        load_row<NP>(a.residual + at, hidden, r);
+        if (!a.pending) return;
+        RowPieces<NP> y;
+        load_branch<NP, T>(a.pending, a.parts, a.part_stride, at, hidden, y);
+        const float inv = a.post ? rsqrtf(block_sum(row_squares(y), red) / (float)hidden + a.post_eps) : 1.f;
+#pragma unroll
+        for (int n = 0; n < NP; ++n)
+#pragma unroll
+            for (int v = 0; v < 4; ++v) r.v[n][v] += a.post ? y.v[n][v] * inv * pw.v[n][v] : y.v[n][v];
+    };
+    RowPieces<NP> before, x;
+    bool have = false;                                 // `before` holds the row ahead of the one at hand
+    for (int t = first; t <= last; ++t) {
+        const int req = a.token_req[t];
+        if (t == a.req_indptr[req]) {                  // the request's first token of the step: its slot has the row before (anywhere in memory)
+            const float* tail = a.state + (size_t)a.slots[req] * a.slot_stride + a.tail_off;
+#pragma unroll
+            for (int n = 0; n < NP; ++n)
+#pragma unroll
+                for (int v = 0; v < 4; ++v) {
+                    const int i = 4 * (threadIdx.x + n * blockDim.x) + v;
+                    before.v[n][v] = i < hidden ? tail[i] : 0.f;
+                }
+        } else if (!have) settle(t - 1, before);
+        settle(t, x);
+        if (a.pending) store_row<NP>(a.settled + (size_t)t * hidden, hidden, x);
+        for (int s = 0; s < a.count; ++s) {
+            RowPieces<NP> m;
+            load_row<NP>(a.mu + (size_t)s * hidden, hidden, m);
+#pragma unroll
+            for (int n = 0; n < NP; ++n)
+#pragma unroll
+                for (int v = 0; v < 4; ++v) m.v[n][v] = fmaf(before.v[n][v] - x.v[n][v], m.v[n][v], x.v[n][v]);
+            store_row<NP>(mixes + ((size_t)s * a.tokens + t) * hidden, hidden, m);
+        }
+        before = x;
+        have = true;
+    }
 }
 
-template <typename T, int VEC>
+template <typename T>
 __global__ void __launch_bounds__(256)
-settle_shift_kernel(const float* __restrict__ residual, float* __restrict__ settled, const void* __restrict__ pending, int parts, size_t part_stride,
-                    const float* __restrict__ post, int post_n, float post_eps, const float* __restrict__ state, size_t slot_stride, size_t tail_off,
-                    const int* __restrict__ slots, const int* __restrict__ req_indptr, const int* __restrict__ token_req,
-                    const float* __restrict__ mu, T* __restrict__ mixes, int count, int tokens, int hidden, int run) {
-    extern __shared__ __attribute__((aligned(16))) float ss_rows[];       // two rows
+settle_shift_kernel(ShiftArgs a, T* __restrict__ mixes) {
+    extern __shared__ float ss_rows[];                 // two rows
     __shared__ float red[16];
-    const int first = blockIdx.x * run, last = min(first + run, tokens) - 1;
-    const int step = blockDim.x * VEC;
-    // the settled row t into `buf` (each thread its own pieces)
+    const int first = blockIdx.x * a.run, last = min(first + a.run, a.tokens) - 1, hidden = a.hidden;
     auto settle = [&](int t, float* buf) {
-        const float* res = residual + (size_t)t * hidden;
+        const size_t at = (size_t)t * hidden;
         float inv = 1.f;
-        if (pending) {
+        if (a.pending) {
             float ss = 0.f;
-            for (int i = threadIdx.x * VEC; i < hidden; i += step) {
-                float y[VEC];
-                if (parts == 0) load_piece<VEC>((const T*)pending + (size_t)t * hidden + i, y);
-                else {
-                    load_piece<VEC>((const float*)pending + (size_t)t * hidden + i, y);
-                    for (int p = 1; p < parts; ++p) {
-                        float z[VEC];
-                        load_piece<VEC>((const float*)pending + p * part_stride + (size_t)t * hidden + i, z);
-#pragma unroll
-                        for (int v = 0; v < VEC; ++v) y[v] += z[v];
-                    }
-                }
-#pragma unroll
-                for (int v = 0; v < VEC; ++v) ss = fmaf(y[v], y[v], ss);
-                store_piece<VEC>(buf + i, y);
+            for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
+                float y = 0.f;
+                if (a.parts == 0) y = to_float(((const T*)a.pending)[at + i]);
+                for (int p = 0; p < a.parts; ++p) y += ((const float*)a.pending)[p * a.part_stride + at + i];
+                ss = fmaf(y, y, ss);
+                buf[i] = y;
             }
-            if (post) inv = rsqrtf(block_sum(ss, red) / (float)hidden + post_eps);
+            if (a.post) inv = rsqrtf(block_sum(ss, red) / (float)hidden + a.post_eps);
         }
-        for (int i = threadIdx.x * VEC; i < hidden; i += step) {
-            float r[VEC];
-            load_piece<VEC>(res + i, r);
-            if (pending) {
-                float y[VEC], w[VEC];
-                load_piece<VEC>(buf + i, y);
-                if (post) {
-                    if (post_n == 1) {
-#pragma unroll
-                        for (int v = 0; v < VEC; ++v) w[v] = post[0];
-                    } else load_piece<VEC>(post + i, w);
-                }
-#pragma unroll
-                for (int v = 0; v < VEC; ++v) r[v] += post ? y[v] * inv * w[v] : y[v];
-            }
-            store_piece<VEC>(buf + i, r);
+        for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
+            float r = a.residual[at + i];
+            if (a.pending) r += a.post ? buf[i] * inv * a.post[a.post_n == 1 ? 0 : i] : buf[i];
+            buf[i] = r;
         }
     };
     float *cur = ss_rows, *before = ss_rows + hidden;
-    if (first > req_indptr[token_req[first]]) settle(first - 1, before);
+    bool have = false;
     for (int t = first; t <= last; ++t) {
-        const int req = token_req[t];
-        const float* tail = t == req_indptr[req] ? state + (size_t)slots[req] * slot_stride + tail_off : nullptr;
+        const int req = a.token_req[t];
+        const float* tail = t == a.req_indptr[req] ? a.state + (size_t)a.slots[req] * a.slot_stride + a.tail_off : nullptr;
+        if (!tail && !have) settle(t - 1, before);
         settle(t, cur);
-        for (int i = threadIdx.x * VEC; i < hidden; i += step) {
-            float x[VEC], b[VEC];
-            load_piece<VEC>(cur + i, x);
-            if (tail) {
-#pragma unroll
-                for (int v = 0; v < VEC; ++v) b[v] = tail[i + v];          // (a slot's tail may start anywhere)
-            } else load_piece<VEC>(before + i, b);
-            if (pending) store_piece<VEC>(settled + (size_t)t * hidden + i, x);
-            for (int s = 0; s < count; ++s) {
-                float m[VEC];
-                load_piece<VEC>(mu + (size_t)s * hidden + i, m);
-#pragma unroll
-                for (int v = 0; v < VEC; ++v) m[v] = fmaf(b[v] - x[v], m[v], x[v]);
-                store_piece<VEC>(mixes + ((size_t)s * tokens + t) * hidden + i, m);
-            }
+        for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
+            const float x = cur[i], b = tail ? tail[i] : before[i];
+            if (a.pending) a.settled[(size_t)t * hidden + i] = x;
+            for (int s = 0; s < a.count; ++s)
+                mixes[((size_t)s * a.tokens + t) * hidden + i] = from_float<T>(fmaf(b - x, a.mu[(size_t)s * hidden + i], x));
         }
         float* other = cur; cur = before; before = other;
+        have = true;
     }
 }
 
@@ -993,28 +1147,27 @@ extern "C" int tl_settle_shift(const void* residual, void* settled, const void* 
     TL_REQUIRE(!post || post_n == 1 || post_n == hidden, "settle_shift: a norm weight of one number or of %d", hidden);
     TL_REQUIRE(!pending || settled != residual, "settle_shift: the sum goes to another place than the residual it is made from");
     TL_REQUIRE(tail_off >= 0 && slot_stride >= tail_off + hidden, "settle_shift: the slots do not hold a row of %d numbers", hidden);
+    TL_REQUIRE(hidden % 4 == 0 || hidden <= 8000, "settle_shift: rows of a multiple of four numbers, or of up to 8000, not %d", hidden);
     TL_REQUIRE(act_dtype == TL_DT_F32 || act_dtype == TL_DT_BF16, "settle_shift: unknown dtype %d", act_dtype);
     if (tokens == 0) return TL_OK;
     const int run = tokens >= 2048 ? 4 : (tokens >= 768 ? 2 : 1);
-    const size_t smem = sizeof(float) * 2 * hidden, part_stride = (size_t)tokens * hidden;
-    const bool vec = hidden % 4 == 0;
+    const ShiftArgs a{(const float*)residual, (float*)settled, pending, parts, (size_t)tokens * hidden, (const float*)post, post_n, post_eps,
+                      (const float*)state, (size_t)slot_stride, (size_t)tail_off, (const int*)slots, (const int*)req_indptr, (const int*)token_req,
+                      (const float*)mu, count, tokens, hidden, run};
     const int grid = (tokens + run - 1) / run;
-#define TL_SS(T, V)                                                                                                                              \
-    {                                                                                                                                            \
-        auto kernel = settle_shift_kernel<T, V>;                                                                                                 \
-        static bool raised = false;                                                                                                              \
-        if (smem > 48 * 1024 && !raised) {                                                                                                       \
-            hipError_t e = hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 96 * 1024 + 64);                 \
-            if (e != hipSuccess) { tl_set_error("settle_shift: cannot get %zu bytes of shared memory: %s", smem, hipGetErrorString(e)); return TL_ERR_HIP; } \
-            raised = true;                                                                                                                       \
-        }                                                                                                                                        \
-        kernel<<<grid, 256, smem, stream>>>((const float*)residual, (float*)settled, pending, parts, part_stride, (const float*)post, post_n, post_eps, \
-            (const float*)state, (size_t)slot_stride, (size_t)tail_off, (const int*)slots, (const int*)req_indptr, (const int*)token_req,        \
-            (const float*)mu, (T*)mixes, count, tokens, hidden, run);                                                                            \
-    }
-    if (act_dtype == TL_DT_F32) { if (vec) TL_SS(float, 4) else TL_SS(float, 1) }
-    else { if (vec) TL_SS(bf16_t, 4) else TL_SS(bf16_t, 1) }
+    const uintptr_t bits = (uintptr_t)residual | (uintptr_t)settled | (uintptr_t)pending | (uintptr_t)post | (uintptr_t)mu | (uintptr_t)mixes;
+    if (hidden % 4 == 0 && bits % 16 == 0) {
+        const RowPlan plan = plan_row(hidden);
+#define TL_SS(T, N) settle_shift_rows_kernel<T, N><<<grid, plan.threads, 0, stream>>>(a, (T*)mixes)
+#define TL_SS_T(T) if (plan.pieces == 1) TL_SS(T, 1); else if (plan.pieces == 2) TL_SS(T, 2); else TL_SS(T, 3)
+        if (act_dtype == TL_DT_F32) { TL_SS_T(float); } else { TL_SS_T(bf16_t); }
+#undef TL_SS_T
 #undef TL_SS
+    } else {
+        const size_t smem = sizeof(float) * 2 * hidden;
+        if (act_dtype == TL_DT_F32) settle_shift_kernel<float><<<grid, 256, smem, stream>>>(a, (float*)mixes);
+        else settle_shift_kernel<bf16_t><<<grid, 256, smem, stream>>>(a, (bf16_t*)mixes);
+    }
     TL_CHECK_LAUNCH("settle_shift");
     return TL_OK;
 }

@@ -42,7 +42,7 @@ def _steps(lengths, cuts):
 # ------------------------------------------------------------------ sums and mixes
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("hidden, kind", [(42, "whole"), (64, "slabs"), (37, "slabs"), (1028, "whole"), (96, "plain"), (50, "nothing")])
+@pytest.mark.parametrize("hidden, kind", [(42, "whole"), (64, "slabs"), (37, "slabs"), (1028, "whole"), (96, "plain"), (50, "nothing"), (5000, "whole"), (9004, "slabs"), (4102, "slabs")])
 def test_sum_and_mixes_of_neighbouring_tokens(dtype, hidden, kind):
     """Two requests in portions, the rows of the tokens before in scrambled slots at an odd offset; the pending output normed, added as it is,
     in slabs, or absent."""
@@ -106,12 +106,12 @@ def test_sum_and_mixes_of_long_prompts(T):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("parts", [0, 3])
-def test_sum_of_a_normed_branch_handed_on_without_a_norm(dtype, parts):
+@pytest.mark.parametrize("parts, H", [(0, 150), (3, 150), (5, 152), (0, 4104), (2, 9000), (8, 2048)])
+def test_sum_of_a_normed_branch_handed_on_without_a_norm(dtype, parts, H):
     from torchlet_amd.config.base import OffsetRMSNormSpec
     from torchlet_amd.parts import NORMS, Stream
     g = torch.Generator().manual_seed(3)
-    T, H, eps = 6, 150, 1e-5
+    T, eps = 6, 1e-5
     norm = NORMS.build(OffsetRMSNormSpec(dim=H, eps=eps, offset=0.0, weight_name=""), dtype, torch.device("cuda"))
     w = (1.0 + torch.randn(H, generator=g) * 0.3).to(torch.bfloat16)
     norm.load_weights({"": w})
@@ -124,6 +124,14 @@ def test_sum_of_a_normed_branch_handed_on_without_a_norm(dtype, parts):
     torch.testing.assert_close(stream.residual.cpu().double(), new, atol=2e-5, rtol=1e-5)
     torch.testing.assert_close(h.cpu().double(), new, **_tol(dtype, 1 if dtype == torch.float32 else 0.5))
     assert stream.pending is None and stream.post is None
+    rows = torch.tensor([4, 0, 4], dtype=torch.int32, device="cuda")         # and the norm of some rows of a sum still pending, the stream left as it is
+    stream.pending, stream.post = y.cuda(), (norm.weight, norm.eps)
+    few = norm.forward(stream, rows=rows, gain=0.7)
+    b = y.double().sum(0) if parts else y.double()
+    want = plain.rms((stream.residual.cpu().double() + plain.rms(b, eps) * w.double())[[4, 0, 4]], eps) * w.double() * 0.7
+    torch.testing.assert_close(few.cpu().double(), want, **_tol(dtype, 3))
+    torch.testing.assert_close(stream.residual.cpu().double(), new, atol=2e-5, rtol=1e-5)
+    stream.pending = stream.post = None
     again = norm.settle(stream)                                  # nothing pending: the residual as it is
     torch.testing.assert_close(again.cpu(), stream.residual.to(dtype).cpu(), atol=0.0, rtol=0.0)
 

@@ -69,7 +69,7 @@ def _every_cut(folder, dtype, page, seqs, refs, tol, what):
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("name", ["A", "B", "C"])
 def test_every_way_of_cutting_requests_equals_plain(folders, name, dtype):
-    """Whole requests; most of a request and its last tokens one by one; portions of changing size down to two tokens; up to four live
+    """Whole requests; a long portion and then single tokens; uneven portions down to two tokens; up to four live
     requests with portions beside single tokens, in a pool that holds no more than the live ones need, so pages and slots are used again."""
     lengths = [37, 5, 70, 1, 18, 33] if name != "B" else [90, 1, 47, 130]
     conf, w = tiny_vabelorn.CONFIGS[name], _weights(name)

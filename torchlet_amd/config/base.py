@@ -116,7 +116,7 @@ class PairRotarySpec(PartSpec):
     factor: float = 1.0        # linear scaling: every frequency is divided by it
     # ``yarn = (factor, original, fast, slow)``: frequencies are blended between themselves and themselves over ``factor``, pair by pair: pairs
     # that turn more than ``fast`` times over ``original`` positions stay, pairs that turn less than ``slow`` times are divided, linearly in the
-    # pair's index between; cosines and sines are multiplied by ``0.1 ln(factor) + 1``
+    # pair's index between; cosines and sines grow by the magnitude ``1 + 0.1 ln(factor)``
     yarn: tuple | None = None
 
 
@@ -210,7 +210,7 @@ class CappedAttentionSpec(PartSpec):
     qk_bias: bool = False
     o_bias: bool = False
     # ``fixed_sink``: the softmax's denominator also holds ``exp`` of this fixed number, the same for all heads (0: one is added).
-    # ``value_norm``: every head's value is divided by its root mean square (``qk_norm_eps``, no weight) before it is cached.
+    # ``value_norm``: values pass a weightless RMS norm per head (``qk_norm_eps``) on their way into the cache.
     # ``value_position``: an encoding over the first dimensions of a value: a cached value is turned by its own position, and a head's output
     # (the sum over the values) at position ``i`` is turned back by ``i``.
     fixed_sink: float | None = None
@@ -273,8 +273,8 @@ class SelectiveStateSpec(PartSpec):
 class WKVSpec(PartSpec):
     """Time mixing with a matrix state whose decays depend on the token (RWKV): r, k, v, the gate and the decay each read a mix of the token's
     input and the one's before it, ``h + (h' - h) * mu``; per head and key channel ``w = exp(-exp(w0 + W_w2 tanh(W_w1 mix)))``; per head ``o = (S +
-    diag(u) k v^T)^T r``, then ``S <- diag(w) S + k v^T``; each head's output is divided by its root mean square (``norm_eps``), multiplied by a
-    weight and by ``silu`` of the gate.  ``decay_rank``: the inner size of the decay's two matrices in the random-weights mode (a checkpoint's
+    diag(u) k v^T)^T r``, then ``S <- diag(w) S + k v^T``; outputs pass an RMS norm per head (``norm_eps``), a weight and ``silu`` of the
+    gate.  ``decay_rank``: the inner size of the decay's two matrices in the random-weights mode (a checkpoint's
     tensors say their own)."""
     kind: ClassVar[str] = "wkv"
     hidden: int = 0
@@ -288,7 +288,7 @@ class WKVSpec(PartSpec):
 @dataclass(frozen=True)
 class TokenSideSpec(PartSpec):
     """A per-layer token input: with ``e`` the layer's slice (``dim`` numbers) of the token's row in a second table, ``y = proj(act(gate(x)) * e)``
-    enters the stream as ``x + y / sqrt(mean(y^2) + eps) * w``."""
+    enters the stream through an RMS norm with a weight, ``x + w * y / rms(y)``."""
     kind: ClassVar[str] = "token_side"
     hidden: int = 0
     dim: int = 0

@@ -14,8 +14,8 @@ A third one keeps several copies of the residual, joined by hyper-connections (:
 A fourth one norms a sublayer's output as well as its input (:class:`SandwichBlock`): ``x <- x + post1(mixer(norm1(x)))``, then ``x <- x +
 post2(ffn(norm2(x)))``; the output is left pending with its norm's weight, and the next norm's kernel norms it, adds it and norms the sum.
 
-A fifth one norms the sublayers' outputs only (:class:`OutputNormBlock`): ``x <- x + norm1(mixer(x))``, then ``x <- x + norm2(ffn(x))``, and may add a
-per-layer token input after them.
+A fifth one norms the sublayers' outputs only (:class:`OutputNormBlock`): the first sublayer leaves ``z = x + norm1(mixer(x))``, the second ``z +
+norm2(ffn(z))``, and a per-layer token input may be added after them.
 """
 from __future__ import annotations
 

@@ -1,7 +1,7 @@
 """A per-layer token input: besides the token's embedding, every layer adds something that it makes of the stream and of the layer's own
 slice ``e`` of the token's row in a second table::
 
-    y = proj (act(gate x) * e);    x <- x + y / sqrt(mean(y^2) + eps) * w
+    y = proj (act(gate x) * e);    x <- x + w * y / rms(y)
 
 The table is the model's (one tensor for all layers); :meth:`TokenSide.attach` hands the layer its columns.  ``y`` is left pending on the stream
 with its norm, so that the next kernel that reads the stream norms it and adds it in 32-bit.

@@ -150,11 +150,11 @@ def interleave_gate_up(gate, up):
     return torch.stack((g.view(blocks, 32, K), u.view(blocks, 32, K)), dim=1).reshape(blocks * 64, K).contiguous()
 
 
-GATE_ACTIVATIONS = {"silu": 0, "relu": 1}
+GATE_ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2}
 
 
 def _gate(g, activation):
-    return torch.relu(g) if activation == "relu" else g / (1 + torch.exp(-g))
+    return torch.relu(g) if activation == "relu" else _act(g, "gelu_tanh") if activation == "gelu_tanh" else g / (1 + torch.exp(-g))
 
 
 def linear_swiglu(x, gate_up, out, activation="silu"):
@@ -373,7 +373,7 @@ def local_attention_mfma_fits(dtype, dim, vdim, page_size):
 
 
 def local_attention(q, out, k_plane, v_plane, block_table, token_req, positions, heads, kv_heads, dim, vdim, page_size, scale,
-                    softcap=0.0, chunk=0, window=0, gain=1.0, tiles=None, sink=None, pooled=None, keep_first=0, turn_back=None):
+                    softcap=0.0, chunk=0, window=0, gain=1.0, tiles=None, sink=None, pooled=None, keep_first=0, turn_back=None, gate=None):
     group = heads // kv_heads
     for t in range(q.shape[0]):
         p, r = int(positions[t]), int(token_req[t])
@@ -402,6 +402,8 @@ def local_attention(q, out, k_plane, v_plane, block_table, token_req, positions,
         o = torch.einsum("hn,nhd->hd", w, v)[None]
         if turn_back is not None:
             _turn_heads(o, positions[t: t + 1], *turn_back, sign=-1.0)
+        if gate is not None:
+            o = o * torch.sigmoid(gate[t].float())[None, :, None]
         out[t] = (o.reshape(-1) * gain).to(out.dtype)
 
 
@@ -431,7 +433,8 @@ def _turn_heads(v, positions, inv_freq, dims, halves, magnitude=1.0, sign=1.0):
         v[..., 0:dims:2], v[..., 1:dims:2] = a * c - b * sn, b * c + a * sn
 
 
-def head_norm_rotate(x, heads_a, heads_b, dim, norm_a, norm_b, eps, positions, inv_freq, dims, halves, raw_b=None, magnitude=1.0, values=None, pages=None):
+def head_norm_rotate(x, heads_a, heads_b, dim, norm_a, norm_b, eps, positions, inv_freq, dims, halves, raw_b=None, magnitude=1.0, values=None, pages=None, unit=False,
+                     heat=None):
     T = x.shape[0]
     width = (heads_a + heads_b) * dim
     if raw_b is not None:
@@ -441,14 +444,18 @@ def head_norm_rotate(x, heads_a, heads_b, dim, norm_a, norm_b, eps, positions, i
         w = torch.cat([(norm_a if norm_a is not None else torch.ones(dim)).float().expand(heads_a, dim),
                        (norm_b if norm_b is not None else torch.ones(dim)).float().expand(heads_b, dim)])
         v = v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps) * w
+    if unit:
+        v = v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps)
+    if heat is not None:
+        v[:, :heads_a] *= (1.0 + heat[0] * torch.log(((positions + 1) // heat[1] + 1).float()))[:, None, None]
     if inv_freq is not None:
         _turn_heads(v, positions, inv_freq, dims, halves, magnitude)
     x[:, :width] = v.reshape(T, -1).to(x.dtype)
     if values is None:
         return
-    heads_c, vdim, unit, c_freq, c_dims, c_halves = values
+    heads_c, vdim, unit_c, c_freq, c_dims, c_halves = values
     c = x[:, width:].float().reshape(T, heads_c, vdim).clone()
-    if unit:
+    if unit_c:
         c = c / torch.sqrt(c.pow(2).mean(-1, keepdim=True) + eps)
     if c_freq is not None:
         _turn_heads(c, positions, c_freq, c_dims, c_halves)
@@ -492,12 +499,13 @@ def bigram_embedding(token_ids, table, out, scale, bigram, buckets, mul_prev, mu
             last_token[int(slots[r]), 0] = int(token_ids[int(req_indptr[r + 1]) - 1])
 
 
-def sandwich_norm(residual, pending, post_weight, post_eps, extra, weight, eps, out, rows=None, gain=1.0):
+def sandwich_norm(residual, pending, post_weight, post_eps, extra, weight, eps, out, rows=None, gain=1.0, branch_gain=1.0):
     y = None
     if pending is not None:
         y = pending.sum(0) if pending.dim() == 3 else pending.float()
         if post_weight is not None:
             y = y / torch.sqrt(y.pow(2).mean(-1, keepdim=True) + post_eps) * post_weight.float()
+        y = y * branch_gain
     r = residual if rows is None else residual[rows.long()]
     add = None
     if extra is not None:
@@ -589,30 +597,34 @@ def latent_attention_mfma_fits(dtype, heads, rank, rot):
     return False
 
 
-def _turn(x, positions, inv_freq):
-    """x [T, ..., rot]: the first 2 * len(inv_freq) entries turned in neighbouring pairs."""
+def _turn(x, positions, inv_freq, halves=False):
+    """x [T, ..., rot]: the first 2 * len(inv_freq) entries turned in neighbouring pairs, or each with the one len(inv_freq) further on."""
     d = 2 * inv_freq.numel()
     ang = positions.float()[:, None] * inv_freq[None, :]
     shape = [x.shape[0]] + [1] * (x.dim() - 2) + [d // 2]
     c, s = ang.cos().view(shape), ang.sin().view(shape)
-    u, v = x[..., 0:d:2], x[..., 1:d:2]
+    first, second = (slice(0, d // 2), slice(d // 2, d)) if halves else (slice(0, d, 2), slice(1, d, 2))
+    u, v = x[..., first], x[..., second]
     y = x.clone()
-    y[..., 0:d:2] = u * c - v * s
-    y[..., 1:d:2] = v * c + u * s
+    y[..., first] = u * c - v * s
+    y[..., second] = v * c + u * s
     return y
 
 
 def latent_prepare(down, q_rank, rank, rot, rot_dims, wq, wkv, eps, positions, inv_freq, cq, token_req=None, block_table=None,
-                   plane=None, page_size=0, kv_off=None):
+                   plane=None, page_size=0, kv_off=None, halves=False, queries=None):
     kv_off = q_rank if kv_off is None else kv_off
     x = down.float()
     norm = lambda t, w: t / torch.sqrt(t.pow(2).mean(-1, keepdim=True) + eps) * w.float()
     if q_rank:
         cq.copy_(norm(x[:, :q_rank], wq).to(cq.dtype))
+    if queries is not None:
+        rows, heads, head, plain = queries
+        rotate_pairs(down, head, plain, rows, rank + rot, rank, positions, inv_freq, heads, rot, halves)
     if plane is None:
         return
     c = norm(x[:, kv_off: kv_off + rank], wkv)
-    kr = _turn(x[:, kv_off + rank: kv_off + rank + rot], positions, inv_freq)
+    kr = _turn(x[:, kv_off + rank: kv_off + rank + rot], positions, inv_freq, halves)
     row = torch.cat((c, kr), dim=-1).to(plane.dtype)
     for t in range(down.shape[0]):
         p = int(positions[t])
@@ -621,10 +633,10 @@ def latent_prepare(down, q_rank, rank, rot, rot_dims, wq, wkv, eps, positions, i
             plane[page, 0, p % page_size] = row[t]
 
 
-def rotate_pairs(src, src_head, src_off, dst, dst_head, dst_off, positions, inv_freq, heads, rot):
+def rotate_pairs(src, src_head, src_off, dst, dst_head, dst_off, positions, inv_freq, heads, rot, halves=False):
     T = src.shape[0]
     x = torch.stack([src[:, h * src_head + src_off: h * src_head + src_off + rot] for h in range(heads)], dim=1).float()
-    y = _turn(x, positions, inv_freq).to(dst.dtype)
+    y = _turn(x, positions, inv_freq, halves).to(dst.dtype)
     for h in range(heads):
         dst[:, h * dst_head + dst_off: h * dst_head + dst_off + rot] = y[:, h]
 
@@ -655,10 +667,12 @@ def latent_attention(q, out, plane, block_table, req_indptr, ctx_lens, tile_req,
             out[first + i] = o.reshape(-1).to(out.dtype)
 
 
-def heads_linear(x, x_head, weight, out, out_head, general=False):
+def heads_linear(x, x_head, weight, out, out_head, general=False, gate=None):
     G, N, K = weight.shape
     for g in range(G):
-        out[:, g * out_head: g * out_head + N] = (x[:, g * x_head: g * x_head + K].float() @ weight[g].float().T).to(out.dtype)
+        cols = slice(g * out_head, g * out_head + N)
+        y = x[:, g * x_head: g * x_head + K].float() @ weight[g].float().T
+        out[:, cols] = (y if gate is None else y * torch.sigmoid(gate[:, cols].float())).to(out.dtype)
 
 
 def _act(y, activation):
@@ -683,19 +697,25 @@ def experts_linear(x, slot_token, weight, offsets, out, activation="none", gener
             out[lo:hi] = _act(rows.float() @ weight[e].float().T, activation).to(out.dtype)
 
 
-def route(logits, top, scores="chosen", choice_bias=None, weight_scale=1.0, weight_eps=0.0):
+def route(logits, top, scores="chosen", choice_bias=None, weight_scale=1.0, weight_eps=0.0, groups=None):
     T, E = logits.shape
+    shut = torch.zeros(T, E)
+    if groups is not None:          # (all the forms below choose by something that grows with the logit; no bias beside groups in the tests)
+        count, keep = groups
+        kept = logits.view(T, count, -1).amax(-1).topk(keep, dim=-1).indices
+        open_ = torch.zeros(T, count, dtype=torch.bool).scatter_(1, kept, True).repeat_interleave(E // count, dim=1)
+        shut = torch.where(open_, 0.0, float("-inf"))
     if scores == "all":
         s = torch.softmax(logits, dim=-1)
-        best = (s if choice_bias is None else s + choice_bias).topk(top, dim=-1)
+        best = (shut + (s if choice_bias is None else s + choice_bias)).topk(top, dim=-1)
         weights = s.gather(1, best.indices)
     elif scores == "sigmoid":
         s = torch.sigmoid(logits)
-        best = (s if choice_bias is None else s + choice_bias).topk(top, dim=-1)
+        best = (shut + (s if choice_bias is None else s + choice_bias)).topk(top, dim=-1)
         weights = s.gather(1, best.indices)
         weights = weights / (weights.sum(-1, keepdim=True) + weight_eps)
     else:
-        best = logits.topk(top, dim=-1)               # ties: not met in tests
+        best = (logits + shut).topk(top, dim=-1)               # ties: not met in tests
         weights = torch.softmax(best.values, dim=-1)
     weights = weights * weight_scale
     chosen = best.indices.reshape(-1)

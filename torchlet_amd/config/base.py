@@ -96,7 +96,7 @@ class AttentionSpec(PartSpec):
 
 @dataclass(frozen=True)
 class SwiGLUSpec(PartSpec):
-    """``down(act(gate(h)) * up(h))`` without biases; ``activation``: ``silu`` or ``relu``; the three matrices' names below the part's."""
+    """``down(act(gate(h)) * up(h))`` without biases; ``activation``: ``silu``, ``relu`` or ``gelu_tanh``; the three matrices' names below the part's."""
     kind: ClassVar[str] = "swiglu"
     hidden: int = 0
     intermediate: int = 0
@@ -171,8 +171,10 @@ class LatentAttentionSpec(PartSpec):
     position: PartSpec | None = None     # encoding of the rotated parts
     # ``q_rank`` 0: no query latent, ``q = W_q h`` (tensor ``q``).  ``rot_dim`` 0: no rotated part.  ``window``: a query reads the last
     # ``window`` positions, itself included.  ``gate``: head ``n``'s output is multiplied by ``sigmoid(W_g h)[n]`` (tensor ``g [heads, hidden]``).
+    # ``gate_values``: the heads' values side by side are multiplied number by number by ``sigmoid(W_g h)`` (tensor ``g [heads * vdim, hidden]``).
     window: int | None = None
     gate: bool = False
+    gate_values: bool = False
 
 
 @dataclass(frozen=True)
@@ -216,6 +218,15 @@ class CappedAttentionSpec(PartSpec):
     fixed_sink: float | None = None
     value_norm: bool = False
     value_position: PartSpec | None = None
+    # ``qk_unit_norm``: queries and keys are divided by their root mean square per head (``qk_norm_eps``), without weights.  ``query_heat = (coef,
+    # every)``: the query at position ``p`` is multiplied by ``1 + coef * ln(floor((p + 1) / every) + 1)`` behind its norm.  ``v_bias``: with ``qk_bias``,
+    # the value projection has a bias too (``v.b``).  ``gate``: head ``n``'s output is multiplied by ``sigmoid(W_g h)[n]`` (tensor ``g [heads,
+    # hidden]``).  ``reads_cache``: the mixer projects queries only and reads keys and values that another run of the order has cached.
+    qk_unit_norm: bool = False
+    query_heat: tuple | None = None
+    v_bias: bool = False
+    gate: bool = False
+    reads_cache: bool = False
 
 
 @dataclass(frozen=True)
@@ -326,7 +337,8 @@ class RoutedExpertsSpec(PartSpec):
     experts' outputs.  ``scores``: ``"chosen"``: the choice goes by the logits and the weights are the softmax over the chosen ones alone;
     ``"all"``: the scores are the softmax over all logits and the weights are the chosen experts' scores as they are; ``"sigmoid"``: the
     scores are the logits' sigmoids and the weights the chosen scores divided by their sum (plus ``weight_eps``).  ``choice_bias``: a
-    vector ``correction`` is added to the scores for the choice only.  ``identity``: the router has that many outputs beyond ``experts``;
+    vector ``correction`` is added to the scores for the choice only.  ``groups = (count, keep)``: the experts lie in ``count`` equal groups side
+    by side, a group counts as much as its best expert, and the choice is among the experts of the ``keep`` best groups.  ``identity``: the router has that many outputs beyond ``experts``;
     an expert chosen among those returns its input.  ``weight_scale``: a factor on the weights.  ``shared``: the specification of one more
     feed-forward (tensors below ``shared``) that runs for every token and is added to the experts' weighted sum."""
     kind: ClassVar[str] = "routed_experts"
@@ -343,6 +355,7 @@ class RoutedExpertsSpec(PartSpec):
     weight_scale: float = 1.0
     weight_eps: float = 1e-20
     shared: PartSpec | None = None
+    groups: tuple | None = None
 
 
 @dataclass(frozen=True)
@@ -360,6 +373,14 @@ class BlockSpec(PartSpec):
     ffn_name: str = "mlp"
     mixer_norm_name: str = "input_layernorm"
     ffn_norm_name: str = "post_attention_layernorm"
+
+
+@dataclass(frozen=True)
+class ScaledBlockSpec(BlockSpec):
+    """One layer whose branches enter the residual times a fixed factor: ``x <- x + branch_gain * mixer(mixer_norm(x))``, then ``x <- x +
+    branch_gain * ffn(ffn_norm(x))``.  ``ffn`` (and then ``ffn_norm``) may be ``None``: the layer ends after the first step."""
+    kind: ClassVar[str] = "scaled_residual"
+    branch_gain: float = 1.0
 
 
 @dataclass(frozen=True)

@@ -40,6 +40,11 @@ __device__ __forceinline__ float wave_max(float v) {
     return v;
 }
 
+__device__ __forceinline__ float sigmoid(float v) { return 1.f / (1.f + expf(-v)); }
+
+// z / 2 (1 + tanh(y)), y = sqrt(2 / pi) (z + 0.044715 z^3), with (1 + tanh(y)) / 2 = sigmoid(2 y).
+__device__ __forceinline__ float gelu_tanh(float z) { return z * sigmoid(1.5957691216057308f * fmaf(0.044715f * z * z, z, z)); }
+
 // Sum over a block of up to 1024 threads; every thread gets the result.
 // `red` points to at least 16 floats of shared memory.
 __device__ __forceinline__ float block_sum(float v, float* red) {

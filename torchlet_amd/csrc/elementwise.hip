@@ -450,7 +450,7 @@ extern "C" int tl_rope_cache_write(void* qkv, int row_stride, int tokens, int q_
 }
 
 // ------------------------------------------------------------------ SwiGLU gate
-// out[t, i] = act(gu[t, i]) * gu[t, inter + i]; act 0: silu(g) = g / (1 + exp(-g)), act 1: relu.
+// out[t, i] = act(gu[t, i]) * gu[t, inter + i]; act 0: silu(g) = g / (1 + exp(-g)), act 1: relu, act 2: the tanh form of gelu.
 template <typename T>
 __global__ void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter, size_t total, int act) {
     const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -459,11 +459,11 @@ __global__ void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, int
     const int i = (int)(idx % inter);
     const float g = to_float(gu[t * 2 * inter + i]);
     const float u = to_float(gu[t * 2 * inter + inter + i]);
-    out[idx] = from_float<T>((act == 1 ? fmaxf(g, 0.f) : g / (1.f + expf(-g))) * u);
+    out[idx] = from_float<T>((act == 1 ? fmaxf(g, 0.f) : act == 2 ? gelu_tanh(g) : g / (1.f + expf(-g))) * u);
 }
 
 extern "C" int tl_swiglu(const void* gu, void* out, int tokens, int inter, int act_dtype, int act, hipStream_t stream) {
-    TL_REQUIRE(tokens >= 0 && inter > 0 && (act == 0 || act == 1), "swiglu: bad sizes tokens=%d inter=%d, or an unknown gate %d", tokens, inter, act);
+    TL_REQUIRE(tokens >= 0 && inter > 0 && act >= 0 && act <= 2, "swiglu: bad sizes tokens=%d inter=%d, or an unknown gate %d", tokens, inter, act);
     const size_t total = (size_t)tokens * inter;
     if (total == 0) return TL_OK;
     dim3 block(256), grid((unsigned)((total + 255) / 256));
@@ -838,12 +838,12 @@ static RowPlan plan_row(int hidden) {
 // ------------------------------------------------------------------ norm of the branch output, addition, norm of the sum
 // One block per output row, the row kept in shared memory between the passes:
 //   y = pending[row] (one tensor of the activation type, or `parts` float slabs added up);
-//   r = residual[row] (+ extra[row]) + y * (post ? rsqrt(mean(y^2) + post_eps) * post[i] : 1);   written back unless `rows` selects
+//   r = residual[row] (+ extra[row]) + y * branch_gain * (post ? rsqrt(mean(y^2) + post_eps) * post[i] : 1);   written back unless `rows` selects
 //   out = r * rsqrt(mean(r^2) + eps) * weight[i] * gain, or, without a `weight`, r * gain (the sum itself, in the activation type).
 // `post` and `weight` are float vectors of post_n / weight_n numbers: `hidden` of them, or one for all coordinates.
 template <typename T>
 __global__ void sandwich_norm_kernel(float* __restrict__ residual, const void* __restrict__ pending, int parts, size_t part_stride,
-                                     const float* __restrict__ post, int post_n, float post_eps, const float* __restrict__ extra,
+                                     const float* __restrict__ post, int post_n, float post_eps, float branch_gain, const float* __restrict__ extra,
                                      const float* __restrict__ weight, int weight_n, float eps, float gain, T* __restrict__ out,
                                      const int* __restrict__ rows, int hidden) {
     extern __shared__ float sn_row[];
@@ -854,7 +854,7 @@ __global__ void sandwich_norm_kernel(float* __restrict__ residual, const void* _
     const T* pen = (pending && parts == 0) ? (const T*)pending + (size_t)srow * hidden : nullptr;
     const float* pparts = (pending && parts > 0) ? (const float*)pending + (size_t)srow * hidden : nullptr;
     const float* ex = extra ? extra + (size_t)srow * hidden : nullptr;
-    float inv_y = 1.f;
+    float inv_y = branch_gain;
     if (pending) {
         float ss = 0.f;
         for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
@@ -865,14 +865,14 @@ __global__ void sandwich_norm_kernel(float* __restrict__ residual, const void* _
             sn_row[i] = y;
             ss = fmaf(y, y, ss);
         }
-        if (post) inv_y = rsqrtf(block_sum(ss, red) / (float)hidden + post_eps);
+        if (post) inv_y = rsqrtf(block_sum(ss, red) / (float)hidden + post_eps) * branch_gain;
     }
     const bool update = (pending != nullptr || ex != nullptr) && rows == nullptr;
     float ss = 0.f;
     for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
         float r = res[i];
         if (ex) r += ex[i];
-        if (pending) r += post ? sn_row[i] * inv_y * post[post_n == 1 ? 0 : i] : sn_row[i];
+        if (pending) r += post ? sn_row[i] * inv_y * post[post_n == 1 ? 0 : i] : sn_row[i] * inv_y;
         if (update) res[i] = r;
         sn_row[i] = r;
         ss = fmaf(r, r, ss);
@@ -891,7 +891,7 @@ __global__ void sandwich_norm_kernel(float* __restrict__ residual, const void* _
 template <typename T, int NP>
 __global__ void __launch_bounds__(1024)
 sandwich_norm_rows_kernel(float* __restrict__ residual, const void* __restrict__ pending, int parts, size_t part_stride,
-                          const float* __restrict__ post, int post_n, float post_eps, const float* __restrict__ extra,
+                          const float* __restrict__ post, int post_n, float post_eps, float branch_gain, const float* __restrict__ extra,
                           const float* __restrict__ weight, int weight_n, float eps, float gain, T* __restrict__ out,
                           const int* __restrict__ rows, int hidden) {
     __shared__ float red[16];
@@ -903,13 +903,13 @@ sandwich_norm_rows_kernel(float* __restrict__ residual, const void* __restrict__
     if (pending && post) load_weights<NP>(post, post_n, hidden, pw);
     if (extra) load_row<NP>(extra + at, hidden, ex);
     if (weight) load_weights<NP>(weight, weight_n, hidden, w);
-    const float inv_y = pending && post ? rsqrtf(block_sum(row_squares(y), red) / (float)hidden + post_eps) : 1.f;
+    const float inv_y = branch_gain * (pending && post ? rsqrtf(block_sum(row_squares(y), red) / (float)hidden + post_eps) : 1.f);
 #pragma unroll
     for (int n = 0; n < NP; ++n)
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
             if (extra) r.v[n][v] += ex.v[n][v];
-            if (pending) r.v[n][v] += post ? y.v[n][v] * inv_y * pw.v[n][v] : y.v[n][v];
+            if (pending) r.v[n][v] += post ? y.v[n][v] * inv_y * pw.v[n][v] : y.v[n][v] * inv_y;
         }
     if ((pending || extra) && !rows) store_row<NP>(residual + at, hidden, r);
     const float inv = weight ? rsqrtf(block_sum(row_squares(r), red) / (float)hidden + eps) * gain : gain;
@@ -921,7 +921,7 @@ sandwich_norm_rows_kernel(float* __restrict__ residual, const void* __restrict__
 }
 
 extern "C" int tl_sandwich_norm(void* residual, const void* pending, int parts, int part_rows, const void* post, int post_n, float post_eps,
-                                const void* extra, const void* weight, int weight_n, float eps, float gain, void* out, const void* rows,
+                                float branch_gain, const void* extra, const void* weight, int weight_n, float eps, float gain, void* out, const void* rows,
                                 int out_rows, int hidden, int act_dtype, hipStream_t stream) {
     TL_REQUIRE(parts >= 0 && parts <= 64 && out_rows >= 0 && hidden > 0 && hidden <= 12288, "sandwich_norm: bad sizes rows=%d hidden=%d parts=%d", out_rows, hidden, parts);
     TL_REQUIRE((!weight || weight_n == 1 || weight_n == hidden) && (!post || post_n == 1 || post_n == hidden), "sandwich_norm: weights of one number or of %d", hidden);
@@ -933,7 +933,7 @@ extern "C" int tl_sandwich_norm(void* residual, const void* pending, int parts, 
         const RowPlan plan = plan_row(hidden);
 #define TL_SN(T, N)                                                                                                                               \
     sandwich_norm_rows_kernel<T, N><<<out_rows, plan.threads, 0, stream>>>((float*)residual, pending, parts, part_stride, (const float*)post, post_n, post_eps, \
-        (const float*)extra, (const float*)weight, weight_n, eps, gain, (T*)out, (const int*)rows, hidden)
+        branch_gain, (const float*)extra, (const float*)weight, weight_n, eps, gain, (T*)out, (const int*)rows, hidden)
 #define TL_SN_T(T) if (plan.pieces == 1) TL_SN(T, 1); else if (plan.pieces == 2) TL_SN(T, 2); else TL_SN(T, 3)
         if (act_dtype == TL_DT_F32) { TL_SN_T(float); } else { TL_SN_T(bf16_t); }
 #undef TL_SN_T
@@ -944,10 +944,10 @@ extern "C" int tl_sandwich_norm(void* residual, const void* pending, int parts, 
     const int threads = hidden >= 2048 ? 512 : 256;
     if (act_dtype == TL_DT_F32)
         sandwich_norm_kernel<float><<<out_rows, threads, smem, stream>>>((float*)residual, pending, parts, part_stride, (const float*)post, post_n, post_eps,
-            (const float*)extra, (const float*)weight, weight_n, eps, gain, (float*)out, (const int*)rows, hidden);
+            branch_gain, (const float*)extra, (const float*)weight, weight_n, eps, gain, (float*)out, (const int*)rows, hidden);
     else if (act_dtype == TL_DT_BF16)
         sandwich_norm_kernel<bf16_t><<<out_rows, threads, smem, stream>>>((float*)residual, pending, parts, part_stride, (const float*)post, post_n, post_eps,
-            (const float*)extra, (const float*)weight, weight_n, eps, gain, (bf16_t*)out, (const int*)rows, hidden);
+            branch_gain, (const float*)extra, (const float*)weight, weight_n, eps, gain, (bf16_t*)out, (const int*)rows, hidden);
     else TL_REQUIRE(false, "sandwich_norm: unknown dtype %d", act_dtype);
     TL_CHECK_LAUNCH("sandwich_norm");
     return TL_OK;

@@ -13,7 +13,7 @@
 __device__ __forceinline__ float activate(float v, int act) {
     if (act == ACT_RELU2) { v = fmaxf(v, 0.f); return v * v; }
     if (act == ACT_SILU) return v / (1.f + expf(-v));
-    if (act == ACT_GELU_TANH) return 0.5f * v * (1.f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
+    if (act == ACT_GELU_TANH) return gelu_tanh(v);
     if (act == ACT_GELU) return 0.5f * v * (1.f + erff(v * 0.7071067811865476f));
     return v;
 }
@@ -29,6 +29,8 @@ __host__ __device__ __forceinline__ bool known_activation(int act) { return (act
 //   offsets != null: group g owns the rows offsets[g] .. offsets[g + 1] - 1 (sorted slots); blockIdx.x runs over an upper
 //                    bound of all groups' tiles and finds its group by walking the offsets; `src` (optional) maps a
 //                    sorted slot to the row of `a` it reads (a token routed to an expert), output rows are the slots.
+//   gate (optional, without offsets, no activation): out[m, c] is multiplied by sigmoid(gate[m, c]) before its one rounding (row m of `gate`
+//                    is gate_ld numbers after the one before, of the activation type).
 #define GG_T 64
 #define GG_K 16
 
@@ -36,7 +38,7 @@ template <typename T>
 __global__ void __launch_bounds__(256)
 grouped_gemm_kernel(const T* __restrict__ a, int a_ld, int a_group, const int* __restrict__ src, const T* __restrict__ w,
                     T* __restrict__ out, int out_ld, int out_group, const int* __restrict__ offsets, int groups, int rows,
-                    int N, int K, int act) {
+                    int N, int K, int act, const T* __restrict__ gate, int gate_ld) {
     __shared__ float sa[GG_K][GG_T + 4];
     __shared__ float sw[GG_K][GG_T + 4];
     int g, m0, m_end;
@@ -101,7 +103,10 @@ grouped_gemm_kernel(const T* __restrict__ a, int a_ld, int a_group, const int* _
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int n = n0 + tx * 4 + j;
-            if (n < N) orow[n] = from_float<T>(activate(acc[i][j], act));
+            if (n >= N) continue;
+            float v = activate(acc[i][j], act);
+            if (gate) v *= sigmoid(to_float(gate[(size_t)m * gate_ld + out_col + n]));
+            orow[n] = from_float<T>(v);
         }
     }
 }
@@ -125,7 +130,7 @@ union GmFrag {
 __global__ void __launch_bounds__(256)
 grouped_gemm_mfma_kernel(const bf16_t* __restrict__ a, int a_ld, int a_group, const int* __restrict__ src, const bf16_t* __restrict__ w,
                          bf16_t* __restrict__ out, int out_ld, int out_group, const int* __restrict__ offsets, int groups, int rows,
-                         int N, int K, int act) {
+                         int N, int K, int act, const bf16_t* __restrict__ gate, int gate_ld) {
     int g, m0, m_end;
     if (offsets == nullptr) {
         g = blockIdx.z; m0 = blockIdx.x * GM_BM; m_end = rows;
@@ -190,6 +195,11 @@ grouped_gemm_mfma_kernel(const bf16_t* __restrict__ a, int a_ld, int a_group, co
                     if (n + v + 1 < N) orow[(n + v) / 2] = from_float<bf16_t>(activate(acc[i][j][v], base_act) * acc[i][j][v + 1]);
                 continue;
             }
+            if (gate) {                                 // (no activation beside a gate)
+                const bf16_t* grow = gate + (size_t)m * gate_ld + out_col;
+#pragma unroll
+                for (int v = 0; v < 4; ++v) acc[i][j][v] *= sigmoid(to_float(grow[min(n + v, N - 1)]));
+            }
             if (n + 3 < N && ((out_ld | out_col) & 3) == 0) {
                 union { uint2 u; uint16_t e[4]; } pk;
 #pragma unroll
@@ -205,10 +215,12 @@ grouped_gemm_mfma_kernel(const bf16_t* __restrict__ a, int a_ld, int a_group, co
 }
 
 extern "C" int tl_grouped_gemm(const void* a, int a_ld, int a_group, const void* src, const void* w, void* out, int out_ld, int out_group,
-                               const void* offsets, int groups, int rows, int N, int K, int act, int dtype, int general, hipStream_t stream) {
+                               const void* offsets, int groups, int rows, int N, int K, int act, const void* gate, int gate_ld, int dtype, int general,
+                               hipStream_t stream) {
     TL_REQUIRE(groups > 0 && rows >= 0 && N > 0 && K > 0 && a_ld > 0 && out_ld > 0, "grouped_gemm: bad sizes");
     TL_REQUIRE(known_activation(act), "grouped_gemm: unknown activation %d", act);
     TL_REQUIRE(!(act & ACT_PAIRS) || (N % 2 == 0 && out_group == 0), "grouped_gemm: an activation in pairs needs an even number of columns");
+    TL_REQUIRE(!gate || (!offsets && act == ACT_NONE && gate_ld >= (groups - 1) * out_group + N), "grouped_gemm: a gate stands beside groups of equal rows, with a number per output column");
     if (rows == 0) return TL_OK;
     // with offsets, `rows` is the number of sorted slots in all groups together: every group may end in a partial tile
     dim3 grid(offsets ? (rows + GG_T - 1) / GG_T + groups : (rows + GG_T - 1) / GG_T, (N + GG_T - 1) / GG_T, offsets ? 1 : groups), block(256);
@@ -217,16 +229,16 @@ extern "C" int tl_grouped_gemm(const void* a, int a_ld, int a_group, const void*
     if (dtype == TL_DT_BF16 && aligned && !general) {
         dim3 mgrid(offsets ? (rows + GM_BM - 1) / GM_BM + groups : (rows + GM_BM - 1) / GM_BM, (N + GM_BN - 1) / GM_BN, offsets ? 1 : groups);
         grouped_gemm_mfma_kernel<<<mgrid, block, 0, stream>>>((const bf16_t*)a, a_ld, a_group, (const int*)src, (const bf16_t*)w, (bf16_t*)out, out_ld,
-                                                              out_group, (const int*)offsets, groups, rows, N, K, act);
+                                                              out_group, (const int*)offsets, groups, rows, N, K, act, (const bf16_t*)gate, gate_ld);
         TL_CHECK_LAUNCH("grouped_gemm_mfma");
         return TL_OK;
     }
     if (dtype == TL_DT_F32)
         grouped_gemm_kernel<float><<<grid, block, 0, stream>>>((const float*)a, a_ld, a_group, (const int*)src, (const float*)w, (float*)out, out_ld,
-                                                               out_group, (const int*)offsets, groups, rows, N, K, act);
+                                                               out_group, (const int*)offsets, groups, rows, N, K, act, (const float*)gate, gate_ld);
     else if (dtype == TL_DT_BF16)
         grouped_gemm_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)a, a_ld, a_group, (const int*)src, (const bf16_t*)w, (bf16_t*)out, out_ld,
-                                                                out_group, (const int*)offsets, groups, rows, N, K, act);
+                                                                out_group, (const int*)offsets, groups, rows, N, K, act, (const bf16_t*)gate, gate_ld);
     else TL_REQUIRE(false, "grouped_gemm: unknown dtype %d", dtype);
     TL_CHECK_LAUNCH("grouped_gemm");
     return TL_OK;
@@ -239,9 +251,11 @@ extern "C" int tl_grouped_gemm(const void* a, int a_ld, int a_group, const void*
 //           chosen experts' scores as they are.
 //   mode 2: the scores are the logits' sigmoids; the choice goes by score + bias[e] (bias optional), the weights are the chosen
 //           experts' scores divided by their sum plus weight_eps.
-// In every mode the weights are multiplied by weight_scale at the end.
+// In every mode the weights are multiplied by weight_scale at the end.  group_size > 0: the experts lie in groups of that many neighbours, a
+// group counts as much as the best of its experts (by what the choice goes by), and only the group_keep best groups' experts can be chosen.
 __global__ void route_topk_kernel(const float* __restrict__ logits, int experts, int top, int mode, const float* __restrict__ bias,
-                                  int* __restrict__ chosen, float* __restrict__ weights, int tokens, float weight_scale, float weight_eps) {
+                                  int* __restrict__ chosen, float* __restrict__ weights, int tokens, float weight_scale, float weight_eps, int group_size,
+                                  int group_keep) {
     const int t = blockIdx.x * (blockDim.x / TL_WAVE) + threadIdx.x / TL_WAVE, lane = threadIdx.x % TL_WAVE;
     if (t >= tokens) return;
     const float* z = logits + (size_t)t * experts;
@@ -255,15 +269,16 @@ __global__ void route_topk_kernel(const float* __restrict__ logits, int experts,
         den = wave_sum(sum);
     }
     float first = 0.f, sum = 0.f, mine = 0.f;           // lane j keeps the j-th choice's term
-    unsigned long long taken = 0;                       // bit i: this lane's expert lane + 64 * i is chosen already
-    for (int j = 0; j < top; ++j) {
-        float best = -INFINITY, score = 0.f;
+    // the best of this token's experts whose bit in `skip` (bit i: this lane's expert lane + 64 * i) is not set: its index, what it is chosen by, its score
+    auto pick = [&](unsigned long long skip, float& best, float& score) {
+        best = -INFINITY;
+        score = 0.f;
         int at = 0x7fffffff;
         for (int e = lane, i = 0; e < experts; e += TL_WAVE, ++i) {
             float v = z[e], sc = 0.f;
             if (mode == 1) { sc = expf(v - zmax) / den; v = bias ? sc + bias[e] : sc; }
             else if (mode == 2) { sc = 1.f / (1.f + expf(-v)); v = bias ? sc + bias[e] : sc; }
-            if (!((taken >> i) & 1ull) && (v > best || (v == best && e < at))) { best = v; at = e; score = sc; }
+            if (!((skip >> i) & 1ull) && (v > best || (v == best && e < at))) { best = v; at = e; score = sc; }
         }
 #pragma unroll
         for (int o = TL_WAVE / 2; o > 0; o >>= 1) {
@@ -272,6 +287,22 @@ __global__ void route_topk_kernel(const float* __restrict__ logits, int experts,
             const int oa = __shfl_xor(at, o, TL_WAVE);
             if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; score = os; }
         }
+        return min(at, experts - 1);                    // (outputs that are no numbers choose nothing: the last expert stands in)
+    };
+    unsigned long long taken = 0;                       // the experts that are chosen already, or whose group is not kept
+    if (group_size > 0) {
+        unsigned long long kept = 0;                    // the best expert outside the kept groups tells the next best group
+        for (int j = 0; j < group_keep; ++j) {
+            float best, score;
+            const int g = pick(kept, best, score) / group_size;
+            for (int e = lane, i = 0; e < experts; e += TL_WAVE, ++i)
+                if (e / group_size == g) kept |= 1ull << i;
+        }
+        taken = ~kept;
+    }
+    for (int j = 0; j < top; ++j) {
+        float best, score;
+        const int at = pick(taken, best, score);
         if (at % TL_WAVE == lane) taken |= 1ull << (at / TL_WAVE);
         if (j == 0) first = best;
         const float p = mode != 0 ? score : expf(best - first);
@@ -304,13 +335,16 @@ route_sort_kernel(const int* __restrict__ chosen, int pairs, int top, int expert
 }
 
 extern "C" int tl_route(const void* logits, int tokens, int experts, int top, int mode, const void* bias, void* chosen, void* weights,
-                        void* offsets, void* slot_token, void* pair_slot, float weight_scale, float weight_eps, hipStream_t stream) {
+                        void* offsets, void* slot_token, void* pair_slot, float weight_scale, float weight_eps, int groups, int groups_kept,
+                        hipStream_t stream) {
     TL_REQUIRE(mode >= 0 && mode <= 2, "route: unknown mode %d", mode);
     TL_REQUIRE(tokens >= 0 && experts > 0 && top > 0 && top <= experts && top <= TL_WAVE && experts <= 64 * TL_WAVE, "route: bad sizes (experts %d, top %d)", experts, top);
     TL_REQUIRE((experts + 1) * sizeof(int) <= 64 * 1024, "route: too many experts (%d)", experts);
+    TL_REQUIRE(groups >= 0 && (groups == 0 || (experts % groups == 0 && groups_kept > 0 && groups_kept <= groups && top <= groups_kept * (experts / groups))),
+               "route: %d of %d groups of %d experts do not hold %d choices", groups_kept, groups, experts, top);
     if (tokens == 0) return TL_OK;
     route_topk_kernel<<<(tokens + 3) / 4, 4 * TL_WAVE, 0, stream>>>((const float*)logits, experts, top, mode, (const float*)bias, (int*)chosen, (float*)weights, tokens,
-                                                                    weight_scale, weight_eps);
+                                                                    weight_scale, weight_eps, groups > 0 ? experts / groups : 0, groups_kept);
     TL_CHECK_LAUNCH("route_topk");
     route_sort_kernel<<<1, 1024, (experts + 1) * sizeof(int), stream>>>((const int*)chosen, tokens * top, top, experts, (int*)offsets,
                                                                        (int*)slot_token, (int*)pair_slot);

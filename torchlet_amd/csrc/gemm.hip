@@ -500,9 +500,10 @@ constexpr int skinny_depth() {
     return d < 2 ? 2 : (d > 8 ? 8 : d);
 }
 
-// The gate of a fused gate/up product: GATE 1: silu(g) * u, GATE 2: relu(g) * u (the value of SW in the kernels below; 0: no gate).
+// The gate of a fused gate/up product: GATE 1: silu(g) * u, GATE 2: relu(g) * u, GATE 3: gelu(g) * u in its tanh form (the value of SW in the
+// kernels below; 0: no gate).
 template <int GATE>
-__device__ __forceinline__ float gate_mul(float g, float u) { return GATE == 2 ? fmaxf(g, 0.f) * u : g / (1.f + expf(-g)) * u; }
+__device__ __forceinline__ float gate_mul(float g, float u) { return (GATE == 3 ? gelu_tanh(g) : GATE == 2 ? fmaxf(g, 0.f) : g / (1.f + expf(-g))) * u; }
 
 // SW (gate/up product with the SwiGLU gate applied to the accumulators): w holds blocks of 64
 // rows, 32 gate rows followed by the 32 up rows of the same columns; a work-group's strip is up to 16
@@ -1990,9 +1991,10 @@ static int gemm_gated(const void* x, const void* w, void* out, int M, int I, int
     return TL_OK;
 }
 
-// `act`: the gate's activation, 0 silu, 1 relu.
+// `act`: the gate's activation, 0 silu, 1 relu, 2 the tanh form of gelu.
 extern "C" int tl_gemm_swiglu(const void* x, const void* w, void* out, int M, int I, int K, int ldx, int ldo, int act, hipStream_t stream) {
-    TL_REQUIRE(act == 0 || act == 1, "gemm_swiglu: unknown gate %d", act);
+    TL_REQUIRE(act >= 0 && act <= 2, "gemm_swiglu: unknown gate %d", act);
+    if (act == 2) return gemm_gated<3>(x, w, out, M, I, K, ldx, ldo, stream);
     return act == 1 ? gemm_gated<2>(x, w, out, M, I, K, ldx, ldo, stream) : gemm_gated<1>(x, w, out, M, I, K, ldx, ldo, stream);
 }
 

@@ -11,7 +11,7 @@ __device__ __forceinline__ void shared_barrier() {
     asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
 }
 
-// The pair (u, v) at entries (2i, 2i + 1) turned by position * inv_freq[i].
+// The pair (u, v) turned by position * f.
 __device__ __forceinline__ void turn_pair(float u, float v, float pos, float f, float& a, float& b) {
     float s, c;
     sincosf(pos * f, &s, &c);
@@ -23,16 +23,47 @@ __device__ __forceinline__ void turn_pair(float u, float v, float pos, float f, 
 // down [tokens, ld]: q_rank numbers of the query latent (q_rank 0: none), and from column kv_off on rank numbers of the key/value
 // latent, then rot of the shared key part.
 // cq = rmsnorm(first q_rank) * wq;  page row of the token = [rmsnorm(the rank numbers) * wkv, the last rot with the first
-// rot_dims of them turned in pairs].  A token whose block-table entry is 0 (the sentinel page) writes nothing.
+// rot_dims of them turned in pairs: entries 2i and 2i + 1, or, `halves`, i and i + rot_dims / 2].  A token whose block-table entry is 0
+// (the sentinel page) writes nothing.
+// `rows` (where the queries themselves are columns of `down`): head h's rotated part, the rot numbers from column h * head + plain on, goes
+// to columns rank .. rank + rot - 1 of the head's row there (rank + rot numbers a head, rows_ld a token), turned by the same angles.
+#define LAT_MAX_PAIRS 512
+struct QueryParts {
+    int heads, head, plain, rows_ld;
+};
 template <typename T>
 __global__ void latent_prepare_kernel(const T* __restrict__ down, int ld, int q_rank, int kv_off, int rank, int rot, int rot_dims,
                                       const void* __restrict__ wq, int wq_f32, const void* __restrict__ wkv, int wkv_f32, float eps,
                                       const int* __restrict__ positions, const float* __restrict__ inv_freq,
                                       const int* __restrict__ token_req, const int* __restrict__ block_table, int bt_stride,
-                                      T* __restrict__ plane, int page_size, T* __restrict__ cq) {
+                                      T* __restrict__ plane, int page_size, T* __restrict__ cq, int halves, T* __restrict__ rows, QueryParts parts) {
     __shared__ float red[16];
+    __shared__ float cs[LAT_MAX_PAIRS], sn[LAT_MAX_PAIRS];      // the token's angles: all heads and the shared key part turn by them
     const int t = blockIdx.x;
     const T* row = down + (size_t)t * ld;
+    const int half = rot_dims / 2;
+    for (int i = threadIdx.x; i < half; i += blockDim.x) sincosf((float)positions[t] * inv_freq[i], &sn[i], &cs[i]);
+    __syncthreads();
+    // number j of a rotated part: its partner lies as far on as the pair is wide
+    auto turn_part = [&](const T* src, T* dst) {
+        return [=](int j) {
+            if (j < half) {
+                const int a = halves ? j : 2 * j, b = halves ? j + half : 2 * j + 1;
+                const float u = to_float(src[a]), v = to_float(src[b]);
+                dst[a] = from_float<T>(u * cs[j] - v * sn[j]);
+                dst[b] = from_float<T>(v * cs[j] + u * sn[j]);
+            } else {
+                dst[half + j] = src[half + j];                  // (what lies beyond the rotated dimensions passes)
+            }
+        };
+    };
+    const int steps = rot - half;                               // pairs, then single numbers
+    if (rows) {
+        for (int i = threadIdx.x; i < parts.heads * steps; i += blockDim.x) {
+            const int h = i / steps;
+            turn_part(row + (size_t)h * parts.head + parts.plain, rows + (size_t)t * parts.rows_ld + (size_t)h * (rank + rot) + rank)(i % steps);
+        }
+    }
     float ss = 0.f, inv = 0.f;
     if (q_rank > 0) {
         for (int i = threadIdx.x; i < q_rank; i += blockDim.x) { const float x = to_float(row[i]); ss = fmaf(x, x, ss); }
@@ -53,27 +84,25 @@ __global__ void latent_prepare_kernel(const T* __restrict__ down, int ld, int q_
     for (int i = threadIdx.x; i < rank; i += blockDim.x)
         dst[i] = from_float<T>(to_float(row[kv_off + i]) * inv * load_vec(wkv, wkv_f32, i));
     const T* kr = row + kv_off + rank;
-    for (int i = threadIdx.x; i < rot_dims / 2; i += blockDim.x) {
-        float a, b;
-        turn_pair(to_float(kr[2 * i]), to_float(kr[2 * i + 1]), (float)pos, inv_freq[i], a, b);
-        dst[rank + 2 * i] = from_float<T>(a);
-        dst[rank + 2 * i + 1] = from_float<T>(b);
-    }
-    for (int i = rot_dims + threadIdx.x; i < rot; i += blockDim.x) dst[rank + i] = kr[i];
+    for (int i = threadIdx.x; i < steps; i += blockDim.x) turn_part(kr, dst + rank)(i);
 }
 
 extern "C" int tl_latent_prepare(const void* down, int ld, int q_rank, int kv_off, int rank, int rot, int rot_dims, const void* wq, int wq_f32,
                                  const void* wkv, int wkv_f32, float eps, const void* positions, const void* inv_freq,
                                  const void* token_req, const void* block_table, int bt_stride, void* plane, int page_size,
-                                 void* cq, int tokens, int dtype, hipStream_t stream) {
+                                 void* cq, int halves, void* rows, int rows_ld, int q_heads, int q_head, int q_plain, int tokens, int dtype,
+                                 hipStream_t stream) {
     TL_REQUIRE(tokens >= 0 && q_rank >= 0 && kv_off >= q_rank && rank > 0 && rot >= 0 && rot_dims % 2 == 0 && rot_dims <= rot && ld >= kv_off + rank + rot,
                "latent_prepare: bad sizes");
+    TL_REQUIRE(rot_dims / 2 <= LAT_MAX_PAIRS && (rot_dims == 0 || (positions && inv_freq)), "latent_prepare: up to %d rotated pairs, got %d", LAT_MAX_PAIRS, rot_dims / 2);
+    TL_REQUIRE(!rows || (q_heads > 0 && q_plain >= 0 && q_head >= q_plain + rot && ld >= (q_heads - 1) * q_head + q_plain + rot && rows_ld >= q_heads * (rank + rot)),
+               "latent_prepare: the queries' rotated parts do not fit");
     TL_REQUIRE(q_rank == 0 || (wq && cq), "latent_prepare: a query latent needs its norm's weight and a place to go");
     TL_REQUIRE(plane == nullptr || (page_size > 0 && block_table != nullptr && token_req != nullptr), "latent_prepare: a cache write needs the block table");
     if (tokens == 0) return TL_OK;
     dim3 grid(tokens), block(256);
 #define TL_ARGS(T) (const T*)down, ld, q_rank, kv_off, rank, rot, rot_dims, wq, wq_f32, wkv, wkv_f32, eps, (const int*)positions, (const float*)inv_freq, \
-                   (const int*)token_req, (const int*)block_table, bt_stride, (T*)plane, page_size, (T*)cq
+                   (const int*)token_req, (const int*)block_table, bt_stride, (T*)plane, page_size, (T*)cq, halves, (T*)rows, QueryParts{q_heads, q_head, q_plain, rows_ld}
     if (dtype == TL_DT_F32) latent_prepare_kernel<float><<<grid, block, 0, stream>>>(TL_ARGS(float));
     else if (dtype == TL_DT_BF16) latent_prepare_kernel<bf16_t><<<grid, block, 0, stream>>>(TL_ARGS(bf16_t));
     else TL_REQUIRE(false, "latent_prepare: unknown dtype %d", dtype);
@@ -83,12 +112,13 @@ extern "C" int tl_latent_prepare(const void* down, int ld, int q_rank, int kv_of
 }
 
 // ------------------------------------------------------------------ rotated query parts into place
-// dst[t, h, dst_off + i] = the entries src[t, h, src_off + i], i < rot, the first rot_dims of them turned in pairs.
+// dst[t, h, dst_off + i] = the entries src[t, h, src_off + i], i < rot, the first rot_dims of them turned in pairs: 2j with 2j + 1, or,
+// `halves`, j with j + rot_dims / 2.
 template <typename T>
 __global__ void rotate_pairs_kernel(const T* src, int src_ld, int src_head, int src_off,       // (src may be dst: a thread reads its
                                     T* dst, int dst_ld, int dst_head, int dst_off,               // pair before it writes it)
                                     const int* __restrict__ positions, const float* __restrict__ inv_freq,
-                                    int heads, int rot, int rot_dims) {
+                                    int heads, int rot, int rot_dims, int halves) {
     const int t = blockIdx.x;
     const float pos = (float)positions[t];
     const int half = rot_dims / 2, tail = rot - rot_dims;
@@ -97,10 +127,11 @@ __global__ void rotate_pairs_kernel(const T* src, int src_ld, int src_head, int 
         const T* s = src + (size_t)t * src_ld + h * src_head + src_off;
         T* d = dst + (size_t)t * dst_ld + h * dst_head + dst_off;
         if (j < half) {
+            const int ia = halves ? j : 2 * j, ib = halves ? j + half : 2 * j + 1;
             float a, b;
-            turn_pair(to_float(s[2 * j]), to_float(s[2 * j + 1]), pos, inv_freq[j], a, b);
-            d[2 * j] = from_float<T>(a);
-            d[2 * j + 1] = from_float<T>(b);
+            turn_pair(to_float(s[ia]), to_float(s[ib]), pos, inv_freq[j], a, b);
+            d[ia] = from_float<T>(a);
+            d[ib] = from_float<T>(b);
         } else {
             d[rot_dims + j - half] = s[rot_dims + j - half];
         }
@@ -108,17 +139,17 @@ __global__ void rotate_pairs_kernel(const T* src, int src_ld, int src_head, int 
 }
 
 extern "C" int tl_rotate_pairs(const void* src, int src_ld, int src_head, int src_off, void* dst, int dst_ld, int dst_head, int dst_off,
-                               const void* positions, const void* inv_freq, int tokens, int heads, int rot, int rot_dims, int dtype,
+                               const void* positions, const void* inv_freq, int tokens, int heads, int rot, int rot_dims, int halves, int dtype,
                                hipStream_t stream) {
     TL_REQUIRE(tokens >= 0 && heads > 0 && rot >= 0 && rot_dims % 2 == 0 && rot_dims <= rot, "rotate_pairs: bad sizes");
     if (tokens == 0 || rot == 0) return TL_OK;
     dim3 grid(tokens), block(256);
     if (dtype == TL_DT_F32)
         rotate_pairs_kernel<float><<<grid, block, 0, stream>>>((const float*)src, src_ld, src_head, src_off, (float*)dst, dst_ld, dst_head, dst_off,
-                                                               (const int*)positions, (const float*)inv_freq, heads, rot, rot_dims);
+                                                               (const int*)positions, (const float*)inv_freq, heads, rot, rot_dims, halves);
     else if (dtype == TL_DT_BF16)
         rotate_pairs_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)src, src_ld, src_head, src_off, (bf16_t*)dst, dst_ld, dst_head, dst_off,
-                                                                (const int*)positions, (const float*)inv_freq, heads, rot, rot_dims);
+                                                                (const int*)positions, (const float*)inv_freq, heads, rot, rot_dims, halves);
     else TL_REQUIRE(false, "rotate_pairs: unknown dtype %d", dtype);
     TL_CHECK_LAUNCH("rotate_pairs");
     return TL_OK;
@@ -334,8 +365,8 @@ latent_attention_mfma_kernel(const bf16_t* __restrict__ q, int q_ld, bf16_t* __r
 #pragma unroll
     for (int c = 0; c < LM_DC_MAX; ++c)
         qf[c].u = (c < dc && row_ok) ? *(const uint4*)(q + (size_t)tok * q_ld + (size_t)rh * D + 32 * c + 8 * g) : make_uint4(0, 0, 0, 0);
-    const int nt = rank / 16 / WPR;                  // blocks of 16 latent columns of this wave: t0 .. t0 + nt - 1
-    const int t0 = share * nt;
+    // blocks of 16 latent columns of this wave: t0 .. t0 + nt - 1 (the last wave of a block of rows may have fewer than the others, or none)
+    const int t_each = (rank / 16 + WPR - 1) / WPR, t0 = share * t_each, nt = min(t_each, rank / 16 - t0);
     lm_f32x4 acc[NT];
 #pragma unroll
     for (int t = 0; t < NT; ++t) acc[t] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
@@ -513,10 +544,10 @@ latent_attention_mfma_kernel(const bf16_t* __restrict__ q, int q_ld, bf16_t* __r
 static size_t lm_smem_bytes(int rank, int rot) { return sizeof(bf16_t) * ((size_t)LM_KEYS * (rank + rot + 8) + (size_t)rank * (LM_KEYS + 4)) + sizeof(int) * LM_BT_MAX; }
 
 // Whether the matrix-core kernel is built for these sizes: rows of a multiple of 32 numbers up to 640, latents of a
-// multiple of 64 numbers up to 512, 16-byte aligned query rows.
+// multiple of 16 numbers up to 512, 16-byte aligned query rows.
 static bool lm_fits(int rank, int rot, int q_ld, const void* q, const void* plane, int bt_stride) {
     const int D = rank + rot;
-    return bt_stride <= LM_BT_MAX && D % 32 == 0 && D <= 32 * LM_DC_MAX && rank % 64 == 0 && rank <= 512 && q_ld % 8 == 0 &&
+    return bt_stride <= LM_BT_MAX && D % 32 == 0 && D <= 32 * LM_DC_MAX && rank % 16 == 0 && rank <= 512 && q_ld % 8 == 0 &&
            ((uintptr_t)q % 16) == 0 && ((uintptr_t)plane % 16) == 0 && lm_smem_bytes(rank, rot) <= 160 * 1024;
 }
 
@@ -545,7 +576,7 @@ static int launch_lm(const void* q, int q_ld, void* out, const void* plane, cons
 
 extern "C" int tl_latent_attention_mfma_fits(int rank, int rot, int q_ld) {
     const int D = rank + rot;
-    return (D % 32 == 0 && D <= 32 * LM_DC_MAX && rank % 64 == 0 && rank <= 512 && q_ld % 8 == 0 && lm_smem_bytes(rank, rot) <= 160 * 1024) ? 1 : 0;
+    return (D % 32 == 0 && D <= 32 * LM_DC_MAX && rank % 16 == 0 && rank <= 512 && q_ld % 8 == 0 && lm_smem_bytes(rank, rot) <= 160 * 1024) ? 1 : 0;
 }
 
 // q [tokens, q_ld]: per head rank + rot numbers (head h at column h * (rank + rot)); out [tokens, heads * rank];

@@ -10,6 +10,7 @@
 // and value are the means of the cached keys and values of the positions b * pool .. b * pool + pool - 1 and lie, as a token's would, in
 // row b of planes of their own with a block table of their own (pool_blocks_kernel makes them when a step brings a block's last token).
 // A third one: values that lie in the cache turned by their own positions; a head's output at position p is turned back by p.
+// A fourth one: a gate per head; a token's output of head h is multiplied by sigmoid(gate[token, h]).
 #include "common.h"
 
 // ------------------------------------------------------------------ cache write
@@ -99,7 +100,7 @@ local_attention_kernel(const T* __restrict__ q, int q_ld, T* __restrict__ out, i
                        const T* __restrict__ v_plane, const int* __restrict__ block_table, int table_ld, const int* __restrict__ token_req,
                        const int* __restrict__ positions, int heads, int kv_heads, int dim, int vdim, int page_size, float scale, float cap,
                        LocalMask mask, float gain, const float* __restrict__ sink, const T* __restrict__ pk_plane, const T* __restrict__ pv_plane,
-                       const int* __restrict__ pool_table, int pool_table_ld, int pool, OutputTurn back) {
+                       const int* __restrict__ pool_table, int pool_table_ld, int pool, OutputTurn back, const T* __restrict__ gate, int gate_ld) {
     __shared__ float sq[LA_MAX_DIM];
     __shared__ float sm[LA_WAVES], sl[LA_WAVES];
     __shared__ float sacc[LA_WAVES][LA_MAX_DIM];
@@ -171,7 +172,8 @@ local_attention_kernel(const T* __restrict__ q, int q_ld, T* __restrict__ out, i
             den = fmaf(sl[w], f[w], den);
         }
         if (sink) den += expf(sink[head] - top);
-        const float norm = gain / den;
+        float norm = gain / den;
+        if (gate) norm *= sigmoid(to_float(gate[(size_t)t * gate_ld + head]));
         auto joined = [&](int col) {
             float o = 0.f;
             for (int w = 0; w < LA_WAVES; ++w) o = fmaf(sacc[w][col], f[w], o);
@@ -236,7 +238,7 @@ local_attention_mfma_kernel(const bf16_t* __restrict__ q, int q_ld, bf16_t* __re
                             const int* __restrict__ tile_tok0, int heads, int kv_heads, int page_size, float scale, float cap,
                             LocalMask mask, float gain, const float* __restrict__ sink, const bf16_t* __restrict__ pk_plane,
                             const bf16_t* __restrict__ pv_plane, const int* __restrict__ pool_table, int pool_table_ld, int pool_table_width, int pool,
-                            OutputTurn back) {
+                            OutputTurn back, const bf16_t* __restrict__ gate, int gate_ld) {
     constexpr int dim = DK * 32, vdim = DV * 16;
     extern __shared__ float la_smem[];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, li = lane & 15, kq = lane >> 4;
@@ -402,8 +404,10 @@ local_attention_mfma_kernel(const bf16_t* __restrict__ q, int q_ld, bf16_t* __re
             u = fmaf(o[ca], f, u);
             if (cb >= 0) v = fmaf(o[cb], f, v);
         }
-        u *= gain / den;
-        v *= gain / den;
+        float norm = gain / den;
+        if (gate) norm *= sigmoid(to_float(gate[(size_t)(first + tok0 + tok) * gate_ld + head]));
+        u *= norm;
+        v *= norm;
     };
     bf16_t* const orow0 = out + (size_t)(first + tok0) * out_ld + head * vdim;
     if (back.freq) {
@@ -431,7 +435,7 @@ static void launch_local_mfma(const void* q, int q_ld, void* out, int out_ld, co
                               int table_ld, int table_width, const void* req_indptr, const void* ctx_lens, const void* tile_req,
                               const void* tile_tok0, int tiles, int heads, int kv_heads, int page_size, float scale, float cap, LocalMask mask,
                               float gain, const void* sink, const void* pk_plane, const void* pv_plane, const void* pool_table, int pool_table_ld,
-                              int pool_table_width, int pool, OutputTurn back, hipStream_t stream) {
+                              int pool_table_width, int pool, OutputTurn back, const void* gate, int gate_ld, hipStream_t stream) {
     dim3 grid(tiles, heads), block(LAM_WAVES * TL_WAVE);
     const size_t smem = sizeof(float) * LAM_WAVES * LAM_TOKENS * (2 + DV * 16);
     auto kernel = local_attention_mfma_kernel<DK, DV>;
@@ -443,13 +447,13 @@ static void launch_local_mfma(const void* q, int q_ld, void* out, int out_ld, co
     kernel<<<grid, block, smem, stream>>>((const bf16_t*)q, q_ld, (bf16_t*)out, out_ld, (const bf16_t*)k_plane, (const bf16_t*)v_plane,
         (const int*)block_table, table_ld, table_width, (const int*)req_indptr, (const int*)ctx_lens, (const int*)tile_req, (const int*)tile_tok0,
         heads, kv_heads, page_size, scale, cap, mask, gain, (const float*)sink, (const bf16_t*)pk_plane, (const bf16_t*)pv_plane, (const int*)pool_table,
-        pool_table_ld, pool_table_width, pool, back);
+        pool_table_ld, pool_table_width, pool, back, (const bf16_t*)gate, gate_ld);
 }
 
 // Whether the matrix-core kernel is built for these sizes.
 extern "C" int tl_local_attention_mfma_fits(int dim, int vdim, int page_size) {
     const bool dk = dim == 32 || dim == 64 || dim == 96 || dim == 128 || dim == 192 || dim == 256;
-    const bool dv = vdim == 16 || vdim == 32 || vdim == 64 || vdim == 96 || vdim == 128 || vdim == 192 || vdim == 256;
+    const bool dv = vdim > 0 && vdim % 16 == 0 && (vdim <= 128 || vdim == 160 || vdim == 192 || vdim == 256);
     return dk && dv && page_size % 8 == 0;
 }
 
@@ -460,7 +464,9 @@ extern "C" int tl_local_attention_tiles(const void* q, int q_ld, void* out, int 
                                         const void* tile_req, const void* tile_tok0, int tiles, int heads, int kv_heads, int dim, int vdim,
                                         int page_size, float scale, float cap, int chunk, int window, float gain, const void* sink,
                                         const void* pk_plane, const void* pv_plane, const void* pool_table, int pool_table_ld, int pool_table_width,
-                                        int pool, int keep_first, const void* turn_freq, int turn_dims, int turn_halves, hipStream_t stream) {
+                                        int pool, int keep_first, const void* turn_freq, int turn_dims, int turn_halves, const void* gate, int gate_ld,
+                                        hipStream_t stream) {
+    TL_REQUIRE(!gate || gate_ld >= heads, "local_attention_tiles: a gate has a number per head");
     TL_REQUIRE(!turn_freq || (turn_dims > 0 && turn_dims % 2 == 0 && turn_dims <= vdim && vdim % 2 == 0), "local_attention_tiles: an output of %d columns turned over %d", vdim, turn_dims);
     TL_REQUIRE(keep_first >= 0 && (keep_first == 0 || (window > 0 && chunk == 0)), "local_attention_tiles: kept first tokens stand beside a window, without chunks");
     TL_REQUIRE(pool >= 0 && (pool == 0 || (window > 0 && pk_plane && pv_plane && pool_table && pool_table_ld >= pool_table_width && pool_table_width > 0)),
@@ -475,14 +481,18 @@ extern "C" int tl_local_attention_tiles(const void* q, int q_ld, void* out, int 
 #define TL_LAM(DK, DV)                                                                                                                      \
     launch_local_mfma<DK, DV>(q, q_ld, out, out_ld, k_plane, v_plane, block_table, table_ld, table_width, req_indptr, ctx_lens, tile_req,  \
                               tile_tok0, tiles, heads, kv_heads, page_size, scale, cap, mask, gain, sink, pk_plane, pv_plane, pool_table,        \
-                              pool_table_ld, pool_table_width, pool, back, stream)
+                              pool_table_ld, pool_table_width, pool, back, gate, gate_ld, stream)
 #define TL_LAM_V(DK)                                     \
     switch (vdim) {                                      \
         case 16: TL_LAM(DK, 1); break;                   \
         case 32: TL_LAM(DK, 2); break;                   \
+        case 48: TL_LAM(DK, 3); break;                   \
         case 64: TL_LAM(DK, 4); break;                   \
+        case 80: TL_LAM(DK, 5); break;                   \
         case 96: TL_LAM(DK, 6); break;                   \
+        case 112: TL_LAM(DK, 7); break;                  \
         case 128: TL_LAM(DK, 8); break;                  \
+        case 160: TL_LAM(DK, 10); break;                 \
         case 192: TL_LAM(DK, 12); break;                 \
         default: TL_LAM(DK, 16); break;                  \
     }
@@ -504,8 +514,9 @@ extern "C" int tl_local_attention(const void* q, int q_ld, void* out, int out_ld
                                   const void* block_table, int table_ld, int table_width, const void* token_req, const void* positions,
                                   int tokens, int heads, int kv_heads, int dim, int vdim, int page_size, float scale, float cap, int chunk,
                                   int window, float gain, const void* sink, const void* pk_plane, const void* pv_plane, const void* pool_table,
-                                  int pool_table_ld, int pool, int keep_first, const void* turn_freq, int turn_dims, int turn_halves, int dtype,
-                                  hipStream_t stream) {
+                                  int pool_table_ld, int pool, int keep_first, const void* turn_freq, int turn_dims, int turn_halves, const void* gate,
+                                  int gate_ld, int dtype, hipStream_t stream) {
+    TL_REQUIRE(!gate || gate_ld >= heads, "local_attention: a gate has a number per head");
     TL_REQUIRE(!turn_freq || (turn_dims > 0 && turn_dims % 2 == 0 && turn_dims <= vdim && vdim % 2 == 0), "local_attention: an output of %d columns turned over %d", vdim, turn_dims);
     TL_REQUIRE(keep_first >= 0 && (keep_first == 0 || (window > 0 && chunk == 0)), "local_attention: kept first tokens stand beside a window, without chunks");
     TL_REQUIRE(pool >= 0 && (pool == 0 || (window > 0 && pk_plane && pv_plane && pool_table)), "local_attention: pooled blocks need a window, their planes and their block table");
@@ -520,11 +531,13 @@ extern "C" int tl_local_attention(const void* q, int q_ld, void* out, int out_ld
     if (dtype == TL_DT_F32)
         local_attention_kernel<float><<<grid, block, 0, stream>>>((const float*)q, q_ld, (float*)out, out_ld, (const float*)k_plane, (const float*)v_plane,
             (const int*)block_table, table_ld, (const int*)token_req, (const int*)positions, heads, kv_heads, dim, vdim, page_size, scale, cap, mask, gain,
-            (const float*)sink, (const float*)pk_plane, (const float*)pv_plane, (const int*)pool_table, pool_table_ld, pool, back);
+            (const float*)sink, (const float*)pk_plane, (const float*)pv_plane, (const int*)pool_table, pool_table_ld, pool, back,
+            (const float*)gate, gate_ld);
     else if (dtype == TL_DT_BF16)
         local_attention_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)q, q_ld, (bf16_t*)out, out_ld, (const bf16_t*)k_plane, (const bf16_t*)v_plane,
             (const int*)block_table, table_ld, (const int*)token_req, (const int*)positions, heads, kv_heads, dim, vdim, page_size, scale, cap, mask, gain,
-            (const float*)sink, (const bf16_t*)pk_plane, (const bf16_t*)pv_plane, (const int*)pool_table, pool_table_ld, pool, back);
+            (const float*)sink, (const bf16_t*)pk_plane, (const bf16_t*)pv_plane, (const int*)pool_table, pool_table_ld, pool, back,
+            (const bf16_t*)gate, gate_ld);
     else TL_REQUIRE(false, "local_attention: unknown dtype %d", dtype);
     TL_CHECK_LAUNCH("local_attention");
     return TL_OK;
@@ -598,6 +611,8 @@ extern "C" int tl_pool_blocks(const void* k_plane, const void* v_plane, int page
 // ------------------------------------------------------------------ norm per head and rotation, in place
 // x [T, ld] holds per token heads_a + heads_b heads of `dim` numbers side by side (queries, then keys).  One wave per token and head, in float:
 //   norm (norm_a / norm_b != null): v <- v / sqrt(mean(v^2) + eps) * w[d], w = norm_a for the first heads_a heads, norm_b for the others;
+//   without weights (`unit`): v <- v / sqrt(mean(v^2) + eps) for the heads of both kinds;
+//   a temperature (`heat`) of the first heads_a heads (the queries): v <- v * (1 + coef * ln(floor((position + 1) / every) + 1));
 //   rotation (inv_freq != null) of the first `dims` numbers by angle_i = float(position) * inv_freq[i]: pair (2i, 2i + 1), or, `halves`,
 //   pair (i, i + dims / 2); (u, v) <- (u cos - v sin, v cos + u sin).  What lies beyond `dims` is not turned.  One rounding at the end.
 // `raw_b` (optional, [T, raw_ld]): the heads_b heads as they come, before norm and rotation, are copied there (values that are the keys
@@ -608,6 +623,10 @@ struct ValueHeads {
     int heads, vdim, unit;
     const float* inv_freq;
     int dims, halves;
+};
+struct QueryHeat {
+    float coef;
+    int every;                       // 0: none
 };
 template <typename T>
 struct PagesOf {
@@ -621,7 +640,7 @@ template <typename T>
 __global__ void __launch_bounds__(HNR_WAVES * TL_WAVE)
 head_norm_rotate_kernel(T* __restrict__ x, int ld, int tokens, int heads_a, int heads_b, int dim, const float* __restrict__ norm_a,
                         const float* __restrict__ norm_b, float eps, const int* __restrict__ positions, const float* __restrict__ inv_freq,
-                        int dims, int halves, T* __restrict__ raw_b, int raw_ld, float magnitude, ValueHeads values, PagesOf<T> to) {
+                        int dims, int halves, T* __restrict__ raw_b, int raw_ld, float magnitude, int unit, QueryHeat heat, ValueHeads values, PagesOf<T> to) {
     __shared__ float sv[HNR_WAVES][LA_MAX_DIM];
     const int wave = threadIdx.x / TL_WAVE, lane = threadIdx.x % TL_WAVE;
     const int heads_ab = heads_a + heads_b, heads = heads_ab + values.heads, keys_dim = dim;
@@ -632,7 +651,7 @@ head_norm_rotate_kernel(T* __restrict__ x, int ld, int tokens, int heads_a, int 
     T* row = x + (size_t)t * ld + (is_value ? (size_t)heads_ab * dim + (size_t)(h - heads_ab) * values.vdim : (size_t)h * dim);
     float* v = sv[wave];
     const float* w = is_value ? nullptr : (h < heads_a ? norm_a : norm_b);
-    const bool normed = is_value ? values.unit != 0 : w != nullptr;
+    const bool normed = is_value ? values.unit != 0 : (unit || w != nullptr);
     if (is_value) { dim = values.vdim; inv_freq = values.inv_freq; dims = values.dims; halves = values.halves; magnitude = 1.f; }
     float ss = 0.f;
     if (live) {
@@ -648,6 +667,10 @@ head_norm_rotate_kernel(T* __restrict__ x, int ld, int tokens, int heads_a, int 
     if (live && normed) {
         const float inv = 1.f / sqrtf(ss / (float)dim + eps);
         for (int d = lane; d < dim; d += TL_WAVE) v[d] = v[d] * inv * (w ? w[d] : 1.f);
+    }
+    if (live && heat.every > 0 && h < heads_a) {         // (a lane goes over the numbers it normed itself)
+        const float f = 1.f + heat.coef * logf((float)((positions[t] + 1) / heat.every + 1));
+        for (int d = lane; d < dim; d += TL_WAVE) v[d] *= f;
     }
     __syncthreads();
     if (live && inv_freq) {
@@ -687,7 +710,10 @@ extern "C" int tl_head_norm_rotate(void* x, int ld, int tokens, int heads_a, int
                                    const void* positions, const void* inv_freq, int dims, int halves, void* raw_b, int raw_ld, float magnitude,
                                    int heads_c, int vdim, int unit_c, const void* inv_freq_c, int dims_c, int halves_c, const void* token_req,
                                    const void* block_table, int table_ld, int table_width, void* k_plane, void* v_plane, int pages, int page_size,
-                                   int dtype, hipStream_t stream) {
+                                   int unit, float heat_coef, int heat_every, int dtype, hipStream_t stream) {
+    TL_REQUIRE(!unit || (!norm_a && !norm_b), "head_norm_rotate: a norm has weights or it has none");
+    TL_REQUIRE(heat_every >= 0 && (heat_every == 0 || positions), "head_norm_rotate: a temperature goes by positions");
+    const QueryHeat heat{heat_coef, heat_every};
     TL_REQUIRE(heads_c >= 0 && (heads_c == 0 || (vdim > 0 && vdim <= LA_MAX_DIM && ld >= (heads_a + heads_b) * dim + heads_c * vdim)), "head_norm_rotate: bad sizes of the values");
     TL_REQUIRE(heads_c == 0 || !inv_freq_c || (positions && dims_c > 0 && dims_c % 2 == 0 && dims_c <= vdim), "head_norm_rotate: a rotation over %d of %d numbers of a value", dims_c, vdim);
     TL_REQUIRE(!k_plane || (v_plane && heads_c == heads_b && heads_c > 0 && positions && token_req && block_table && table_width > 0 && table_ld >= table_width && pages > 0 && page_size > 0),
@@ -703,11 +729,11 @@ extern "C" int tl_head_norm_rotate(void* x, int ld, int tokens, int heads_a, int
     const int grid = (int)((items + HNR_WAVES - 1) / HNR_WAVES);
     if (dtype == TL_DT_F32)
         head_norm_rotate_kernel<float><<<grid, HNR_WAVES * TL_WAVE, 0, stream>>>((float*)x, ld, tokens, heads_a, heads_b, dim, (const float*)norm_a,
-            (const float*)norm_b, eps, (const int*)positions, (const float*)inv_freq, dims, halves, (float*)raw_b, raw_ld, magnitude, values,
+            (const float*)norm_b, eps, (const int*)positions, (const float*)inv_freq, dims, halves, (float*)raw_b, raw_ld, magnitude, unit, heat, values,
             PagesOf<float>{(const int*)token_req, (const int*)block_table, table_ld, table_width, (float*)k_plane, (float*)v_plane, pages, page_size});
     else if (dtype == TL_DT_BF16)
         head_norm_rotate_kernel<bf16_t><<<grid, HNR_WAVES * TL_WAVE, 0, stream>>>((bf16_t*)x, ld, tokens, heads_a, heads_b, dim, (const float*)norm_a,
-            (const float*)norm_b, eps, (const int*)positions, (const float*)inv_freq, dims, halves, (bf16_t*)raw_b, raw_ld, magnitude, values,
+            (const float*)norm_b, eps, (const int*)positions, (const float*)inv_freq, dims, halves, (bf16_t*)raw_b, raw_ld, magnitude, unit, heat, values,
             PagesOf<bf16_t>{(const int*)token_req, (const int*)block_table, table_ld, table_width, (bf16_t*)k_plane, (bf16_t*)v_plane, pages, page_size});
     else TL_REQUIRE(false, "head_norm_rotate: unknown dtype %d", dtype);
     TL_CHECK_LAUNCH("head_norm_rotate");

@@ -25,7 +25,7 @@ _libs: dict[str, ctypes.CDLL] = {}
 
 _DT = {torch.float32: 0, torch.bfloat16: 1}
 
-GATE_ACTIVATIONS = {"silu": 0, "relu": 1}      # the activation of a gated feed-forward's gate
+GATE_ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2}      # the activation of a gated feed-forward's gate
 
 
 def _lib(name: str) -> ctypes.CDLL:
@@ -189,8 +189,8 @@ def bigram_embedding(token_ids: torch.Tensor, table: torch.Tensor, out: torch.Te
 
 def sandwich_norm(residual: torch.Tensor, pending: torch.Tensor | None, post_weight: torch.Tensor | None, post_eps: float,
                   extra: torch.Tensor | None, weight: torch.Tensor | None, eps: float, out: torch.Tensor, rows: torch.Tensor | None = None,
-                  gain: float = 1.0) -> None:
-    """``r = residual (+ extra) + (pending / sqrt(mean(pending^2) + post_eps) * post_weight, or pending as it is without a post_weight)``, written
+                  gain: float = 1.0, branch_gain: float = 1.0) -> None:
+    """``r = residual (+ extra) + branch_gain * (pending / sqrt(mean(pending^2) + post_eps) * post_weight, or pending as it is without a post_weight)``, written
     back to the float32 residual ``[T, H]`` unless ``rows`` selects rows; ``out = r / sqrt(mean(r^2) + eps) * weight * gain`` in its own dtype, or
     (``weight=None``) ``r * gain``, the sum without a norm of its own.
     ``pending``: ``[T, H]`` of ``out``'s dtype or float32 slabs ``[P, T, H]`` that are added up; ``extra``: float32 ``[T, H]``; ``weight`` and
@@ -217,7 +217,7 @@ def sandwich_norm(residual: torch.Tensor, pending: torch.Tensor | None, post_wei
             raise KernelError(f"sandwich_norm: {what} must be float32, one number or {H}")
     lib = _lib("elementwise")
     _check(lib, lib.tl_sandwich_norm(_ptr(residual), _ptr(pending), c_int(parts), c_int(T), _ptr(post_weight if pending is not None else None),
-                                     c_int(post_weight.numel() if post_weight is not None else 0), c_float(post_eps), _ptr(extra), _ptr(weight),
+                                     c_int(post_weight.numel() if post_weight is not None else 0), c_float(post_eps), c_float(branch_gain), _ptr(extra), _ptr(weight),
                                      c_int(weight.numel() if weight is not None else 0), c_float(eps), c_float(gain), _ptr(out), _ptr(rows), c_int(n), c_int(H),
                                      c_int(_dt(out, "sandwich_norm")), _stream()))
 
@@ -494,7 +494,7 @@ def interleave_gate_up(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
 
 def linear_swiglu(x: torch.Tensor, gate_up: torch.Tensor, out: torch.Tensor, activation: str = "silu") -> None:
     """``out = act(x @ gate.T) * (x @ up.T)`` on the matrix cores with the gate applied to the
-    32-bit accumulators (``activation``: ``silu`` or ``relu``); ``gate_up`` from :func:`interleave_gate_up`,
+    32-bit accumulators (``activation``: one of :data:`GATE_ACTIVATIONS`); ``gate_up`` from :func:`interleave_gate_up`,
     bfloat16 only, ``x [M, K]`` with K a multiple of 8."""
     M, K = x.shape
     I = out.shape[1]
@@ -882,7 +882,7 @@ def paged_attention_prompt(q: torch.Tensor, out: torch.Tensor, k_plane: torch.Te
 
 
 def swiglu(gate_up: torch.Tensor, out: torch.Tensor, activation: str = "silu") -> None:
-    """``out[t, i] = act(gate_up[t, i]) * gate_up[t, I + i]``; ``activation``: ``silu`` or ``relu``."""
+    """``out[t, i] = act(gate_up[t, i]) * gate_up[t, I + i]``; ``activation``: one of :data:`GATE_ACTIVATIONS`."""
     T, I2 = gate_up.shape
     if I2 % 2 or out.shape != (T, I2 // 2) or out.dtype != gate_up.dtype or not out.is_contiguous() or not gate_up.is_contiguous():
         raise KernelError("swiglu: shapes or dtypes do not fit")
@@ -1251,14 +1251,14 @@ LOCAL_ATTENTION_TILE_TOKENS = 16      # tokens of a tile of the matrix-core kern
 
 def local_attention_mfma_fits(dtype: torch.dtype, dim: int, vdim: int, page_size: int) -> bool:
     """Whether the matrix-core kernel of :func:`local_attention` is built for these sizes (bfloat16; key sizes 32, 64, 96, 128, 192, 256;
-    value sizes 16, 32, 64, 96, 128, 192, 256; pages of a multiple of 8 tokens)."""
+    value sizes of a multiple of 16 up to 128, 160, 192, 256; pages of a multiple of 8 tokens)."""
     return dtype == torch.bfloat16 and bool(_lib("local_attention").tl_local_attention_mfma_fits(c_int(dim), c_int(vdim), c_int(page_size)))
 
 
 def local_attention(q: torch.Tensor, out: torch.Tensor, k_plane: torch.Tensor, v_plane: torch.Tensor, block_table: torch.Tensor,
                     token_req: torch.Tensor, positions: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int, page_size: int,
                     scale: float, softcap: float = 0.0, chunk: int = 0, window: int = 0, gain: float = 1.0, tiles=None,
-                    sink: torch.Tensor | None = None, pooled=None, keep_first: int = 0, turn_back=None) -> None:
+                    sink: torch.Tensor | None = None, pooled=None, keep_first: int = 0, turn_back=None, gate: torch.Tensor | None = None) -> None:
     """Attention of the step's queries ``q [T, heads * dim]`` over their requests' cached keys and values (which hold the step's own tokens
     already): query head ``i`` reads key/value head ``i // (heads / kv_heads)``; ``score = q . k * scale``, then (``softcap > 0``) ``softcap *
     tanh(score / softcap)``; a query at position ``p`` reads the keys ``j <= p`` with ``j // chunk == p // chunk`` (``chunk > 0``) and ``j > p -
@@ -1270,8 +1270,12 @@ def local_attention(q: torch.Tensor, out: torch.Tensor, k_plane: torch.Tensor, v
     ``p`` also reads the rows ``0 .. (p - window + 1) // pool - 1`` of these planes (laid out like the tokens', with a block table of their own).
     ``keep_first`` (with a window, without chunks): a query also reads the keys at the positions ``0 .. keep_first - 1``, wherever it stands.
     ``turn_back = (inv_freq, dims, halves)``: the first ``dims`` columns of a head's output at position ``p`` turn by ``-float32(p) * inv_freq[m]``
-    (float32 ``[dims / 2]``), pair ``m`` being ``2m`` and ``2m + 1`` or, ``halves``, ``m`` and ``m + dims / 2``."""
+    (float32 ``[dims / 2]``), pair ``m`` being ``2m`` and ``2m + 1`` or, ``halves``, ``m`` and ``m + dims / 2``.  ``gate [T, heads]`` (of ``q``'s dtype, rows may
+    be strided): head ``n``'s output of token ``t`` is multiplied by ``sigmoid(gate[t, n])``."""
     T = q.shape[0]
+    if gate is not None and (gate.dtype != q.dtype or gate.shape != (T, heads) or gate.stride(1) != 1):
+        raise KernelError(f"local_attention: a gate is [T, {heads}] of the queries' dtype")
+    gate_args = (_ptr(gate), c_int(gate.stride(0) if gate is not None else 0))
     if keep_first < 0 or (keep_first and (window <= 0 or chunk)):
         raise KernelError("local_attention: kept first tokens stand beside a window, without chunks")
     _check_local_planes("local_attention", k_plane, v_plane, q.dtype, kv_heads, dim, vdim, page_size)
@@ -1314,14 +1318,14 @@ def local_attention(q: torch.Tensor, out: torch.Tensor, k_plane: torch.Tensor, v
                                                  _ptr(req_indptr), _ptr(ctx_lens), _ptr(tile_req), _ptr(tile_tok0), c_int(n_tiles), c_int(heads),
                                                  c_int(kv_heads), c_int(dim), c_int(vdim), c_int(page_size), c_float(scale), c_float(softcap),
                                                  c_int(chunk), c_int(window), c_float(gain), *pool_args, c_int(pool_table.shape[1] if pool else 0),
-                                                 c_int(pool), c_int(keep_first), *turn_args, _stream()))
+                                                 c_int(pool), c_int(keep_first), *turn_args, *gate_args, _stream()))
         return
     _i32(token_req, "token_req", T)
     _i32(positions, "positions", T)
     _check(lib, lib.tl_local_attention(_ptr(q), c_int(q.stride(0)), _ptr(out), c_int(out.stride(0)), _ptr(k_plane), _ptr(v_plane), c_int(k_plane.shape[0]),
                                        _ptr(block_table), c_int(block_table.stride(0)), c_int(block_table.shape[1]), _ptr(token_req), _ptr(positions),
                                        c_int(T), c_int(heads), c_int(kv_heads), c_int(dim), c_int(vdim), c_int(page_size), c_float(scale),
-                                       c_float(softcap), c_int(chunk), c_int(window), c_float(gain), *pool_args, c_int(pool), c_int(keep_first), *turn_args,
+                                       c_float(softcap), c_int(chunk), c_int(window), c_float(gain), *pool_args, c_int(pool), c_int(keep_first), *turn_args, *gate_args,
                                        c_int(_dt(q, "local_attention")), _stream()))
 
 
@@ -1352,7 +1356,7 @@ def pool_blocks(k_plane: torch.Tensor, v_plane: torch.Tensor, block_table: torch
 
 def head_norm_rotate(x: torch.Tensor, heads_a: int, heads_b: int, dim: int, norm_a: torch.Tensor | None, norm_b: torch.Tensor | None, eps: float,
                      positions: torch.Tensor | None, inv_freq: torch.Tensor | None, dims: int, halves: bool,
-                     raw_b: torch.Tensor | None = None, magnitude: float = 1.0, values=None, pages=None) -> None:
+                     raw_b: torch.Tensor | None = None, magnitude: float = 1.0, values=None, pages=None, unit: bool = False, heat=None) -> None:
     """In place on ``x [T, (heads_a + heads_b) * dim]`` (a row-strided view: queries, then keys), per token and head, in 32-bit with one rounding:
     a root-mean-square norm over the head's ``dim`` numbers with the weight ``norm_a`` (the first ``heads_a`` heads) or ``norm_b`` (float32
     ``[dim]``; ``None``: no norm), then the rotation of the first ``dims`` numbers by ``float32(position) * inv_freq[i]`` (float32 ``[dims / 2]``;
@@ -1361,10 +1365,11 @@ def head_norm_rotate(x: torch.Tensor, heads_a: int, heads_b: int, dim: int, norm
     and sines of these heads.  ``values = (heads_c, vdim, unit, inv_freq, dims, halves)``: behind those heads ``x`` holds ``heads_c`` of ``vdim`` numbers
     that are divided by their root mean square (``unit``; the same ``eps``) and turned likewise (``inv_freq=None``: not).  ``pages = (token_req, block_table,
     k_plane, v_plane, page_size)``: the second heads and the values go to their places in the pages, as :func:`kv_cache_write` puts keys and
-    values there, instead of back to ``x``."""
+    values there, instead of back to ``x``.  ``unit``: the heads' norm has no weights (``norm_a`` and ``norm_b`` are ``None``).  ``heat = (coef, every)``: the
+    first ``heads_a`` heads are multiplied by ``1 + coef * ln(floor((position + 1) / every) + 1)`` after their norm."""
     T = x.shape[0]
     heads = heads_a + heads_b
-    heads_c, vdim, unit, c_freq, c_dims, c_halves = values if values is not None else (0, 0, False, None, 0, False)
+    heads_c, vdim, unit_c, c_freq, c_dims, c_halves = values if values is not None else (0, 0, False, None, 0, False)
     if raw_b is not None and (raw_b.dtype != x.dtype or raw_b.shape != (T, heads_b * dim) or raw_b.stride(1) != 1):
         raise KernelError(f"head_norm_rotate: the copy of the second heads must be [T, {heads_b * dim}] of {x.dtype}")
     if x.dim() != 2 or x.stride(1) != 1 or x.shape[1] != heads * dim + heads_c * vdim or max(dim, vdim) > LOCAL_ATTENTION_MAX_DIM:
@@ -1372,6 +1377,13 @@ def head_norm_rotate(x: torch.Tensor, heads_a: int, heads_b: int, dim: int, norm
     for w in (norm_a, norm_b):
         if w is not None and (w.dtype != torch.float32 or w.shape != (dim,) or not w.is_contiguous()):
             raise KernelError(f"head_norm_rotate: a norm's weight must be contiguous float32 [{dim}]")
+    if unit and (norm_a is not None or norm_b is not None):
+        raise KernelError("head_norm_rotate: a norm has weights or it has none")
+    heat_coef, heat_every = heat if heat is not None else (0.0, 0)
+    if heat is not None:
+        _i32(positions, "positions", T)
+        if positions is None or heat_every < 1:
+            raise KernelError("head_norm_rotate: a temperature goes by positions, in steps of at least one")
     if (norm_a is None) != (norm_b is None) and heads_a and heads_b:
         raise KernelError("head_norm_rotate: a norm for both kinds of heads or for neither")
     if inv_freq is not None:
@@ -1397,13 +1409,13 @@ def head_norm_rotate(x: torch.Tensor, heads_a: int, heads_b: int, dim: int, norm
             raise KernelError("head_norm_rotate: the block table must be int32 [requests, blocks]")
         page_args = (_ptr(token_req), _ptr(block_table), c_int(block_table.stride(0)), c_int(block_table.shape[1]), _ptr(k_plane), _ptr(v_plane),
                      c_int(k_plane.shape[0]), c_int(page_size))
-    used = positions if inv_freq is not None or c_freq is not None or pages is not None else None
+    used = positions if inv_freq is not None or c_freq is not None or pages is not None or heat is not None else None
     lib = _lib("local_attention")
     _check(lib, lib.tl_head_norm_rotate(_ptr(x), c_int(x.stride(0)), c_int(T), c_int(heads_a), c_int(heads_b), c_int(dim), _ptr(norm_a), _ptr(norm_b),
                                         c_float(eps), _ptr(used), _ptr(inv_freq), c_int(dims if inv_freq is not None else 0),
                                         c_int(1 if halves else 0), _ptr(raw_b), c_int(raw_b.stride(0) if raw_b is not None else 0), c_float(magnitude),
-                                        c_int(heads_c), c_int(vdim), c_int(1 if unit else 0), _ptr(c_freq), c_int(c_dims if c_freq is not None else 0),
-                                        c_int(1 if c_halves else 0), *page_args,
+                                        c_int(heads_c), c_int(vdim), c_int(1 if unit_c else 0), _ptr(c_freq), c_int(c_dims if c_freq is not None else 0),
+                                        c_int(1 if c_halves else 0), *page_args, c_int(1 if unit else 0), c_float(heat_coef), c_int(heat_every),
                                         c_int(_dt(x, "head_norm_rotate")), _stream()))
 
 
@@ -1411,6 +1423,7 @@ def head_norm_rotate(x: torch.Tensor, heads_a: int, heads_b: int, dim: int, norm
 
 LATENT_ATTENTION_ROWS = 16       # rows (tokens x heads) a work-group of the latent attention owns
 LATENT_MAX_RANK = 1024
+LATENT_MAX_PAIRS = 512           # rotated pairs of a cache row
 
 
 LATENT_MFMA_ROWS = 64            # rows of a tile of its matrix-core kernel
@@ -1425,25 +1438,33 @@ def latent_tile_tokens(heads: int, rows: int = LATENT_ATTENTION_ROWS) -> int:
 
 def latent_attention_mfma_fits(dtype: torch.dtype, heads: int, rank: int, rot: int) -> bool:
     """Whether :func:`latent_attention` runs these sizes on the matrix cores (bfloat16, cache rows of a multiple of 32 numbers up
-    to 640, latents of a multiple of 64 numbers up to 512); it then takes tiles of up to 64 rows, else of up to 16."""
+    to 640, latents of a multiple of 16 numbers up to 512); it then takes tiles of up to 64 rows, else of up to 16."""
     return dtype == torch.bfloat16 and bool(_lib("latent").tl_latent_attention_mfma_fits(c_int(rank), c_int(rot), c_int(heads * (rank + rot))))
 
 
 def latent_prepare(down: torch.Tensor, q_rank: int, rank: int, rot: int, rot_dims: int, wq: torch.Tensor | None, wkv: torch.Tensor,
                    eps: float, positions: torch.Tensor, inv_freq: torch.Tensor, cq: torch.Tensor | None, token_req: torch.Tensor | None = None,
-                   block_table: torch.Tensor | None = None, plane: torch.Tensor | None = None, page_size: int = 0, kv_off: int | None = None) -> None:
+                   block_table: torch.Tensor | None = None, plane: torch.Tensor | None = None, page_size: int = 0, kv_off: int | None = None,
+                   halves: bool = False, queries=None) -> None:
     """From the fused first projection ``down [T, >= kv_off + rank + rot]``: ``cq = rmsnorm(down[:, :q_rank]) * wq`` (``q_rank`` 0: no query
     latent, ``wq`` and ``cq`` ``None``) and, with a plane ``[pages, 1, page, rank + rot]``, the token's cache row ``[rmsnorm(down[:, kv_off:kv_off +
     rank]) * wkv, the next rot numbers with the first rot_dims of them turned in pairs by the token's position]``.  ``kv_off``: the column
-    where the key/value latent starts (default: right after the query latent)."""
+    where the key/value latent starts (default: right after the query latent).  ``halves``: entry ``i`` of a rotated part is paired with ``i +
+    rot_dims / 2`` instead of ``2i`` with ``2i + 1``.  ``queries = (rows [T, heads * (rank + rot)], heads, head, plain)``: the queries are columns of
+    ``down``, ``head`` numbers each, and the ``rot`` numbers of head ``h`` behind its first ``plain`` go, turned alike, to the last ``rot`` columns
+    of the head's ``rank + rot`` in ``rows``."""
     T = down.shape[0]
     kv_off = q_rank if kv_off is None else kv_off
     if down.stride(1) != 1 or kv_off < q_rank or down.shape[1] < kv_off + rank + rot or (q_rank == 0) != (cq is None) or (q_rank == 0) != (wq is None) \
             or (cq is not None and (cq.shape != (T, q_rank) or cq.dtype != down.dtype or not cq.is_contiguous())):
         raise KernelError("latent_prepare: shapes do not fit")
     _i32(positions, "positions", T)
-    if inv_freq.dtype != torch.float32 or inv_freq.numel() != rot_dims // 2 or rot_dims % 2 or rot_dims > rot:
+    if inv_freq.dtype != torch.float32 or inv_freq.numel() != rot_dims // 2 or rot_dims % 2 or rot_dims > min(rot, 2 * LATENT_MAX_PAIRS):
         raise KernelError("latent_prepare: inv_freq must be float32 [rot_dims / 2]")
+    rows, heads, head, plain = queries if queries is not None else (None, 0, 0, 0)
+    if rows is not None and (rows.dtype != down.dtype or rows.shape != (T, heads * (rank + rot)) or not rows.is_contiguous() or heads < 1 or plain < 0
+                             or head < plain + rot or down.shape[1] < (heads - 1) * head + plain + rot):
+        raise KernelError(f"latent_prepare: the queries' rows must be contiguous [T, {heads * (rank + rot)}] of {down.dtype}, behind heads of {plain} + {rot} numbers")
     bt_stride = 0
     if plane is not None:
         _i32(token_req, "token_req", T)
@@ -1455,13 +1476,14 @@ def latent_prepare(down: torch.Tensor, q_rank: int, rank: int, rot: int, rot_dim
     _check(lib, lib.tl_latent_prepare(_ptr(down), c_int(down.stride(0)), c_int(q_rank), c_int(kv_off), c_int(rank), c_int(rot), c_int(rot_dims),
                                       _ptr(wq), c_int(_vec(wq, q_rank, "query latent norm")), _ptr(wkv), c_int(_vec(wkv, rank, "latent norm")),
                                       c_float(eps), _ptr(positions), _ptr(inv_freq), _ptr(token_req), _ptr(block_table), c_int(bt_stride),
-                                      _ptr(plane), c_int(page_size), _ptr(cq), c_int(T), c_int(_dt(down, "latent_prepare")), _stream()))
+                                      _ptr(plane), c_int(page_size), _ptr(cq), c_int(1 if halves else 0), _ptr(rows), c_int(heads * (rank + rot)), c_int(heads), c_int(head),
+                                      c_int(plain), c_int(T), c_int(_dt(down, "latent_prepare")), _stream()))
 
 
 def rotate_pairs(src: torch.Tensor, src_head: int, src_off: int, dst: torch.Tensor, dst_head: int, dst_off: int,
-                 positions: torch.Tensor, inv_freq: torch.Tensor, heads: int, rot: int) -> None:
+                 positions: torch.Tensor, inv_freq: torch.Tensor, heads: int, rot: int, halves: bool = False) -> None:
     """Per token and head, ``rot`` numbers from ``src[t, h * src_head + src_off:]`` to ``dst[t, h * dst_head + dst_off:]``, the first
-    ``2 * len(inv_freq)`` of them turned in neighbouring pairs by ``position * inv_freq``."""
+    ``2 * len(inv_freq)`` of them turned by ``position * inv_freq`` in neighbouring pairs or, ``halves``, each with the one ``len(inv_freq)`` further on."""
     T = src.shape[0]
     rot_dims = 2 * inv_freq.numel()
     if src.dtype != dst.dtype or src.stride(1) != 1 or dst.stride(1) != 1 or dst.shape[0] != T or rot_dims > rot \
@@ -1473,7 +1495,7 @@ def rotate_pairs(src: torch.Tensor, src_head: int, src_off: int, dst: torch.Tens
     lib = _lib("latent")
     _check(lib, lib.tl_rotate_pairs(_ptr(src), c_int(src.stride(0)), c_int(src_head), c_int(src_off), _ptr(dst), c_int(dst.stride(0)),
                                     c_int(dst_head), c_int(dst_off), _ptr(positions), _ptr(inv_freq), c_int(T), c_int(heads), c_int(rot),
-                                    c_int(rot_dims), c_int(_dt(src, "rotate_pairs")), _stream()))
+                                    c_int(rot_dims), c_int(1 if halves else 0), c_int(_dt(src, "rotate_pairs")), _stream()))
 
 
 def latent_attention(q: torch.Tensor, out: torch.Tensor, plane: torch.Tensor, block_table: torch.Tensor, req_indptr: torch.Tensor | None,
@@ -1533,19 +1555,23 @@ def latent_attention(q: torch.Tensor, out: torch.Tensor, plane: torch.Tensor, bl
 ACTIVATIONS = {"none": 0, "relu2": 1, "silu": 2, "gelu_tanh": 3, "gelu": 4, "relu2_pairs": 17, "silu_pairs": 18, "gelu_tanh_pairs": 19, "gelu_pairs": 20}
 
 
-def heads_linear(x: torch.Tensor, x_head: int, weight: torch.Tensor, out: torch.Tensor, out_head: int, general: bool = False) -> None:
+def heads_linear(x: torch.Tensor, x_head: int, weight: torch.Tensor, out: torch.Tensor, out_head: int, general: bool = False,
+                 gate: torch.Tensor | None = None) -> None:
     """Per head ``h``: ``out[:, h * out_head : h * out_head + N] = x[:, h * x_head : h * x_head + K] @ weight[h].T`` with
     ``weight [heads, N, K]``; ``x`` and ``out`` may be views with longer rows.  bfloat16 with K a multiple of 32 and 16-byte aligned
-    rows runs on the matrix cores (``general=True`` forces the general kernel)."""
+    rows runs on the matrix cores (``general=True`` forces the general kernel).  ``gate`` (``out``'s shape and dtype, rows may be strided): every output
+    number is multiplied by the sigmoid of its gate's before its one rounding."""
     G, N, K = weight.shape
     T = x.shape[0]
+    if gate is not None and (gate.dtype != x.dtype or gate.shape != out.shape or gate.stride(1) != 1):
+        raise KernelError("heads_linear: the gate does not fit the output")
     if x.dtype != weight.dtype or out.dtype != x.dtype or x.stride(1) != 1 or out.stride(1) != 1 or out.shape[0] != T or not weight.is_contiguous() \
             or x.shape[1] < (G - 1) * x_head + K or out.shape[1] < (G - 1) * out_head + N:
         raise KernelError("heads_linear: shapes or dtypes do not fit")
     lib = _lib("experts")
     _check(lib, lib.tl_grouped_gemm(_ptr(x), c_int(x.stride(0)), c_int(x_head), c_void_p(0), _ptr(weight), _ptr(out), c_int(out.stride(0)),
-                                    c_int(out_head), c_void_p(0), c_int(G), c_int(T), c_int(N), c_int(K), c_int(0),
-                                    c_int(_dt(x, "heads_linear")), c_int(1 if general else 0), _stream()))
+                                    c_int(out_head), c_void_p(0), c_int(G), c_int(T), c_int(N), c_int(K), c_int(0), _ptr(gate),
+                                    c_int(gate.stride(0) if gate is not None else 0), c_int(_dt(x, "heads_linear")), c_int(1 if general else 0), _stream()))
 
 
 def experts_linear(x: torch.Tensor, slot_token: torch.Tensor | None, weight: torch.Tensor, offsets: torch.Tensor, out: torch.Tensor,
@@ -1564,7 +1590,7 @@ def experts_linear(x: torch.Tensor, slot_token: torch.Tensor | None, weight: tor
     _i32(slot_token, "slot_token", S)
     lib = _lib("experts")
     _check(lib, lib.tl_grouped_gemm(_ptr(x), c_int(x.stride(0)), c_int(0), _ptr(slot_token), _ptr(weight), _ptr(out), c_int(out.shape[1]), c_int(0),
-                                    _ptr(offsets), c_int(G), c_int(S), c_int(N), c_int(K), c_int(ACTIVATIONS[activation]),
+                                    _ptr(offsets), c_int(G), c_int(S), c_int(N), c_int(K), c_int(ACTIVATIONS[activation]), c_void_p(0), c_int(0),
                                     c_int(_dt(x, "experts_linear")), c_int(1 if general else 0), _stream()))
 
 
@@ -1572,13 +1598,14 @@ ROUTER_SCORES = {"chosen": 0, "all": 1, "sigmoid": 2}
 
 
 def route(logits: torch.Tensor, top: int, scores: str = "chosen", choice_bias: torch.Tensor | None = None, weight_scale: float = 1.0,
-          weight_eps: float = 0.0):
+          weight_eps: float = 0.0, groups: tuple | None = None):
     """The router's choice for every row of float32 ``logits [T, experts]`` and the sort of the (token, choice) pairs by expert.
     ``scores="chosen"``: the ``top`` largest logits are chosen and weighed by the softmax over those alone; ``"all"``: the scores are the
     softmax over all logits, the ``top`` largest of score (+ ``choice_bias [experts]``, float32, which enters the choice only) are chosen
     and weighed by their scores as they are; ``"sigmoid"``: the scores are the logits' sigmoids, the choice goes by score (+ ``choice_bias``)
-    and the weights are the chosen scores divided by their sum plus ``weight_eps``.  All weights are multiplied by ``weight_scale``.  The
-    lower index wins a tie.  Returns ``(weights [T, top] float32, offsets [experts + 1],
+    and the weights are the chosen scores divided by their sum plus ``weight_eps``.  All weights are multiplied by ``weight_scale``.
+    ``groups = (count, keep)``: the experts lie in ``count`` equal groups side by side, a group counts as much as its best expert (by what the
+    choice goes by), and the choice is among the experts of the ``keep`` best groups.  The lower index wins a tie.  Returns ``(weights [T, top] float32, offsets [experts + 1],
     slot_token [T * top], pair_slot [T * top])``, all on the GPU: expert ``e`` owns the slots ``offsets[e] .. offsets[e + 1] - 1``, slot
     ``s`` reads token ``slot_token[s]``, and the output row of token ``t``'s ``j``-th choice is ``pair_slot[t * top + j]``."""
     T, E = logits.shape
@@ -1586,12 +1613,15 @@ def route(logits: torch.Tensor, top: int, scores: str = "chosen", choice_bias: t
         raise KernelError("route: contiguous float32 logits, up to 4096 experts and up to 64 choices")
     if choice_bias is not None and (choice_bias.dtype != torch.float32 or choice_bias.shape != (E,) or not choice_bias.is_contiguous()):
         raise KernelError(f"route: the choice's bias must be contiguous float32 [{E}]")
+    count, keep = groups if groups is not None else (0, 0)
+    if groups is not None and (count < 1 or E % count or not 1 <= keep <= count or top > keep * (E // count)):
+        raise KernelError(f"route: {keep} of {count} groups of {E} experts do not hold {top} choices")
     ints = torch.empty(T * top * 3 + E + 1, dtype=torch.int32, device=logits.device)
     chosen, slot_token, pair_slot, offsets = ints[: T * top], ints[T * top: 2 * T * top], ints[2 * T * top: 3 * T * top], ints[3 * T * top:]
     weights = torch.empty((T, top), dtype=torch.float32, device=logits.device)
     lib = _lib("experts")
     _check(lib, lib.tl_route(_ptr(logits), c_int(T), c_int(E), c_int(top), c_int(ROUTER_SCORES[scores]), _ptr(choice_bias), _ptr(chosen), _ptr(weights),
-                             _ptr(offsets), _ptr(slot_token), _ptr(pair_slot), c_float(weight_scale), c_float(weight_eps), _stream()))
+                             _ptr(offsets), _ptr(slot_token), _ptr(pair_slot), c_float(weight_scale), c_float(weight_eps), c_int(count), c_int(keep), _stream()))
     return weights, offsets, slot_token, pair_slot
 
 

@@ -226,10 +226,10 @@ class Stream:
     Blocks that norm a branch's output before it is added leave that norm on the stream as well: ``post = (weight, eps)`` means that
     ``pending`` enters as ``pending / sqrt(mean(pending^2) + eps) * weight`` (32-bit; ``weight`` one number or ``hidden`` of them).
     ``extra``: a 32-bit ``[T, hidden]`` tensor that the next norm adds to the residual too (an embedding that enters the stream again).
-    Only norms that say ``folds_post_norm`` know the two.  A mixer that says ``reads_stream`` may be handed the stream itself: it reads the
+    ``gain``: a factor with which ``pending`` enters.  Only norms that say ``folds_post_norm`` know the three.  A mixer that says ``reads_stream`` may be handed the stream itself: it reads the
     32-bit residual with what is pending on it and leaves the stream settled (nothing pending)."""
 
-    __slots__ = ("residual", "pending", "normed", "fold", "post", "extra")
+    __slots__ = ("residual", "pending", "normed", "fold", "post", "extra", "gain")
 
     def __init__(self, residual: torch.Tensor, pending: torch.Tensor | None = None):
         self.residual = residual
@@ -238,6 +238,7 @@ class Stream:
         self.fold = None
         self.post = None
         self.extra = None
+        self.gain = 1.0
 
 
 class LazyNorm:

@@ -16,6 +16,8 @@ post2(ffn(norm2(x)))``; the output is left pending with its norm's weight, and t
 
 A fifth one norms the sublayers' outputs only (:class:`OutputNormBlock`): the first sublayer leaves ``z = x + norm1(mixer(x))``, the second ``z +
 norm2(ffn(z))``, and a per-layer token input may be added after them.
+
+A sixth one is the first with a fixed factor on the branches (:class:`ScaledBlock`): ``x <- x + m * mixer(norm1(x))``, ``x <- x + m * ffn(norm2(x))``.
 """
 from __future__ import annotations
 
@@ -59,6 +61,39 @@ class PreNormBlock(Block):
         stream.pending = self.mixer.forward(h, ctx, cache)
         h = (self.ffn_norm.lazy(stream) if getattr(self.ffn, "takes_lazy_norm", False) else None) or self.ffn_norm.forward(stream)
         stream.pending = self.ffn.forward(h, ctx)
+        return stream
+
+
+@BLOCKS.register("scaled_residual")
+class ScaledBlock(Block):
+    """Pre-norm sublayers whose outputs enter the residual times ``branch_gain``: the factor is left on the stream beside the pending output, and
+    the next norm's kernel applies it in 32-bit where it adds the two."""
+    graph_safe = True
+
+    def __init__(self, spec, dtype, device):
+        super().__init__(spec, dtype, device)
+        self.gain = float(spec.branch_gain)
+        self.mixer_norm = NORMS.build(spec.mixer_norm, dtype, device)
+        self.mixer = MIXERS.build(spec.mixer, dtype, device)
+        self.ffn_norm = NORMS.build(spec.ffn_norm, dtype, device) if spec.ffn is not None else None
+        self.ffn = FEED_FORWARDS.build(spec.ffn, dtype, device) if spec.ffn is not None else None
+        self._children = {spec.mixer_norm_name: self.mixer_norm, spec.mixer_name: self.mixer}
+        if self.ffn is not None:
+            self._children.update({spec.ffn_norm_name: self.ffn_norm, spec.ffn_name: self.ffn})
+        for norm in (self.mixer_norm, self.ffn_norm):
+            if norm is not None and not getattr(norm, "folds_post_norm", False):
+                raise ConfigError(f"a block with a factor on its branches needs norms that fold a scaled branch output; {type(norm).__name__} does not")
+
+    parts = PreNormBlock.parts
+    weight_specs = PreNormBlock.weight_specs
+    load_weights = PreNormBlock.load_weights
+
+    def forward(self, stream: Stream, ctx, cache) -> Stream:
+        h = self.mixer_norm.forward(stream)
+        stream.pending, stream.gain = self.mixer.forward(h, ctx, cache), self.gain
+        if self.ffn is not None:
+            h = self.ffn_norm.forward(stream)
+            stream.pending, stream.gain = self.ffn.forward(h, ctx), self.gain
         return stream
 
 

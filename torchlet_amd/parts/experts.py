@@ -12,7 +12,8 @@ The routed layer has other forms as well, each a field of its specification.  Ga
 W_up,e h)``: the rows of gate and up are interleaved into one matrix per expert and the product's epilogue applies the gate to
 each pair of neighbouring columns.  Scores over all experts: ``s = softmax(z)`` over every logit, the ``top`` largest of ``s +
 correction`` are chosen (the correction enters the choice only) and the weights are the chosen ``s`` as they are.  Identity
-experts: the router's last ``identity`` outputs have no tensors; a token that chooses one gets its own input times the weight.
+experts: the router's last ``identity`` outputs have no tensors; a token that chooses one gets its own input times the weight.  Groups: the
+experts lie in equal groups of neighbours, and only the experts of the groups whose best experts score highest can be chosen.
 """
 from __future__ import annotations
 
@@ -78,6 +79,11 @@ class RoutedExperts(FeedForward):
             raise ConfigError(f"a router picks between 1 and all of its experts, not {spec.top} of {self.outputs}")
         if spec.scores not in ops.ROUTER_SCORES:
             raise ConfigError(f"a router's scores are the softmax over the 'chosen' logits or over 'all', or their 'sigmoid', not {spec.scores!r}")
+        self.groups = tuple(int(n) for n in spec.groups) if spec.groups is not None else None
+        if self.groups is not None:
+            count, keep = self.groups
+            if count < 1 or self.outputs % count or not 1 <= keep <= count or spec.top > keep * (self.outputs // count):
+                raise ConfigError(f"a router's {keep} kept of {count} equal groups of {self.outputs} outputs do not hold {spec.top} choices")
         # one more feed-forward that every token passes, added to the weighted sum (any registered kind that returns a whole tensor)
         self.shared = FEED_FORWARDS.build(spec.shared, dtype, device) if spec.shared is not None else None
         self.act = _activation(spec.activation + "_pairs" if spec.gated else spec.activation)
@@ -124,7 +130,7 @@ class RoutedExperts(FeedForward):
         logits = torch.empty((T, self.outputs), dtype=torch.float32, device=h.device)
         ops.linear(h, self.w_router, self.b_router, logits)
         weights, offsets, slot_token, pair_slot = ops.route(logits, self.top, self.spec.scores, self.correction, float(self.spec.weight_scale),
-                                                            float(self.spec.weight_eps))
+                                                            float(self.spec.weight_eps), self.groups)
         z = torch.empty((T * self.top, self.inter), dtype=self.dtype, device=h.device)
         ops.experts_linear(h, slot_token, self.w_up, offsets, z, self.act)
         y = torch.empty((T * self.top, self.hidden), dtype=self.dtype, device=h.device)

@@ -1,5 +1,5 @@
 """Dense SwiGLU feed-forward: ``down(silu(gate(h)) * up(h))``, no biases
-(/root/reference/src/torchlet/v10_triton_paged_gqa/layer/ffn_swiglu.py:22-59).  The gate's activation (``silu`` or ``relu``) and the
+(/root/reference/src/torchlet/v10_triton_paged_gqa/layer/ffn_swiglu.py:22-59).  The gate's activation (``silu``, ``relu`` or ``gelu_tanh``) and the
 three matrices' names come from the specification.
 
 ``gate_proj`` and ``up_proj`` are put into one matrix at load time so that one matrix

@@ -9,7 +9,9 @@ softmax's denominator also holds ``exp(sink_head)`` (a term without key or value
 Each of these is a field of the specification: without a query latent (``q_rank`` 0) the queries are ``W_q h``; without a rotated part
 (``rot_dim`` 0) a score is ``q . k`` alone; with a window a query reads its last ``window`` keys, itself included, and pages that lie wholly
 behind the window go back to the pool; with a gate head ``n``'s output is multiplied by ``sigmoid(W_g h)[n]`` (inside the attention kernel,
-where the sums are divided by the softmax's denominator).
+where the sums are divided by the softmax's denominator); with ``gate_values`` the heads' values are multiplied number by number by
+``sigmoid(W_g h)`` (in the epilogue of the value up-projection).  The rotation pairs neighbours or halves, as its encoding says; without a query
+latent the kernel that writes the cache row turns the queries' rotated parts as well.
 
 Only ``c`` and the rotated key part are cached: one page plane whose rows hold ``kv_rank + rot_dim`` numbers.  The key
 up-projection is taken to the query's side, ``q_t . (W_uk c_s) = (W_uk^T q_t) . c_s``, so a head's query becomes a vector
@@ -47,7 +49,12 @@ class LatentAttention(Mixer):
             raise ConfigError("latent attention: a rotated part needs a position encoding")
         self.position = POSITION_ENCODINGS.build(spec.position, dtype, device) if spec.position is not None else None
         if self.position is not None and not hasattr(self.position, "inv_freq"):
-            raise ConfigError("latent attention folds a rotation in pairs into its kernels; its position encoding must offer inv_freq")
+            raise ConfigError("latent attention folds a rotation into its kernels; its position encoding must offer inv_freq")
+        if self.position is not None and (not hasattr(self.position, "halves") or self.position.dims > self.rot):
+            raise ConfigError(f"latent attention: the encoding {spec.position.kind!r} is not one over the first dimensions of a rotated part of {self.rot}")
+        self.halves = bool(self.position.halves) if self.position is not None else False
+        if spec.gate and spec.gate_values:
+            raise ConfigError("latent attention: a gate is one number per head or one per value")
         if self.position is not None and getattr(self.position, "magnitude", 1.0) != 1.0:
             raise ConfigError("latent attention folds a plain rotation into its kernels; a magnitude on cosine and sine is not built there")
         # tiles of 64 rows where the matrix-core kernel is built for these sizes, of 16 for the general kernel
@@ -56,10 +63,12 @@ class LatentAttention(Mixer):
         self.general_tile_tokens = ops.latent_tile_tokens(self.heads, ops.LATENT_ATTENTION_ROWS)
         self.compute_units = ops.compute_units()
         self.w_down = self.w_dq_norm = self.w_dkv_norm = self.w_uq = self.w_uk_t = self.w_uv = self.sink = self.w_o = None
-        # the columns of the fused first projection: [query latent, or the queries themselves | latent | rotated key part | gate]
-        self.q_cols = self.q_rank if self.q_rank else self.heads * self.dim
+        # the columns of the fused first projection: [query latent, or the queries themselves | latent | rotated key part | gate], filled up with
+        # zero rows of the matrix so that a token's row stays aligned
+        self.q_cols = self.q_rank if self.q_rank else self.heads * (self.dim + self.rot)
         self.gate_at = self.q_cols + self.row
-        self.down_cols = self.gate_at + (self.heads if spec.gate else 0)
+        self.gate_cols = self.heads if spec.gate else self.heads * self.vdim if spec.gate_values else 0
+        self.down_cols = -(-(self.gate_at + self.gate_cols) // 8) * 8
 
     def paged_need(self):
         return PagedNeed(num_heads=1, head_dim=self.row, planes=((1, self.row),), window=self.spec.window)
@@ -88,13 +97,14 @@ class LatentAttention(Mixer):
         })
         if self.spec.sink:
             specs["sink"] = WeightSpec((n,), keep=KEEP_FLOAT32)
-        if self.spec.gate:
-            specs["g"] = WeightSpec((n, H))
+        if self.gate_cols:
+            specs["g"] = WeightSpec((self.gate_cols, H))
         return specs
 
     def load_weights(self, tensors):
         n = self.heads
-        first = [tensors["dq"] if self.q_rank else tensors["q"], tensors["dkv"]] + ([tensors["g"]] if self.spec.gate else [])
+        first = [tensors["dq"] if self.q_rank else tensors["q"], tensors["dkv"]] + ([tensors["g"]] if self.gate_cols else [])
+        first.append(torch.zeros((self.down_cols - self.gate_at - self.gate_cols, self.hidden), dtype=first[0].dtype))
         self.w_down = self._place(torch.cat(first, dim=0), KEEP_COMPUTE)    # one product reads h once
         self.w_dkv_norm = self._place(tensors["dkv.norm"], KEEP_STORED)
         if self.q_rank:
@@ -122,21 +132,22 @@ class LatentAttention(Mixer):
         down = torch.empty((T, self.down_cols), dtype=self.dtype, device=dev)
         ops.linear(h, self.w_down, None, down)
         write = (ctx.token_req, table, plane, cache.page_size) if cache.writable else (None, None, None, 0)
+        # the query against a cache row: [W_uk^T q_unrotated, rotated part], head by head
+        qrow = torch.empty((T, n * self.row), dtype=self.dtype, device=dev)
         if self.q_rank:
             cq = torch.empty((T, self.q_rank), dtype=self.dtype, device=dev)
             ops.latent_prepare(down, self.q_rank, self.rank, self.rot, rot_dims, self.w_dq_norm, self.w_dkv_norm, float(self.spec.norm_eps),
-                               ctx.positions, inv_freq, cq, *write)
+                               ctx.positions, inv_freq, cq, *write, halves=self.halves)
             q = torch.empty((T, n * (self.dim + self.rot)), dtype=self.dtype, device=dev)
             ops.linear(cq, self.w_uq, None, q)
+            if self.rot:
+                ops.rotate_pairs(q, self.dim + self.rot, self.dim, qrow, self.row, self.rank, ctx.positions, inv_freq, n, self.rot, self.halves)
         else:                       # the queries are the first columns of the projection
             ops.latent_prepare(down, 0, self.rank, self.rot, rot_dims, None, self.w_dkv_norm, float(self.spec.norm_eps),
-                               ctx.positions, inv_freq, None, *write, kv_off=self.q_cols)
+                               ctx.positions, inv_freq, None, *write, kv_off=self.q_cols, halves=self.halves,
+                               queries=(qrow, n, self.dim + self.rot, self.dim) if self.rot else None)
             q = down[:, : self.q_cols]
-        # the query against a cache row: [W_uk^T q_unrotated, rotated part], head by head
-        qrow = torch.empty((T, n * self.row), dtype=self.dtype, device=dev)
         ops.heads_linear(q, self.dim + self.rot, self.w_uk_t, qrow, self.row)
-        if self.rot:
-            ops.rotate_pairs(q, self.dim + self.rot, self.dim, qrow, self.row, self.rank, ctx.positions, inv_freq, n, self.rot)
         # (sequences whose block table the matrix-core kernel cannot keep in shared memory go to the general kernel and its tiles)
         general = table.shape[1] > ops.LATENT_MFMA_MAX_BLOCKS
         tq = self.general_tile_tokens if general else self.tile_tokens
@@ -149,7 +160,8 @@ class LatentAttention(Mixer):
                              general=general, max_new_tokens=ctx.max_new_tokens, window=self.window,
                              gate=down[:, self.gate_at:] if self.spec.gate else None)
         values = torch.empty((T, n * self.vdim), dtype=self.dtype, device=dev)
-        ops.heads_linear(mixed_latent, self.rank, self.w_uv, values, self.vdim)
+        ops.heads_linear(mixed_latent, self.rank, self.w_uv, values, self.vdim,
+                         gate=down[:, self.gate_at: self.gate_at + self.gate_cols] if self.spec.gate_values else None)
         if self.dtype == torch.bfloat16 and ops.linear_partials_pay(T, self.hidden, n * self.vdim):
             return ops.linear_partials(values, self.w_o)      # few rows against a narrow matrix: the next norm adds the slabs up
         out = torch.empty((T, self.hidden), dtype=self.dtype, device=dev)

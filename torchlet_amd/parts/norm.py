@@ -27,8 +27,8 @@ def _over_streams(kind: str, stream: Stream, weight, bias, eps: float, dtype, ro
 
 
 def _no_post_norm(stream: Stream, kind: str) -> None:
-    if stream.post is not None or stream.extra is not None:
-        raise ValueError(f"a {kind} does not fold a normed branch output or a second addend into the stream; a norm that says folds_post_norm does")
+    if stream.post is not None or stream.extra is not None or stream.gain != 1.0:
+        raise ValueError(f"a {kind} does not fold a normed or scaled branch output or a second addend into the stream; a norm that says folds_post_norm does")
 
 
 def _settle(stream: Stream, dtype: torch.dtype) -> torch.Tensor:
@@ -40,8 +40,9 @@ def _settle(stream: Stream, dtype: torch.dtype) -> torch.Tensor:
         return stream.residual
     out = torch.empty(stream.residual.shape, dtype=dtype, device=stream.residual.device)
     post_w, post_eps = stream.post if stream.post is not None else (None, 0.0)
-    ops.sandwich_norm(stream.residual, stream.pending, post_w, post_eps, stream.extra, None, 0.0, out)
+    ops.sandwich_norm(stream.residual, stream.pending, post_w, post_eps, stream.extra, None, 0.0, out, branch_gain=stream.gain)
     stream.pending = stream.post = stream.extra = None
+    stream.gain = 1.0
     return out
 
 
@@ -120,7 +121,7 @@ class ScalarRMSNorm(Norm):
     """``r / sqrt(mean(r^2) + eps) * g`` with one number ``g`` for all coordinates, in 32-bit.  It folds everything a stream can carry
     into the residual on the way, in the same kernel: the pending branch output, plain or, where the block left a norm on it
     (``stream.post``), divided by its own root mean square and multiplied by that norm's weight first; and a second addend
-    (``stream.extra``)."""
+    (``stream.extra``); a factor on the pending output (``stream.gain``)."""
     graph_safe = True
     folds_post_norm = True
 
@@ -142,9 +143,10 @@ class ScalarRMSNorm(Norm):
         n = stream.residual.shape[0] if rows is None else rows.numel()
         out = torch.empty((n, self.dim), dtype=self.dtype, device=stream.residual.device)
         post_w, post_eps = stream.post if stream.post is not None else (None, 0.0)
-        ops.sandwich_norm(stream.residual, stream.pending, post_w, post_eps, stream.extra, self.weight, self.eps, out, rows, gain)
+        ops.sandwich_norm(stream.residual, stream.pending, post_w, post_eps, stream.extra, self.weight, self.eps, out, rows, gain, stream.gain)
         if rows is None:
             stream.pending = stream.post = stream.extra = None
+            stream.gain = 1.0
         return out
 
     def settle(self, stream: Stream) -> torch.Tensor:
@@ -155,7 +157,7 @@ class ScalarRMSNorm(Norm):
 class OffsetRMSNorm(Norm):
     """``r / sqrt(mean(r^2) + eps) * (offset + w) * gain`` with a weight vector ``w`` stored around zero (``offset`` 1), in 32-bit: the
     offset and the fixed gain are folded into the vector once, at load, in 32-bit.  Like :class:`ScalarRMSNorm` it folds everything a
-    stream can carry (the pending branch output, normed with the weight its block left beside it; a second addend) in the same kernel."""
+    stream can carry (the pending branch output, normed with the weight its block left beside it or times its factor; a second addend) in the same kernel."""
     graph_safe = True
     folds_post_norm = True
 
@@ -178,9 +180,10 @@ class OffsetRMSNorm(Norm):
         n = stream.residual.shape[0] if rows is None else rows.numel()
         out = torch.empty((n, self.dim), dtype=self.dtype, device=stream.residual.device)
         post_w, post_eps = stream.post if stream.post is not None else (None, 0.0)
-        ops.sandwich_norm(stream.residual, stream.pending, post_w, post_eps, stream.extra, self.weight, self.eps, out, rows, gain)
+        ops.sandwich_norm(stream.residual, stream.pending, post_w, post_eps, stream.extra, self.weight, self.eps, out, rows, gain, stream.gain)
         if rows is None:
             stream.pending = stream.post = stream.extra = None
+            stream.gain = 1.0
         return out
 
     def settle(self, stream: Stream) -> torch.Tensor:

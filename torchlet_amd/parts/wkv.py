@@ -90,6 +90,8 @@ class WKV(Mixer):
         """``h``: the stream itself (left settled), or ``[T, hidden]`` in the activation dtype."""
         stream = h if isinstance(h, Stream) else Stream(h.float())
         T, dev = stream.residual.shape[0], stream.residual.device
+        if stream.gain != 1.0:
+            raise ValueError("wkv: a scaled branch output is not folded into the stream by this mixer")
         post_w, post_eps = stream.post if stream.post is not None else (None, 0.0)
         mixes = torch.empty((len(MIXES), T, self.hidden), dtype=self.dtype, device=dev)
         x = ops.settle_shift(stream.residual, stream.pending, post_w, post_eps, cache.state, self.state_floats, ctx.slots, ctx.req_indptr,

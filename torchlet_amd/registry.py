@@ -14,6 +14,7 @@ from .config.fotovik import FotovikConfig
 from .config.migurax import MiguraxConfig
 from .config.nebutar import NebutarConfig
 from .config.qwen2 import Qwen2Config
+from .config.tilalorn import TilalornConfig
 from .config.vabelorn import VabelornConfig
 
 ARCHITECTURES: dict[str, type[ModelConfig]] = {}
@@ -36,6 +37,7 @@ register_architecture(NebutarConfig)
 register_architecture(FotovikConfig)
 register_architecture(BafulornConfig)
 register_architecture(VabelornConfig)
+register_architecture(TilalornConfig)
 
 
 def config_class(name: str) -> type[ModelConfig]:

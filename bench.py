@@ -3,7 +3,7 @@
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch B] [--layers L] [--dtype bfloat16]
                     [--shape 7b|14b|32b] [--context N] [--new-tokens G] [--prefill-tokens T]
-                    [--workload decode|serve|migurax|nebutar|fotovik|bafulorn|vabelorn] [--only decode|step|prefill] [--all]
+                    [--workload decode|serve|migurax|nebutar|fotovik|bafulorn|vabelorn|tilalorn] [--only decode|step|prefill] [--all]
 
 The default run has the layer sizes of Qwen2.5-7B (28 layers, hidden 3584, 28 heads, 4 KV heads, head
 size 128, intermediate 18944, vocabulary 152064) with random weights and goes through the whole engine
@@ -61,6 +61,12 @@ state and decays per token and key channel; grouped-query attention with normed 
 one added to the softmax's denominator; gated dense feed-forwards; a per-layer token input), beside the Fotovik model of the same width and
 layer count (the closest one the framework has: the same attention kernels, recurrences with a matrix state, normed sublayer outputs, dense
 feed-forwards), and the kernels it added or changed beside their like.
+
+``--workload tilalorn [--size s|m]`` does the same for the Tilalorn design (pre-norm layers with a factor on their branches; attention over a cached
+latent in a window with rotated halves and a gate per value; causal grouped-query attention with unit queries and keys, a temperature, capped
+scores, a gate per head and a layer that reads another's keys and values; dense feed-forwards gated by gelu; experts that compete in groups),
+beside the Bafulorn model of the same width and layer count (the closest one the framework has: the same attention kernels and experts), and the
+kernels it added or changed beside their like.
 """
 from __future__ import annotations
 
@@ -103,8 +109,8 @@ def parse_args(argv=None):
     p.add_argument("--context", type=int, default=CONTEXT, help="prompt tokens of each request in the decode runs")
     p.add_argument("--new-tokens", type=int, default=None, help="tokens each request may generate (decode: 256, serve: 128)")
     p.add_argument("--prefill-tokens", type=int, default=2048)
-    p.add_argument("--workload", choices=["decode", "serve", "migurax", "nebutar", "fotovik", "bafulorn", "vabelorn"], default="decode")
-    p.add_argument("--size", choices=["s", "m"], default="s", help="migurax, nebutar, fotovik, bafulorn, vabelorn: layer sizes (s: width 2048, m: width 4096)")
+    p.add_argument("--workload", choices=["decode", "serve", "migurax", "nebutar", "fotovik", "bafulorn", "vabelorn", "tilalorn"], default="decode")
+    p.add_argument("--size", choices=["s", "m"], default="s", help="migurax, nebutar, fotovik, bafulorn, vabelorn, tilalorn: layer sizes (s: width 2048, m: width 4096)")
     p.add_argument("--requests", type=int, default=32)
     p.add_argument("--prompt-min", type=int, default=128)
     p.add_argument("--prompt-max", type=int, default=4096)
@@ -1459,6 +1465,157 @@ def vabelorn(args) -> dict:
     return out
 
 
+# ---------------------------------------------------------------------------------------------- the Tilalorn design
+
+def tilalorn_sizes(size: str) -> dict:
+    """A Tilalorn configuration of four layers at the width of the other designs' sizes: attention over a latent of 512 numbers beside 64 rotated
+    ones, heads of 128 + 64 dimensions in a window of 1024, with experts in four groups and, once more, with a dense feed-forward; causal
+    grouped-query attention with heads of 128 in groups of four, with a dense feed-forward and, on the same keys and values, with experts."""
+    width, heads, ff, experts, eff, top = dict(s=(2048, 16, 5632, 16, 1024, 2), m=(4096, 32, 11264, 32, 2048, 4))[size]
+    latent = dict(heads=heads, dim=128, rot_dim=64, vdim=128, kv_rank=512, scale=192 ** -0.5, rot=dict(dims=64, base=500000.0), mask=dict(size=1024))
+    attention = dict(heads=heads, kv_heads=heads // 4, dim=128, vdim=128, scale=128 ** -0.5, softcap=30.0, q_temp=dict(coef=0.1, every=1024))
+    moe = dict(kind="moe", expert=dict(ff=eff), router=dict(experts=experts, top=top, scale=2.0, groups=dict(count=4, keep=2)))
+    dense = dict(kind="dense", ff=ff)
+    return dict(architecture="Tilalorn", vocab=32000, width=width, max_positions=8192, norm=dict(eps=1e-6), residual_mult=0.25,
+                layers=[dict(type="latent_attention", mixer=latent, mlp=moe), dict(type="attention", mixer=attention, mlp=dense),
+                        dict(type="latent_attention", mixer=latent, mlp=dense), dict(type="attention", mixer=dict(attention, kv_from=1), mlp=moe)])
+
+
+def tilalorn_kernels(ours: dict, like: dict, batch: int, context: int, tokens: int) -> list[dict]:
+    """Each kernel that the design added or changed, alone, at the sizes of ``ours``, in a decode step of ``batch`` requests on ``context`` cached
+    tokens and in a prompt of ``tokens`` tokens, beside the like kernel of the closest path the framework had.  ``frac``: bytes that must
+    move / time against 8 TB/s, or operations / time against the matrix cores' bfloat16 rate."""
+    import torch
+    from torchlet_amd.kernels import ops
+    dev, bf = "cuda", torch.bfloat16
+    rows = []
+
+    def add(name, kind, launch, nbytes=0.0, flops=0.0, peak=MFMA_PEAK_TFLOPS["bfloat16"]):
+        ms = _best_ms(launch, rounds=3, calls=5)
+        row = {"kernel": name, "like": kind, "ms": round(ms, 4)}
+        if nbytes:
+            row.update(bytes=int(nbytes), frac=round(nbytes / (ms * 1e-3) / 1e9 / HBM_PEAK_GBS, 4), bound="hbm")
+        else:
+            row.update(flops=flops, frac=round(flops / (ms * 1e-3) / (peak * 1e12), 4), bound="flops")
+        rows.append(row)
+        say(f"  {name}: {ms:.4f} ms, {row['frac']} of its bound")
+
+    def tables(n_req, total):
+        blocks = -(-total // PAGE)
+        table = (torch.arange(n_req * blocks, dtype=torch.int32, device=dev) + 1).view(n_req, blocks)
+        return table, n_req * blocks + 1
+
+    width = ours["width"]
+    lat, att, moe, ff = ours["layers"][0]["mixer"], ours["layers"][1]["mixer"], ours["layers"][0]["mlp"], ours["layers"][1]["mlp"]["ff"]
+    for kind, T, reqs in (("decode", batch, batch), (f"prompt {tokens}", tokens, 1)):
+        decode, ctx = reqs > 1, context - 1 if reqs > 1 else 0
+        total = ctx + T // reqs
+        tab, pages = tables(reqs, total)
+        indptr, token_req = torch.arange(reqs + 1, dtype=torch.int32, device=dev) * (T // reqs), torch.arange(T, dtype=torch.int32, device=dev) // (T // reqs)
+        positions = (torch.arange(T, dtype=torch.int32, device=dev) % (T // reqs)) + ctx
+        ctx_lens = torch.full((reqs,), ctx, dtype=torch.int32, device=dev)
+
+        def tile_list(size):
+            n = -(-T // size)
+            return torch.zeros(n, dtype=torch.int32, device=dev), torch.arange(n, dtype=torch.int32, device=dev) * size, n
+
+        # ---- attention over the cached latent in a window, rows with a rotated part, beside rows without one and a gate per head (the Bafulorn path)
+        H, rank, window = lat["heads"], lat["kv_rank"], lat["mask"]["size"]
+        seen = lambda p: min(p + 1, window)
+        for label, rot, gated in ((f"window {window}, rotated part", lat["rot_dim"], False), (f"window {window}, gate (Bafulorn path)", 0, True)):
+            D = rank + rot
+            plane = (torch.randn(pages, 1, PAGE, D, device=dev) * 0.3).to(bf)
+            q, o = (torch.randn(T, H * D, device=dev) * 0.1).to(bf), torch.empty(T, H * rank, dtype=bf, device=dev)
+            gate = torch.randn(T, H, device=dev).to(bf) if gated else None
+            tq = ops.latent_tile_tokens(H, ops.LATENT_MFMA_ROWS)
+            tiles = (None, ctx_lens, None, None, reqs) if decode else (indptr, ctx_lens, *tile_list(tq))
+            splits = max(1, min(256 // (reqs * -(-H // 16)), seen(ctx) // 64, 64)) if decode else 1
+            how = dict(nbytes=float(reqs) * seen(ctx) * D * 2) if decode else dict(flops=2.0 * H * (D + rank) * sum(seen(p) for p in range(T)))
+            add(f"latent_attention {kind}, {label}", "" if gated else f"latent_attention {kind}", lambda: ops.latent_attention(
+                q, o, plane, tab, *tiles, tq, H, rank, rot, PAGE, 0.09, None, splits, max_new_tokens=T // reqs, window=window, gate=gate), **how)
+        # ---- the cache row with the queries' rotated parts turned by the same kernel, beside the two kernels of the Migurax path
+        rot, dim, head = lat["rot_dim"], lat["dim"], lat["dim"] + lat["rot_dim"]
+        D = rank + rot
+        plane = torch.zeros(pages, 1, PAGE, D, dtype=bf, device=dev)
+        down, qrow = torch.randn(T, H * head + D, device=dev).to(bf), torch.empty(T, H * D, dtype=bf, device=dev)
+        inv, wn = torch.rand(rot // 2, device=dev), torch.ones(rank, dtype=bf, device=dev)
+        write = dict(token_req=token_req, block_table=tab, plane=plane, page_size=PAGE, kv_off=H * head)
+        nbytes = float(T) * (D * 4 + H * rot * 4)
+        add(f"latent_prepare {kind}, queries too, halves", f"latent_prepare + rotate_pairs {kind}", lambda: ops.latent_prepare(
+            down, 0, rank, rot, rot, None, wn, 1e-6, positions, inv, None, **write, halves=True, queries=(qrow, H, head, dim)), nbytes=nbytes)
+
+        def two_kernels():
+            ops.latent_prepare(down, 0, rank, rot, rot, None, wn, 1e-6, positions, inv, None, **write)
+            ops.rotate_pairs(down, head, dim, qrow, D, rank, positions, inv, H, rot)
+        add(f"latent_prepare + rotate_pairs {kind} (Migurax path)", "", two_kernels, nbytes=nbytes)
+        # ---- the value up-projection with a gate per number in its epilogue, beside it without
+        mixed, w_uv, values = torch.randn(T, H * rank, device=dev).to(bf), (torch.randn(H, lat["vdim"], rank, device=dev) * 0.04).to(bf), torch.empty(T, H * lat["vdim"], dtype=bf, device=dev)
+        gates = torch.randn(T, H * lat["vdim"], device=dev).to(bf)
+        how = dict(nbytes=float(w_uv.numel()) * 2) if decode else dict(flops=2.0 * T * H * rank * lat["vdim"])
+        add(f"heads_linear {kind}, gated", f"heads_linear {kind}", lambda: ops.heads_linear(mixed, rank, w_uv, values, lat["vdim"], gate=gates), **how)
+        add(f"heads_linear {kind} (Bafulorn path)", "", lambda: ops.heads_linear(mixed, rank, w_uv, values, lat["vdim"]), **how)
+        # ---- unit queries and keys, the temperature, keys and values into the pages, beside norms with weights and a rotation (the Vabelorn path)
+        H, G, dk = att["heads"], att["kv_heads"], att["dim"]
+        k_plane, v_plane = (torch.randn(pages, G, PAGE, dk, device=dev) * 0.3).to(bf), (torch.randn(pages, G, dk, PAGE, device=dev) * 0.3).to(bf)
+        qkv = torch.randn(T, (H + 2 * G) * dk, device=dev).to(bf)
+        wq, inv = torch.ones(dk, device=dev), torch.rand(32, device=dev)
+        into = (token_req, tab, k_plane, v_plane, PAGE)
+        nbytes = float(T) * (H + 2 * G) * dk * 4
+        add(f"head_norm_rotate {kind}, unit norm, temperature, into the pages", f"head_norm_rotate {kind}", lambda: ops.head_norm_rotate(
+            qkv, H, G, dk, None, None, 1e-6, positions, None, 0, False, values=(G, dk, False, None, 0, False), pages=into, unit=True, heat=(0.1, 1024)), nbytes=nbytes)
+        add(f"head_norm_rotate {kind}, norm, rotation, into the pages (Vabelorn path)", "", lambda: ops.head_norm_rotate(
+            qkv, H, G, dk, wq, wq, 1e-6, positions, inv, 64, False, values=(G, dk, True, inv, 64, False), pages=into), nbytes=nbytes)
+        # ---- causal attention with capped scores and a gate per head, beside it without the gate (the Nebutar path) and without either
+        q, o = (torch.randn(T, H * dk, device=dev) * 0.3).to(bf), torch.empty(T, H * dk, dtype=bf, device=dev)
+        gate = torch.randn(T, H, device=dev).to(bf)
+        tiles = (indptr, ctx_lens, None, None, reqs) if decode else (indptr, ctx_lens, *tile_list(ops.LOCAL_ATTENTION_TILE_TOKENS))
+        how = dict(nbytes=float(reqs) * (ctx + 1) * G * 2 * dk * 2) if decode else dict(flops=4.0 * H * dk * T * (T + 1) / 2)
+        for label, cap, g_, other in (("capped, gate", att["softcap"], gate, f"local_attention {kind}"), ("capped (Nebutar path)", att["softcap"], None, ""), ("plain (Fotovik path)", 0.0, None, "")):
+            add(f"local_attention {kind}, causal, {label}", other, lambda: ops.local_attention(
+                q, o, k_plane, v_plane, tab, token_req, positions, H, G, dk, dk, PAGE, att["scale"], cap, tiles=tiles, gate=g_), **how)
+        # ---- the gated feed-forward's first product with gelu in its epilogue beside silu
+        gate_up = ops.interleave_gate_up((torch.randn(ff, width, device=dev) * 0.02).to(bf), (torch.randn(ff, width, device=dev) * 0.02).to(bf))
+        x, z = torch.randn(T, width, device=dev).to(bf), torch.empty(T, ff, dtype=bf, device=dev)
+        how = dict(nbytes=2.0 * ff * width * 2) if decode else dict(flops=4.0 * T * ff * width)
+        for act, path in (("gelu_tanh", ""), ("silu", " (Qwen2 path)")):
+            add(f"linear_swiglu {kind}, {act}{path}", "" if path else f"linear_swiglu {kind}", lambda: ops.linear_swiglu(x, gate_up, z, act), **how)
+        # ---- the choice among the experts of the best groups beside the choice among all
+        E, top = moe["router"]["experts"], moe["router"]["top"]
+        logits = torch.randn(T, E, device=dev)
+        nbytes = float(T) * (E * 4 + top * 16)
+        add(f"route {kind}, groups", f"route {kind}", lambda: ops.route(logits, top, "all", None, 2.0, groups=(4, 2)), nbytes=nbytes)
+        add(f"route {kind} (Nebutar path)", "", lambda: ops.route(logits, top, "all", None, 2.0), nbytes=nbytes)
+        # ---- the norm that adds a branch times a factor beside the one that norms the branch first (the Bafulorn path)
+        res, pen, wv, out = torch.randn(T, width, device=dev), torch.randn(T, width, device=dev).to(bf), torch.ones(width, device=dev), torch.empty(T, width, dtype=bf, device=dev)
+        add(f"sandwich_norm {kind}, a factor on the branch", f"sandwich_norm {kind}", lambda: ops.sandwich_norm(res, pen, None, 0.0, None, wv, 1e-6, out, branch_gain=0.25), nbytes=float(T) * width * 12)
+        add(f"sandwich_norm {kind}, normed branch (Bafulorn path)", "", lambda: ops.sandwich_norm(res, pen, wv, 1e-6, None, wv, 1e-6, out), nbytes=float(T) * width * 12)
+    return rows
+
+
+def tilalorn(args) -> dict:
+    import torch
+    ours, like = tilalorn_sizes(args.size), bafulorn_sizes(args.size)
+    out = {"metric": f"Tilalorn design, size {args.size} (width {ours['width']}, 4 layers), prefill of {args.prefill_tokens} tokens and decode at batch "
+                     f"{args.batch} on {args.context}-token caches, beside the Bafulorn design at equal width and layer count, one MI355X",
+           "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
+           "data": "synthetic: seeded random weights, token ids and cache contents", "config": {"tilalorn": ours, "bafulorn": like}}
+    for key, d in (("tilalorn", ours), ("bafulorn", like)):
+        say(f"building the {key} model")
+        cfg, model = _build_from(d, args.dtype)
+        pms, pbest = time_prefill(model, args.prefill_tokens)
+        dms = _decode_ms(model, args.batch, min(args.steps, 64), args.warmup, args.context)
+        out[key] = {"weight_bytes": _weight_bytes(model),
+                    "prefill": {"tokens": args.prefill_tokens, "ms": round(pms, 3), "ms_best": round(pbest, 3), "tokens_per_s": round(args.prefill_tokens * 1e3 / pms, 1)},
+                    "decode": {"batch": args.batch, "context": args.context, "ms_per_step": round(dms, 4), "tokens_per_s": round(args.batch * 1e3 / dms, 1)}}
+        say(f"{key}: {out[key]}")
+        del model
+        torch.cuda.empty_cache()
+    out["value"] = out["tilalorn"]["decode"]["tokens_per_s"]
+    if args.dtype == "bfloat16" and not args.no_points:
+        out["kernels"] = tilalorn_kernels(ours, like, args.batch, args.context, args.prefill_tokens)
+    return out
+
+
 def main(argv=None) -> int:
     args = parse_args(argv)
     args.serve_new_tokens = args.new_tokens or 128
@@ -1484,6 +1641,9 @@ def main(argv=None) -> int:
         return 0
     if args.workload == "vabelorn":
         print(json.dumps(vabelorn(args)))
+        return 0
+    if args.workload == "tilalorn":
+        print(json.dumps(tilalorn(args)))
         return 0
     name, sizes = SHAPES[args.shape]
     full_layers = sizes["num_hidden_layers"]

@@ -156,12 +156,12 @@ class CappedAttention(StagedMixer):
 
     def load_weights(self, tensors):
         first = [tensors[n] for n in ("q" if self.reads_cache else "qk" if self.shared_kv else "qkv")] + ([tensors["g"]] if self.gate_cols else [])
-        first.append(torch.zeros((self.in_width - self.gate_at - self.gate_cols, self.hidden), dtype=first[0].dtype))
+        first.append(first[0].new_zeros((self.in_width - self.gate_at - self.gate_cols, self.hidden)))
         self.w_in = self._place(torch.cat(first, dim=0), KEEP_COMPUTE)
         self.w_o = self._place(tensors["o"], KEEP_COMPUTE)
         if self.spec.qk_bias:
             biases = [tensors[n] for n in ("q.b", "k.b", "v.b") if n in tensors]
-            biases.append(torch.zeros(self.in_width - sum(b.numel() for b in biases), dtype=biases[0].dtype))
+            biases.append(biases[0].new_zeros(self.in_width - sum(b.numel() for b in biases)))
             self.b_in = self._place(torch.cat(biases), KEEP_STORED)
         if self.spec.o_bias:
             self.b_o = self._place(tensors["o.b"], KEEP_STORED)

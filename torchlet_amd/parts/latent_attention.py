@@ -104,7 +104,7 @@ class LatentAttention(Mixer):
     def load_weights(self, tensors):
         n = self.heads
         first = [tensors["dq"] if self.q_rank else tensors["q"], tensors["dkv"]] + ([tensors["g"]] if self.gate_cols else [])
-        first.append(torch.zeros((self.down_cols - self.gate_at - self.gate_cols, self.hidden), dtype=first[0].dtype))
+        first.append(first[0].new_zeros((self.down_cols - self.gate_at - self.gate_cols, self.hidden)))
         self.w_down = self._place(torch.cat(first, dim=0), KEEP_COMPUTE)    # one product reads h once
         self.w_dkv_norm = self._place(tensors["dkv.norm"], KEEP_STORED)
         if self.q_rank:

@@ -158,7 +158,7 @@ def random_config(rnd, big: bool) -> dict:
     for _ in range(rnd.randint(1, 6)):
         if rnd.random() < 0.45:
             kind = "latent_attention"
-            rank, rot = rnd.choice([(64, 32), (80, 16), (112, 16), (256, 64), (96, 32)] if big else [(5, 2), (12, 6), (24, 4)])
+            rank, rot = rnd.choice([(64, 32), (80, 16), (112, 16), (256, 64), (160, 32)] if big else [(5, 2), (12, 6), (24, 4)])
             mixer = _latent(rnd.choice([1, 2, 4, 5]), rnd.choice([32, 64] if big else [4, 6, 10]), rot, rnd.choice([16, 32, 80] if big else [3, 8, 12]),
                             rank, rnd.choice([0.1, 0.25]), rnd.choice([100.0, 10000.0, 1e6]), rnd.choice([None, 1, 3, 7, 16, 33, 50]))
         else:
@@ -166,7 +166,7 @@ def random_config(rnd, big: bool) -> dict:
             sources = [i for i, other in enumerate(layers) if other["type"] == "attention" and "kv_from" not in other["mixer"]]
             source = rnd.choice(sources) if sources and rnd.random() < 0.5 else None
             shape = layers[source]["mixer"] if source is not None else dict(kv_heads=rnd.choice([1, 2, 3]), dim=rnd.choice([32, 64, 96, 128] if big else [4, 6, 10, 24]),
-                                                                              vdim=rnd.choice([16, 48, 64, 80] if big else [3, 8, 12]))
+                                                                              vdim=rnd.choice([16, 48, 64, 112] if big else [3, 8, 12]))
             mixer = _attention(shape["kv_heads"] * rnd.choice([1, 2, 4]), shape["kv_heads"], shape["dim"], shape["vdim"], rnd.choice([0.1, 0.25, shape["dim"] ** -0.5]),
                                rnd.choice([None, 1.5, 20.0]), rnd.choice([None, (0.5, 1), (0.3, 7), (1.0, 64)]), source)
         roll = rnd.random()
